@@ -39,11 +39,31 @@ int qsv_add_normed_rms_norm(float* x, void* h, const void* y, const void* w_post
  * [heads * dim] / [kv_heads * dim]), then turned by the position: pair (2i, 2i + 1), i < rot_n / 2, of every head by rope[pos[t], :,
  * i] (float [positions, 2, rot_n / 2], cos then sin; rope == NULL: no rotation).  q, k, v: rows of type qkv_dtype with their strides.
  *   qf[t, h]         = [ 0 (vdim) | q'[t, h] * scale ]     float [T, heads, vdim + dim]
- *   pool[g, slot[t]] = [ v[t, g] | k'[t, g] ]              [kv_heads, pool_rows, vdim + dim]     (k == NULL: nothing is written) */
+ *   pool[g, slot[t]] = [ v[t, g] | k'[t, g] ]              [kv_heads, pool_rows, vdim + dim]     (k == NULL: nothing is written)
+ * Options (NULL / 0: none): q_b, k_b, v_b (storage type, one per projected channel) are added to the projections before anything else;
+ * halves: pair i = dimensions i and i + rot_n / 2; head_scale (float [heads]) multiplies `scale`; a query row starts with q_pad zeros
+ * (above: q_pad = vdim).  v may be k's own columns (values that are the projected keys). */
 int qsv_qk_norm_rope_prep(float* qf, const void* q, int64_t q_stride, const void* k, int64_t k_stride, const void* v,
                           int64_t v_stride, int qkv_dtype, int heads, int kv_heads, int dim, int vdim, const void* q_w,
                           const void* k_w, int per_head, float eps, const float* rope, int rot_n, float scale, void* pool,
-                          int64_t pool_rows, const int64_t* slot, const int32_t* pos, int n_tokens, int dtype, void* stream);
+                          int64_t pool_rows, const int64_t* slot, const int32_t* pos, int n_tokens, const void* q_b, const void* k_b,
+                          const void* v_b, int halves, const float* head_scale, int q_pad, int dtype, void* stream);
+/* x[t] = rms_norm(table[tokens[t]]) * w    (float) */
+int qsv_embed_rms_norm(float* x, const void* table, const int32_t* tokens, const void* w, float eps, int n_tokens, int width, int dtype,
+                       void* stream);
+/* h[t] = x[t] + sum_j w[j] x[t - (taps - 1) + j]  (w float [taps, width]; the storage type out): inputs before a run's start come from
+ * hist[state_rd[t]] (float [2 * slots, taps - 1, width], oldest first; zeros if state_rd[t] < 0), the run's last token (state_wr[t] >= 0)
+ * writes the new history.  taps == 1: no history. */
+int qsv_residual_conv(void* h, const float* x, const float* w, int taps, float* hist, const int32_t* run_off, const int32_t* state_rd,
+                      const int32_t* state_wr, int n_tokens, int width, int dtype, void* stream);
+/* Norm after the sum: x[t] = rms_norm(alpha x[t] + y[t]) * w, h[t] (may be NULL) = the new x[t] in the storage type.  conv_w != NULL
+ * (only where every run of the step is one token): h[t] = qsv_residual_conv of the new x, its history moved on. */
+int qsv_scaled_add_rms_norm(float* x, void* h, const void* y, float alpha, const void* w, float eps, const float* conv_w, int taps,
+                            float* hist, const int32_t* state_rd, const int32_t* state_wr, int n_tokens, int width, int dtype, void* stream);
+/* out[t] = [ rot(q[t]) | rot(k[t]) | v[t] ] (float) from qkv rows [ q (heads dim) | k (heads dim) | v (heads vdim) .. ]: the first rot_n
+ * dimensions of every q and k head turned by the position, halves layout (rope as above, NULL with rot_n = 0). */
+int qsv_rotate_qk(float* out, const void* qkv, int64_t stride, int heads, int dim, int vdim, const float* rope, int rot_n,
+                  const int32_t* pos, int n_tokens, int dtype, void* stream);
 /* out[r] = rms_norm(x[rows[r]]) * w in the storage type (rows == NULL: row r). */
 int qsv_rms_norm_rows(void* out, const float* x, const int32_t* rows, const void* w, float eps, int n_rows, int width, int dtype,
                       void* stream);
@@ -95,12 +115,13 @@ int qsv_latent_query(float* qf, const void* q, const void* q_abs, const float* r
  *   pooled:     a second set of pools (pooled_stride elements apart, same row layout), block_rows rows per page: the block of
  *               pool_block positions that starts at position s of the sequence has row block_table[s / page] * block_rows +
  *               (s % page) / pool_block (written by qsv_pool_blocks).  A query at position p also sees the rows of the blocks
- *               b < (p - window + 1) / pool_block, those that end before its window starts; no bias with them. */
+ *               b < (p - window + 1) / pool_block, those that end before its window starts; no bias with them;
+ *   slopes:     float [heads]; slopes[h] * (pos[t] - j) is taken off the score (after the query's scale); not with pooled rows. */
 int qsv_latent_attention(void* out, const float* qf, const void* pool, const int32_t* block_table, int table_stride,
                          const int32_t* seq, const int32_t* pos, int window, int n_tokens, int heads, int rank,
                          int row_width, int page, int heads_per_pool, int64_t pool_stride, int chunk, const float* bias,
                          int bias_len, int keep_first, const float* sink, const void* pooled, int64_t pooled_stride, int pool_block,
-                         int block_rows, int dtype, int variant, void* stream);
+                         int block_rows, const float* slopes, int dtype, int variant, void* stream);
 /* pooled[g, row(block)] = mean over the block's positions of pool[g, row(position)], for every token of the step whose position
  * ends a block of pool_block positions ((pos + 1) % pool_block == 0); float sum, one rounding. */
 int qsv_pool_blocks(void* pooled, int64_t pooled_rows, const void* pool, int64_t pool_rows, const int32_t* block_table,
@@ -121,7 +142,30 @@ int qsv_latent_attention_mfma(void* out, const float* qf, const void* pool, cons
                               int row_width, int page, int key_splits, float* part_o, float* part_ml, int n_tokens,
                               int q_first, int heads_per_pool, int64_t pool_stride, int chunk, const float* bias, int bias_len,
                               int keep_first, const float* sink, const void* pooled, int64_t pooled_stride, int pool_block,
-                              int block_rows, void* stream);
+                              int block_rows, const float* slopes, void* stream);
+
+/* ---- talking-heads attention (serve_talking.hip) ------------------------------------------------------------------------------
+ * score(t, h, j) = qf[t, h] . k[kv(h), j], cap > 0: cap tanh(score / cap); w_h = softmax over max(0, pos - window + 1) <= j <= pos (window
+ * 0: all j <= pos);  out[t, h] = sigmoid(gate[t, h]) sum_g talk[h, g] sum_j w_g(j) v[kv(h), j],  kv(h) = h / (heads / kv_heads).
+ * qf float [T, heads, dim]; pool rows [v (vdim) | k (dim)], pool_stride elements between the kv_heads pools.  Two launches: the sums
+ * over the keys for every (head, value pool), part_o float [key_splits, T, heads, kv_heads, vdim] with part_ml float [key_splits, T,
+ * heads, 2] = (maximum, sum) - and qsv_talking_mix (gate NULL: none).
+ * qsv_talking_attention: any sizes (dim, vdim <= 512), one split, part_o already normalised (part_ml of the mix: NULL).
+ * qsv_talking_attention_mfma: where qsv_talking_attention_mfma_ok; tiles as for qsv_latent_attention_mfma, of at most
+ * qsv_talking_attention_tile_tokens(heads, kv_heads, key_pools) tokens; key_pools (a divisor of kv_heads, key_pools dim <= 512): pools
+ * whose heads share a workgroup, as qsv_talking_attention_key_pools proposes. */
+int qsv_talking_attention_key_pools(int heads, int kv_heads, int dim, int decode);
+int qsv_talking_attention_tile_tokens(int heads, int kv_heads, int key_pools);
+int qsv_talking_attention_mfma_ok(int dim, int vdim, int page, int dtype);
+int qsv_talking_attention(float* part_o, const float* qf, const void* pool, const int32_t* block_table, int table_stride,
+                          const int32_t* seq, const int32_t* pos, int window, int n_tokens, int heads, int kv_heads, int dim, int vdim,
+                          int page, int64_t pool_stride, float cap, int dtype, void* stream);
+int qsv_talking_attention_mfma(float* part_o, float* part_ml, const float* qf, const void* pool, const int32_t* block_table,
+                               int table_stride, const int32_t* pos, const int32_t* tiles, int n_tiles, int window, int n_tokens,
+                               int heads, int kv_heads, int dim, int vdim, int page, int64_t pool_stride, float cap, int key_pools,
+                               int key_splits, void* stream);
+int qsv_talking_mix(void* out, const float* part_o, const float* part_ml, const void* talk, const void* gate, int64_t gate_stride,
+                    int key_splits, int n_tokens, int heads, int kv_heads, int vdim, int dtype, void* stream);
 
 /* o[t, i] *= sigmoid(g[t * g_stride + i]),  i < n. */
 int qsv_sigmoid_gate(void* o, const void* g, int64_t g_stride, int n_tokens, int n, int dtype, void* stream);
@@ -225,7 +269,8 @@ int qsv_conv_silu_unit(float* out, const void* proj, int64_t stride, int off, in
  * q, k: [T, qk_heads, dim] (head h reads h / (heads / qk_heads)), v: [T, heads, vdim], each with its row stride, of type
  * qkv_dtype; o: float [T, heads, vdim].  max_run: the longest run's tokens as the host knows them (1: every run is one decoded
  * token - a kernel without staging is used; any larger value, or 0 for unknown: the general kernel). */
-/* Variants (0 / NULL: as above): head_decay != 0: decay is float [T, heads], one factor for all rows of a head's state;
+/* Variants (0 / NULL: as above): head_decay 1: decay is float [T, heads], one factor for all rows of a head's state; 2: float [heads],
+ * the same for every token;
  * kscale (float [T, heads]): k is multiplied by kscale[t, head] where it enters the state; v_cols < vdim: v has v_cols columns per
  * head and the state's column v_cols is fed with ones (it then holds sum of decayed kscale k: a normaliser, read out by q like
  * the others), further columns with zeros. */

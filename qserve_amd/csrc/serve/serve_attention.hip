@@ -22,7 +22,8 @@ __global__ __launch_bounds__(64 * NW) void latent_attention_wave_kernel(
     T* __restrict__ out, const float* __restrict__ qf, const T* pool, const int32_t* __restrict__ block_table,
     int table_stride, const int32_t* __restrict__ seq, const int32_t* __restrict__ pos, int window, int H, int rank, int R,
     int page, int per, int64_t pool_stride, int chunk, const float* __restrict__ bias, int bias_len, int keep_first,
-    const float* __restrict__ sink, const T* pooled, int64_t pooled_stride, int pool_block, int block_rows) {
+    const float* __restrict__ sink, const T* pooled, int64_t pooled_stride, int pool_block, int block_rows,
+    const float* __restrict__ slopes) {
     __shared__ float s_m[NW], s_l[NW];
     __shared__ float s_acc[NW][64 * EPL];
     const size_t t = blockIdx.x / H;
@@ -34,6 +35,7 @@ __global__ __launch_bounds__(64 * NW) void latent_attention_wave_kernel(
     int lo = window > 0 ? max(0, p - window + 1) : 0;
     if (chunk > 0) lo = max(lo, p - p % chunk);                  // chunks are counted from position 0 of the sequence
     const float* brow = bias ? bias + (size_t)h * bias_len : nullptr;
+    const float slope = slopes ? slopes[h] : 0.f;
     const int32_t* bt = block_table + (size_t)seq[t] * table_stride;
     const float* qrow = qf + (t * H + h) * (size_t)R;
     float q[EPL], acc[EPL];
@@ -75,6 +77,7 @@ __global__ __launch_bounds__(64 * NW) void latent_attention_wave_kernel(
             }
             d = wave_sum(d);
             if (brow) d += brow[min(p - jj, bias_len - 1)];
+            if (slopes) d -= slope * (float)(p - jj);
             s[k] = ok ? d : -INFINITY;
         }
         float mx = m;
@@ -127,12 +130,12 @@ template <typename T>
 int launch_wave(void* out, const float* qf, const void* pool, const int32_t* bt, int ts, const int32_t* seq, const int32_t* pos,
                 int window, int n, int H, int rank, int R, int page, int per, int64_t pool_stride, int chunk, const float* bias,
                 int bias_len, int keep_first, const float* sink, const void* pooled, int64_t pooled_stride, int pool_block,
-                int block_rows, hipStream_t st_) {
+                int block_rows, const float* slopes, hipStream_t st_) {
     const dim3 grid(n * H), block(64 * NW);
 #define QSV_ATT(E)                                                                                                        \
     hipLaunchKernelGGL((latent_attention_wave_kernel<T, E>), grid, block, 0, st_, (T*)out, qf, (const T*)pool, bt, ts, seq, pos, \
                        window, H, rank, R, page, per, pool_stride, chunk, bias, bias_len, keep_first, sink, (const T*)pooled,        \
-                       pooled_stride, pool_block, block_rows)
+                       pooled_stride, pool_block, block_rows, slopes)
     if (R <= 64) QSV_ATT(1);
     else if (R <= 128) QSV_ATT(2);
     else if (R <= 192) QSV_ATT(3);
@@ -153,7 +156,7 @@ extern "C" int qsv_latent_attention(void* out, const float* qf, const void* pool
                                     const int32_t* seq, const int32_t* pos, int window, int n, int H, int rank, int R, int page,
                                     int heads_per_pool, int64_t pool_stride, int chunk, const float* bias, int bias_len,
                                     int keep_first, const float* sink, const void* pooled, int64_t pooled_stride, int pool_block,
-                                    int block_rows, int dtype, int variant, void* stream) {
+                                    int block_rows, const float* slopes, int dtype, int variant, void* stream) {
     QSV_REQUIRE(out && qf && pool && block_table && seq && pos, "qsv_latent_attention: null argument");
     QSV_REQUIRE(chunk >= 0 && (!bias || bias_len > 0), "qsv_latent_attention: chunk %d, bias table of %d distances", chunk, bias_len);
     QSV_REQUIRE(n >= 0 && H > 0 && rank > 0 && R >= rank && page > 0 && table_stride > 0 && window >= 0,
@@ -164,13 +167,14 @@ extern "C" int qsv_latent_attention(void* out, const float* qf, const void* pool
     QSV_REQUIRE(!pooled || (window > 0 && !chunk && !bias && !keep_first && pool_block > 0 && block_rows > 0 && pooled_stride >= 0 &&
                             (int64_t)block_rows * pool_block >= page),
                 "qsv_latent_attention: pooled blocks of %d positions, %d rows per page of %d", pool_block, block_rows, page);
+    QSV_REQUIRE(!slopes || !pooled, "qsv_latent_attention: distance slopes with pooled blocks");
     if (n == 0) return QSV_OK;
     QSV_REQUIRE((int64_t)n * H < (1ll << 31), "qsv_latent_attention: too many (token, head) pairs");
     (void)variant;
     int rc = QSV_OK;
     QSV_DISPATCH(dtype, "qsv_latent_attention",
                  rc = launch_wave<T>(out, qf, pool, block_table, table_stride, seq, pos, window, n, H, rank, R, page, heads_per_pool,
-                                     pool_stride, chunk, bias, bias_len, keep_first, sink, pooled, pooled_stride, pool_block, block_rows,
+                                     pool_stride, chunk, bias, bias_len, keep_first, sink, pooled, pooled_stride, pool_block, block_rows, slopes,
                                      (hipStream_t)stream));
     if (rc != QSV_OK) return rc;
     return qsv_launch_status("qsv_latent_attention");

@@ -39,7 +39,7 @@ __global__ __launch_bounds__(64 * NWV, (RT > 10 ? 1 : 2)) void latent_attention_
     int window, int H, int rank, int R, int page, int HP, int TQ, float* __restrict__ part_o, float* __restrict__ part_ml,
     int n_tokens, int s_lo, int s_hi, int per, int64_t pool_stride, int chunk, const float* __restrict__ bias, int bias_len,
     int keep_first, const float* __restrict__ sink, const bf16_t* __restrict__ pooled_base, int64_t pooled_stride, int pool_block,
-    int block_rows) {
+    int block_rows, const float* __restrict__ slopes) {
     constexpr int RS = 32 * RT + 8;                      // row stride (elements) of the row-major tile
     extern __shared__ __attribute__((aligned(16))) unsigned char smem[];
     bf16_t* Ks = (bf16_t*)smem;                          // [BN][RS]
@@ -69,6 +69,8 @@ __global__ __launch_bounds__(64 * NWV, (RT > 10 ? 1 : 2)) void latent_attention_
     int lo_row = window > 0 ? max(0, p_row - window + 1) : 0;
     if (chunk > 0) lo_row = max(lo_row, p_row - p_row % chunk);   // chunks are counted from position 0 of the sequence
     const float* brow = bias ? bias + (size_t)(row_ok ? head : 0) * bias_len : nullptr;
+
+    const float slope = slopes ? slopes[row_ok ? head : 0] : 0.f;
 
     // block key range (tokens of a tile are consecutive positions; read both ends)
     const int p_first = pos[t0], p_last = pos[t0 + ntok - 1];
@@ -197,6 +199,7 @@ __global__ __launch_bounds__(64 * NWV, (RT > 10 ? 1 : 2)) void latent_attention_
                 const int key = k0 + 16 * mt + 4 * g4 + r;
                 const bool vis = (pooled && pre) ? key < nb_row : (key <= p_row && (key >= lo_row || key < keep_first));
                 if (brow) sacc[mt][r] += bv[mt][r];
+                if (slopes) sacc[mt][r] -= slope * (float)(p_row - key);
                 sacc[mt][r] = vis ? sacc[mt][r] : -INFINITY;
                 tmax = fmaxf(tmax, sacc[mt][r]);
             }
@@ -354,7 +357,7 @@ extern "C" int qsv_latent_attention_mfma(void* out, const float* qf, const void*
                                          int H, int rank, int R, int page, int key_splits, float* part_o, float* part_ml,
                                          int n_tokens, int q_first, int heads_per_pool, int64_t pool_stride, int chunk,
                                          const float* bias, int bias_len, int keep_first, const float* sink, const void* pooled,
-                                         int64_t pooled_stride, int pool_block, int block_rows, void* stream) {
+                                         int64_t pooled_stride, int pool_block, int block_rows, const float* slopes, void* stream) {
     QSV_REQUIRE(keep_first >= 0 && (!keep_first || (window > 0 && !chunk)),
                 "qsv_latent_attention_mfma: %d kept first positions need a window and no chunks", keep_first);
     QSV_REQUIRE(!pooled || (window > 0 && !chunk && !bias && !keep_first && pool_block > 0 && block_rows > 0 && pooled_stride >= 0 &&
@@ -364,6 +367,7 @@ extern "C" int qsv_latent_attention_mfma(void* out, const float* qf, const void*
     QSV_REQUIRE(out && qf && pool && block_table && pos && tiles, "qsv_latent_attention_mfma: null argument");
     QSV_REQUIRE(qsv_latent_attention_mfma_ok(rank, R, QSV_BF16) && R >= rank && H > 0 && page > 0 && page % BN == 0 && window >= 0 && n_tiles >= 0,
                 "qsv_latent_attention_mfma: sizes not supported (rank %d, row %d)", rank, R);
+    QSV_REQUIRE(!slopes || !pooled, "qsv_latent_attention_mfma: distance slopes with pooled blocks");
     if (n_tiles == 0) return QSV_OK;
     QSV_REQUIRE(heads_per_pool > 0 && H % heads_per_pool == 0 && pool_stride >= 0,
                 "qsv_latent_attention_mfma: %d heads over pools of %d", H, heads_per_pool);
@@ -387,7 +391,7 @@ extern "C" int qsv_latent_attention_mfma(void* out, const float* qf, const void*
         hipLaunchKernelGGL((latent_attention_mfma_kernel<RT, CT>), grid, block, lds, (hipStream_t)stream, (bf16_t*)out, qf,  \
                            (const bf16_t*)pool, block_table, table_stride, pos, tiles, window, H, rank, R, page, g.HP, g.TQ, \
                            part_o, part_ml, n_tokens, s_lo, s_hi, heads_per_pool, pool_stride, chunk, bias, bias_len,         \
-                           keep_first, sink, (const bf16_t*)pooled, pooled_stride, pool_block, block_rows);                       \
+                           keep_first, sink, (const bf16_t*)pooled, pooled_stride, pool_block, block_rows, slopes);                       \
     } while (0)
     if (rt <= 4 && ct <= 8) QSV_MFMA(4, 8);
     else if (rt <= 6 && ct <= 12) QSV_MFMA(6, 12);

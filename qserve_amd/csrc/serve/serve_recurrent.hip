@@ -150,7 +150,7 @@ __global__ __launch_bounds__(256, OCC) void recurrent_scan_kernel(float* __restr
                     const size_t t = (size_t)(first + c0 + tt);
                     if (r < dim) {
                         if (which == 2 && head_decay) {
-                            const float g = decay[t * H + h];
+                            const float g = head_decay == 2 ? decay[h] : decay[t * H + h];
                             val = make_float4(g, g, g, g);
                         } else {
                             val = which == 0 ? ld4(k, t * k_stride + (size_t)qh * dim + r)
@@ -187,7 +187,7 @@ __global__ __launch_bounds__(256, OCC) void recurrent_scan_kernel(float* __restr
                     if (r < dim)
                         val = which == 0 ? ld(k, t * k_stride + (size_t)qh * dim + r) * (kscale ? kscale[t * H + h] : 1.0f)
                             : which == 1 ? ld(q, t * q_stride + (size_t)qh * dim + r)
-                                         : (head_decay ? decay[t * H + h] : decay[(t * H + h) * (size_t)dim + r]);
+                                         : (head_decay == 2 ? decay[h] : head_decay ? decay[t * H + h] : decay[(t * H + h) * (size_t)dim + r]);
                 }
                 pk[i] = val;
             }
@@ -350,7 +350,7 @@ __global__ __launch_bounds__(256) void recurrent_step_kernel(float* __restrict__
         S[i] = (!fresh && col_ok && ok) ? Sg[(size_t)(r0 + i) * vdim] : 0.f;
         kc[i] = ok ? ld(k, t * k_stride + (size_t)qh * dim + r0 + i) * kb : 0.f;
         qc[i] = ok ? ld(q, t * q_stride + (size_t)qh * dim + r0 + i) : 0.f;
-        gc[i] = ok ? (head_decay ? decay[t * H + h] : decay[(t * H + h) * (size_t)dim + r0 + i]) : 0.f;
+        gc[i] = ok ? (head_decay == 2 ? decay[h] : head_decay ? decay[t * H + h] : decay[(t * H + h) * (size_t)dim + r0 + i]) : 0.f;
     }
     const float vc = !col_ok ? 0.f : j < v_cols ? ld(v, t * v_stride + (size_t)h * v_cols + j) : j == v_cols ? 1.0f : 0.f;
     float acc = 0.f;

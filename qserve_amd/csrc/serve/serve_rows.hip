@@ -533,7 +533,8 @@ extern "C" int qsv_add_normed_rms_norm(float* x, void* h, const void* y, const v
 }
 
 // ---- query / key norms (per head or over the projection), rotated pairs, cache write -----------------------------------------------
-// One workgroup per token.  Statistics: per head a wave's sum over `dim`; over the projection a workgroup sum.  The rotation works
+// q_b / k_b / v_b (each may be NULL) are added to the projections first; the pairs are neighbours or, with `halves`, (i, i + rot_n / 2);
+// head_scale (may be NULL) multiplies the common scale; a query row starts with q_pad zeros.  One workgroup per token.  Statistics: per head a wave's sum over `dim`; over the projection a workgroup sum.  The rotation works
 // on normed values staged in LDS (a pair's two values may sit in different threads).  Dynamic LDS: (heads + kv_heads) * dim floats.
 template <typename T, typename TI>
 __global__ __launch_bounds__(NT) void qk_norm_rope_prep_kernel(float* __restrict__ qf, const TI* __restrict__ q, int64_t q_stride,
@@ -542,7 +543,10 @@ __global__ __launch_bounds__(NT) void qk_norm_rope_prep_kernel(float* __restrict
                                                                const T* __restrict__ q_w, const T* __restrict__ k_w, int per_head,
                                                                float eps, const float* __restrict__ rope, int rot_n, float scale,
                                                                T* __restrict__ pool, int64_t pool_rows,
-                                                               const int64_t* __restrict__ slot, const int32_t* __restrict__ pos) {
+                                                               const int64_t* __restrict__ slot, const int32_t* __restrict__ pos,
+                                                               const T* __restrict__ q_b, const T* __restrict__ k_b,
+                                                               const T* __restrict__ v_b, int halves,
+                                                               const float* __restrict__ head_scale, int q_pad) {
     extern __shared__ float sm[];
     __shared__ float red[NT / 64 + 1];
     const size_t t = blockIdx.x;
@@ -553,67 +557,76 @@ __global__ __launch_bounds__(NT) void qk_norm_rope_prep_kernel(float* __restrict
     const TI* krow = k ? k + t * k_stride : nullptr;
     if (per_head) {
         for (int hh = wv; hh < NH; hh += NT / 64) {
-            const TI* src = hh < H ? qrow + (size_t)hh * dim : krow + (size_t)(hh - H) * dim;
-            const T* w = hh < H ? q_w : k_w;
+            const bool isq = hh < H;
+            const TI* src = isq ? qrow + (size_t)hh * dim : krow + (size_t)(hh - H) * dim;
+            const T* w = isq ? q_w : k_w;
+            const T* bias = isq ? q_b : k_b;
+            const int b0 = (isq ? hh : hh - H) * dim;
             float s = 0.f;
             for (int e = lane; e < dim; e += 64) {
-                const float u = ld(src, e);
+                const float u = ld(src, e) + (bias ? ld(bias, b0 + e) : 0.f);
+                nq[hh * dim + e] = u;
                 s += u * u;
             }
             const float inv = 1.0f / sqrtf(wave_sum(s) / (float)dim + eps);
-            for (int e = lane; e < dim; e += 64) nq[hh * dim + e] = ld(src, e) * inv * ld(w, e);
+            for (int e = lane; e < dim; e += 64) nq[hh * dim + e] *= inv * ld(w, e);
         }
     } else {
         float s = 0.f;
         for (int i = threadIdx.x; i < H * dim; i += NT) {
-            const float u = ld(qrow, i);
+            const float u = ld(qrow, i) + (q_b ? ld(q_b, i) : 0.f);
+            nq[i] = u;
             s += u * u;
         }
         const float qinv = 1.0f / sqrtf(block_sum<NT>(s, red) / (float)(H * dim) + eps);
-        for (int i = threadIdx.x; i < H * dim; i += NT) nq[i] = ld(qrow, i) * qinv * ld(q_w, i);
+        for (int i = threadIdx.x; i < H * dim; i += NT) nq[i] *= qinv * ld(q_w, i);
         if (k) {
             s = 0.f;
             for (int i = threadIdx.x; i < G * dim; i += NT) {
-                const float u = ld(krow, i);
+                const float u = ld(krow, i) + (k_b ? ld(k_b, i) : 0.f);
+                nq[H * dim + i] = u;
                 s += u * u;
             }
             const float kinv = 1.0f / sqrtf(block_sum<NT>(s, red) / (float)(G * dim) + eps);
-            for (int i = threadIdx.x; i < G * dim; i += NT) nq[H * dim + i] = ld(krow, i) * kinv * ld(k_w, i);
+            for (int i = threadIdx.x; i < G * dim; i += NT) nq[H * dim + i] *= kinv * ld(k_w, i);
         }
     }
     __syncthreads();
-    if (rope) {                                        // pairs of neighbours, each by one thread
+    if (rope) {                                        // each pair by one thread
         const int half = rot_n / 2;
         const float* cs = rope + (size_t)pos[t] * rot_n;
         for (int idx = threadIdx.x; idx < NH * half; idx += NT) {
             const int hh = idx / half, i = idx - hh * half;
             const float c = cs[i], sn = cs[half + i];
-            const float a = nq[hh * dim + 2 * i], b = nq[hh * dim + 2 * i + 1];
-            nq[hh * dim + 2 * i] = a * c - b * sn;
-            nq[hh * dim + 2 * i + 1] = b * c + a * sn;
+            const int i0 = hh * dim + (halves ? i : 2 * i), i1 = i0 + (halves ? half : 1);
+            const float a = nq[i0], b = nq[i1];
+            nq[i0] = a * c - b * sn;
+            nq[i1] = b * c + a * sn;
         }
         __syncthreads();
     }
-    const int R = vdim + dim;
-    for (int idx = threadIdx.x; idx < H * R; idx += NT) {
-        const int h = idx / R, c = idx - h * R;
-        qf[t * H * (size_t)R + idx] = c < vdim ? 0.f : nq[h * dim + c - vdim] * scale;
+    const int RQ = q_pad + dim, R = vdim + dim;
+    for (int idx = threadIdx.x; idx < H * RQ; idx += NT) {
+        const int h = idx / RQ, c = idx - h * RQ;
+        qf[t * H * (size_t)RQ + idx] = c < q_pad ? 0.f : nq[h * dim + c - q_pad] * (head_scale ? scale * head_scale[h] : scale);
     }
     if (!k) return;
     const size_t dst = (size_t)slot[t];
     const TI* vrow = v + t * v_stride;
     for (int idx = threadIdx.x; idx < G * R; idx += NT) {
         const int g = idx / R, c = idx - g * R;
-        st(pool, ((size_t)g * pool_rows + dst) * R + c, c < vdim ? ld(vrow, g * vdim + c) : nq[(H + g) * dim + c - vdim]);
+        st(pool, ((size_t)g * pool_rows + dst) * R + c,
+           c < vdim ? ld(vrow, g * vdim + c) + (v_b ? ld(v_b, g * vdim + c) : 0.f) : nq[(H + g) * dim + c - vdim]);
     }
 }
 extern "C" int qsv_qk_norm_rope_prep(float* qf, const void* q, int64_t q_stride, const void* k, int64_t k_stride, const void* v,
                                      int64_t v_stride, int qkv_dtype, int heads, int kv_heads, int dim, int vdim, const void* q_w,
                                      const void* k_w, int per_head, float eps, const float* rope, int rot_n, float scale, void* pool,
-                                     int64_t pool_rows, const int64_t* slot, const int32_t* pos, int n, int dtype, void* stream) {
+                                     int64_t pool_rows, const int64_t* slot, const int32_t* pos, int n, const void* q_b, const void* k_b,
+                                     const void* v_b, int halves, const float* head_scale, int q_pad, int dtype, void* stream) {
     QSV_REQUIRE(qf && q && q_w && pos, "qsv_qk_norm_rope_prep: null argument");
     QSV_REQUIRE(!k || (v && k_w && pool && slot), "qsv_qk_norm_rope_prep: keys without values, weight, pool or rows");
-    QSV_REQUIRE(heads > 0 && kv_heads > 0 && dim > 0 && vdim > 0 && n >= 0 && q_stride >= (int64_t)heads * dim &&
+    QSV_REQUIRE(heads > 0 && kv_heads > 0 && dim > 0 && vdim > 0 && n >= 0 && q_pad >= 0 && q_stride >= (int64_t)heads * dim &&
                     (!k || (k_stride >= (int64_t)kv_heads * dim && v_stride >= (int64_t)kv_heads * vdim)),
                 "qsv_qk_norm_rope_prep: bad sizes");
     QSV_REQUIRE(!rope || (rot_n > 0 && rot_n % 2 == 0 && rot_n <= dim), "qsv_qk_norm_rope_prep: %d rotated dimensions of %d", rot_n, dim);
@@ -626,9 +639,216 @@ extern "C" int qsv_qk_norm_rope_prep(float* qf, const void* q, int64_t q_stride,
     QSV_DISPATCH(dtype, "qsv_qk_norm_rope_prep",                                                                                 \
                  hipLaunchKernelGGL((qk_norm_rope_prep_kernel<T, TI>), dim3(n), dim3(NT), lds, (hipStream_t)stream, qf, (const TI*)q, \
                                     q_stride, (const TI*)k, k_stride, (const TI*)v, v_stride, heads, kv_heads, dim, vdim,          \
-                                    (const T*)q_w, (const T*)k_w, per_head, eps, rope, rot_n, scale, (T*)pool, pool_rows, slot, pos))
+                                    (const T*)q_w, (const T*)k_w, per_head, eps, rope, rot_n, scale, (T*)pool, pool_rows, slot, pos,  \
+                                    (const T*)q_b, (const T*)k_b, (const T*)v_b, halves, head_scale, q_pad))
     if (qkv_dtype == QSV_F32) QSV_QKP(float);
     else QSV_QKP(bf16_t);
 #undef QSV_QKP
     return qsv_launch_status("qsv_qk_norm_rope_prep");
+}
+
+
+// ---- embedding with a norm: x = rms_norm(table[token]) * w -------------------------------------------------------------------------
+template <typename T>
+__global__ __launch_bounds__(NT) void embed_rms_norm_kernel(float* __restrict__ x, const T* __restrict__ table,
+                                                            const int32_t* __restrict__ tokens, const T* __restrict__ w, float eps, int D) {
+    __shared__ float red[NT / 64 + 1];
+    const size_t t = blockIdx.x;
+    const T* row = table + (size_t)tokens[t] * D;
+    float s = 0.f;
+    for (int i = threadIdx.x; i < D; i += NT) s += ld(row, i) * ld(row, i);
+    const float inv = 1.0f / sqrtf(block_sum<NT>(s, red) / (float)D + eps);
+    for (int i = threadIdx.x; i < D; i += NT) x[t * D + i] = ld(row, i) * inv * ld(w, i);
+}
+extern "C" int qsv_embed_rms_norm(float* x, const void* table, const int32_t* tokens, const void* w, float eps, int n, int D, int dtype,
+                                  void* stream) {
+    QSV_REQUIRE(x && table && tokens && w && n >= 0 && D > 0, "qsv_embed_rms_norm: bad arguments");
+    if (n == 0) return QSV_OK;
+    QSV_DISPATCH(dtype, "qsv_embed_rms_norm",
+                 hipLaunchKernelGGL(embed_rms_norm_kernel<T>, dim3(n), dim3(NT), 0, (hipStream_t)stream, x, (const T*)table, tokens,
+                                    (const T*)w, eps, D));
+    return qsv_launch_status("qsv_embed_rms_norm");
+}
+
+// ---- a token's row plus its causal convolution over time: h_t = x_t + sum_j w[j] x_(t - past + j),  j = 0 .. past = taps - 1 ------------
+// Inputs before a run's start come from the sequence's history (rows of `past` inputs, oldest first; none at the sequence's start);
+// a run's last token writes the new history into the state's other copy.
+struct ConvState {
+    const float* w;                 // [taps, D]
+    float* hist;                    // [2 slots, past, D]
+    const int32_t *run_off, *rd, *wr;
+    int past;
+};
+// the input d tokens before token t (the i-th of its run), channels c .. c + 3 (V4) or c
+__device__ __forceinline__ float4 conv_in4(const float* x, const ConvState& cv, size_t t, int i, int rd, int d, int D, int c) {
+    if (d <= i) return ld4v(x, (t - d) * (size_t)D + c);
+    if (rd >= 0) return ld4v(cv.hist, ((size_t)rd * cv.past + (cv.past + i - d)) * D + c);
+    return make_float4(0.f, 0.f, 0.f, 0.f);
+}
+__device__ __forceinline__ float conv_in1(const float* x, const ConvState& cv, size_t t, int i, int rd, int d, int D, int c) {
+    if (d <= i) return x[(t - d) * (size_t)D + c];
+    return rd >= 0 ? cv.hist[((size_t)rd * cv.past + (cv.past + i - d)) * D + c] : 0.f;
+}
+// h of channels c .. c + 3 of token t, whose own row holds v there; writes the history if the token ends its run
+template <typename T>
+__device__ __forceinline__ void conv_tail4(T* h, const float* x, const ConvState& cv, size_t t, int i, int rd, int wr, int D, int c, float4 v) {
+    const float4 w0 = ld4v(cv.w, (size_t)cv.past * D + c);
+    float4 a = make_float4(v.x + w0.x * v.x, v.y + w0.y * v.y, v.z + w0.z * v.z, v.w + w0.w * v.w);
+    for (int d = 1; d <= cv.past; ++d) {
+        const float4 u = conv_in4(x, cv, t, i, rd, d, D, c), w = ld4v(cv.w, (size_t)(cv.past - d) * D + c);
+        a.x += w.x * u.x; a.y += w.y * u.y; a.z += w.z * u.z; a.w += w.w * u.w;
+        if (wr >= 0 && d < cv.past) st4v(cv.hist, ((size_t)wr * cv.past + (cv.past - 1 - d)) * D + c, u);
+    }
+    if (wr >= 0 && cv.past > 0) st4v(cv.hist, ((size_t)wr * cv.past + cv.past - 1) * D + c, v);
+    st4v(h, t * D + c, a);
+}
+template <typename T>
+__device__ __forceinline__ void conv_tail1(T* h, const float* x, const ConvState& cv, size_t t, int i, int rd, int wr, int D, int c, float v) {
+    float a = v + cv.w[(size_t)cv.past * D + c] * v;
+    for (int d = 1; d <= cv.past; ++d) {
+        const float u = conv_in1(x, cv, t, i, rd, d, D, c);
+        a += cv.w[(size_t)(cv.past - d) * D + c] * u;
+        if (wr >= 0 && d < cv.past) cv.hist[((size_t)wr * cv.past + (cv.past - 1 - d)) * D + c] = u;
+    }
+    if (wr >= 0 && cv.past > 0) cv.hist[((size_t)wr * cv.past + cv.past - 1) * D + c] = v;
+    st(h, t * D + c, a);
+}
+template <typename T, bool VEC>
+__global__ __launch_bounds__(NT) void residual_conv_kernel(T* __restrict__ h, const float* __restrict__ x, ConvState cv, int D) {
+    const size_t t = blockIdx.x;
+    const int i = cv.run_off[t], rd = cv.rd[t], wr = cv.wr[t];
+    if (VEC) {
+        for (int c = threadIdx.x * 4; c < D; c += NT * 4) conv_tail4(h, x, cv, t, i, rd, wr, D, c, ld4v(x, t * D + c));
+    } else {
+        for (int c = threadIdx.x; c < D; c += NT) conv_tail1(h, x, cv, t, i, rd, wr, D, c, x[t * D + c]);
+    }
+}
+extern "C" int qsv_residual_conv(void* h, const float* x, const float* w, int taps, float* hist, const int32_t* run_off,
+                                 const int32_t* state_rd, const int32_t* state_wr, int n, int D, int dtype, void* stream) {
+    QSV_REQUIRE(h && x && w && run_off && state_rd && state_wr && n >= 0 && D > 0 && taps >= 1 && (taps == 1 || hist),
+                "qsv_residual_conv: bad arguments");
+    if (n == 0) return QSV_OK;
+    const ConvState cv = {w, hist, run_off, state_rd, state_wr, taps - 1};
+    if (D % 4 == 0)
+        QSV_DISPATCH(dtype, "qsv_residual_conv",
+                     hipLaunchKernelGGL((residual_conv_kernel<T, true>), dim3(n), dim3(NT), 0, (hipStream_t)stream, (T*)h, x, cv, D));
+    else
+        QSV_DISPATCH(dtype, "qsv_residual_conv",
+                     hipLaunchKernelGGL((residual_conv_kernel<T, false>), dim3(n), dim3(NT), 0, (hipStream_t)stream, (T*)h, x, cv, D));
+    return qsv_launch_status("qsv_residual_conv");
+}
+
+// ---- norm after the sum: x = rms_norm(alpha x + y) * w, h = x in the storage type ------------------------------------------------------
+// With `cv.w` (steps in which every run is one token: no row of this launch reads another's new x) h is instead the next mixer's
+// input, x plus its convolution over time.  The row in registers (VPT groups of four values per thread), or any width.
+template <typename T, int VPT>
+__global__ __launch_bounds__(NT) void scaled_add_rms_norm_vec_kernel(float* __restrict__ x, T* __restrict__ h, const T* __restrict__ y,
+                                                                     float alpha, const T* __restrict__ w, float eps, int D, ConvState cv) {
+    __shared__ float red[NT / 64 + 1];
+    const size_t t = blockIdx.x;
+    float4 v[VPT];
+    float s = 0.f;
+#pragma unroll
+    for (int k = 0; k < VPT; ++k) {
+        const int i = (threadIdx.x + k * NT) * 4;
+        if (i >= D) continue;
+        const float4 a = ld4v(x, t * D + i), b = ld4v(y, t * D + i);
+        v[k] = make_float4(alpha * a.x + b.x, alpha * a.y + b.y, alpha * a.z + b.z, alpha * a.w + b.w);
+        s += v[k].x * v[k].x + v[k].y * v[k].y + v[k].z * v[k].z + v[k].w * v[k].w;
+    }
+    const float inv = 1.0f / sqrtf(block_sum<NT>(s, red) / (float)D + eps);
+#pragma unroll
+    for (int k = 0; k < VPT; ++k) {
+        const int i = (threadIdx.x + k * NT) * 4;
+        if (i >= D) continue;
+        const float4 g = ld4v(w, i);
+        v[k] = make_float4(v[k].x * inv * g.x, v[k].y * inv * g.y, v[k].z * inv * g.z, v[k].w * inv * g.w);
+        st4v(x, t * D + i, v[k]);
+        if (!h) continue;
+        if (cv.w) conv_tail4(h, x, cv, t, 0, cv.rd[t], cv.wr[t], D, i, v[k]);
+        else st4v(h, t * D + i, v[k]);
+    }
+}
+template <typename T>
+__global__ __launch_bounds__(NT) void scaled_add_rms_norm_kernel(float* __restrict__ x, T* __restrict__ h, const T* __restrict__ y,
+                                                                 float alpha, const T* __restrict__ w, float eps, int D, ConvState cv) {
+    __shared__ float red[NT / 64 + 1];
+    const size_t t = blockIdx.x;
+    float s = 0.f;
+    for (int i = threadIdx.x; i < D; i += NT) {
+        const float v = alpha * x[t * D + i] + ld(y, t * D + i);
+        s += v * v;
+    }
+    const float inv = 1.0f / sqrtf(block_sum<NT>(s, red) / (float)D + eps);
+    for (int i = threadIdx.x; i < D; i += NT) {
+        const float v = (alpha * x[t * D + i] + ld(y, t * D + i)) * inv * ld(w, i);
+        x[t * D + i] = v;
+        if (!h) continue;
+        if (cv.w) conv_tail1(h, x, cv, t, 0, cv.rd[t], cv.wr[t], D, i, v);
+        else st(h, t * D + i, v);
+    }
+}
+extern "C" int qsv_scaled_add_rms_norm(float* x, void* h, const void* y, float alpha, const void* w, float eps, const float* conv_w,
+                                       int taps, float* hist, const int32_t* state_rd, const int32_t* state_wr, int n, int D, int dtype,
+                                       void* stream) {
+    QSV_REQUIRE(x && y && w && n >= 0 && D > 0, "qsv_scaled_add_rms_norm: bad arguments");
+    QSV_REQUIRE(!conv_w || (h && taps >= 1 && state_rd && state_wr && (taps == 1 || hist)),
+                "qsv_scaled_add_rms_norm: a convolution without its state or output");
+    if (n == 0) return QSV_OK;
+    const ConvState cv = {conv_w, hist, nullptr, state_rd, state_wr, conv_w ? taps - 1 : 0};
+    const int vecs = (D / 4 + NT - 1) / NT;
+    if (D % 4 == 0 && vecs <= 8) {
+#define QSV_SAN(V)                                                                                                               \
+    QSV_DISPATCH(dtype, "qsv_scaled_add_rms_norm",                                                                               \
+                 hipLaunchKernelGGL((scaled_add_rms_norm_vec_kernel<T, V>), dim3(n), dim3(NT), 0, (hipStream_t)stream, x, (T*)h, \
+                                    (const T*)y, alpha, (const T*)w, eps, D, cv))
+        if (vecs <= 1) QSV_SAN(1);
+        else if (vecs <= 2) QSV_SAN(2);
+        else if (vecs <= 4) QSV_SAN(4);
+        else QSV_SAN(8);
+#undef QSV_SAN
+        return qsv_launch_status("qsv_scaled_add_rms_norm");
+    }
+    QSV_DISPATCH(dtype, "qsv_scaled_add_rms_norm",
+                 hipLaunchKernelGGL(scaled_add_rms_norm_kernel<T>, dim3(n), dim3(NT), 0, (hipStream_t)stream, x, (T*)h, (const T*)y,
+                                    alpha, (const T*)w, eps, D, cv));
+    return qsv_launch_status("qsv_scaled_add_rms_norm");
+}
+
+// ---- retention operands: queries and keys turned by the position (halves layout), everything float --------------------------------------
+// out[t] = [ rot(q[t]) (H dim) | rot(k[t]) (H dim) | v[t] (H vdim) ]; rope float [positions, 2, rot_n / 2] or NULL.
+template <typename T>
+__global__ __launch_bounds__(NT) void rotate_qk_kernel(float* __restrict__ out, const T* __restrict__ qkv, int64_t stride, int heads2,
+                                                       int dim, int n_v, const float* __restrict__ rope, int rot_n,
+                                                       const int32_t* __restrict__ pos) {
+    const size_t t = blockIdx.x;
+    const T* row = qkv + t * stride;
+    const int nqk = heads2 * dim, half = rot_n >> 1;
+    float* o = out + t * (size_t)(nqk + n_v);
+    const float* cs = rope ? rope + (size_t)pos[t] * rot_n : nullptr;
+    for (int idx = threadIdx.x; idx < heads2 * half; idx += NT) {
+        const int hh = idx / half, i = idx - hh * half;
+        const float a = ld(row, hh * dim + i), b = ld(row, hh * dim + half + i), c = cs[i], s = cs[half + i];
+        o[hh * dim + i] = a * c - b * s;
+        o[hh * dim + half + i] = b * c + a * s;
+    }
+    if (rot_n < dim) {
+        const int rest = dim - rot_n;
+        for (int idx = threadIdx.x; idx < heads2 * rest; idx += NT) {
+            const int hh = idx / rest, i = hh * dim + rot_n + (idx - hh * rest);
+            o[i] = ld(row, i);
+        }
+    }
+    for (int i = threadIdx.x; i < n_v; i += NT) o[nqk + i] = ld(row, nqk + i);
+}
+extern "C" int qsv_rotate_qk(float* out, const void* qkv, int64_t stride, int heads, int dim, int vdim, const float* rope, int rot_n,
+                             const int32_t* pos, int n, int dtype, void* stream) {
+    QSV_REQUIRE(out && qkv && pos && n >= 0 && heads > 0 && dim > 0 && vdim > 0 && rot_n >= 0 && rot_n % 2 == 0 && rot_n <= dim &&
+                    (rope || rot_n == 0) && stride >= (int64_t)heads * (2 * dim + vdim),
+                "qsv_rotate_qk: bad arguments");
+    if (n == 0) return QSV_OK;
+    QSV_DISPATCH(dtype, "qsv_rotate_qk",
+                 hipLaunchKernelGGL(rotate_qk_kernel<T>, dim3(n), dim3(NT), 0, (hipStream_t)stream, out, (const T*)qkv, stride, 2 * heads,
+                                    dim, heads * vdim, rope, rot_n, pos));
+    return qsv_launch_status("qsv_rotate_qk");
 }

@@ -33,19 +33,20 @@ def _interleave(gate, up):
 
 
 class GatedFeedForward:
-    """Dense gated feed-forward: down . (act(gate . h) * (up . h)), no biases; act: "silu" or "gelu_tanh"."""
+    """Dense gated feed-forward: down . (act(gate . h) * (up . h)), no biases; act: "silu", "gelu_tanh", or "clamped" (g = min(gate . h,
+    limit), u = clamp(up . h, -limit, limit), unit g sigmoid(1.702 g) (u + 1))."""
 
-    def __init__(self, ops, *, gate, up, down, act="silu"):
+    def __init__(self, ops, *, gate, up, down, act="silu", limit=0.0):
         if gate.shape != up.shape or down.shape != (gate.size(1), gate.size(0)):
             raise ValueError("gated feed-forward: gate / up / down shapes do not fit each other")
-        if act not in ("silu", "gelu_tanh"):
-            raise ValueError(f"gated feed-forward: unknown activation {act!r}")
-        self.ops, self.w_in, self.w_down, self.act = ops, _interleave(gate, up), down.contiguous(), act
+        if act not in ("silu", "gelu_tanh", "clamped") or (act == "clamped" and not limit > 0.0):
+            raise ValueError(f"gated feed-forward: activation {act!r}, limit {limit}")
+        self.ops, self.w_in, self.w_down, self.act, self.limit = ops, _interleave(gate, up), down.contiguous(), act, float(limit)
 
     def __call__(self, h):
         from .ops import linear
         a = linear(h, self.w_in)
-        return linear(self.ops.glu(a) if self.act == "silu" else self.ops.glu(a, self.act), self.w_down)
+        return linear(self.ops.glu(a) if self.act == "silu" else self.ops.glu(a, self.act, self.limit), self.w_down)
 
 
 class TopKGatedMoE:

@@ -94,7 +94,7 @@ class HipOps:
     attention_split_target = 512        # workgroups a launch of the matrix-core attention should at least have
 
     def latent_attention(self, qf, pool, batch, window, rank, page, variant=0, key_splits=None, q_first=0, chunk=None, bias=None,
-                         keep_first=0, sink=None, pooled=None, pool_block=0):
+                         keep_first=0, sink=None, pooled=None, pool_block=0, slopes=None):
         """batch: the step's StepBatch (block table, sequence slot and position per token, work tiles).  variant: 0 = the
         matrix-core kernel where it takes the sizes, 1 = always the wave kernel.  key_splits: None = chosen from the number
         of workgroups and the context.  q_first: the caller's promise that every query is zero before that element.
@@ -103,8 +103,9 @@ class HipOps:
         is added to the score of query i and key j.  keep_first: the first that many positions of the sequence stay visible
         behind the window.  sink float [H]: exp(sink[h]) joins the softmax's denominator (no key, no value).  pooled (shaped like
         pool, ceil(page / pool_block) rows per page, written by `pool_blocks`): one more key / value row per block of pool_block
-        positions that lies wholly before the window."""
+        positions that lies wholly before the window.  slopes float [H]: slopes[h] * (i - j) is taken off the score."""
         T, H, R = qf.shape
+        assert slopes is None or (slopes.dtype == torch.float32 and slopes.numel() == H and slopes.is_contiguous() and pooled is None)
         assert sink is None or (sink.dtype == torch.float32 and sink.numel() == H and sink.is_contiguous())
         assert pooled is None or (window and pool_block > 0 and bias is None and not chunk and not keep_first and pooled.dim() == pool.dim()
                                   and pooled.dtype == pool.dtype and pooled.size(-1) == R)
@@ -112,7 +113,8 @@ class HipOps:
         per_page = (page + pool_block - 1) // pool_block if pooled is not None else 0
         assert pooled is None or pooled.size(-2) == pool.size(-2) // page * per_page
         more = (int(keep_first or 0), 0 if sink is None else sink.data_ptr(), 0 if pooled is None else pooled.data_ptr(),
-                0 if pooled is None or pooled.dim() == 2 else pooled.stride(0), int(pool_block) if pooled is not None else 0, per_page)
+                0 if pooled is None or pooled.dim() == 2 else pooled.stride(0), int(pool_block) if pooled is not None else 0, per_page,
+                0 if slopes is None else slopes.data_ptr())
         assert bias is None or (bias.dtype == torch.float32 and bias.dim() == 2 and bias.size(0) == H and bias.is_contiguous())
         extra = (int(chunk or 0), 0 if bias is None else bias.data_ptr(), 0 if bias is None else bias.size(1))
         block_table, seq, pos = batch.block_table, batch.seq, batch.pos
@@ -331,27 +333,35 @@ class HipOps:
         self.check(self.L.qsv_relu_sq(a.data_ptr(), a.numel(), self.code, self._s()), "relu_sq")
         return a
 
-    def qk_norm_rope_prep(self, q, k, v, heads, kv_heads, dim, vdim, q_w, k_w, per_head, eps, rope, rot_n, scale, pool, batch):
+    def qk_norm_rope_prep(self, q, k, v, heads, kv_heads, dim, vdim, q_w, k_w, per_head, eps, rope, rot_n, scale, pool, batch,
+                          q_b=None, k_b=None, v_b=None, halves=False, head_scale=None, q_pad=None):
         """q [T, heads * dim], k [T, kv_heads * dim], v [T, kv_heads * vdim] (float or storage type, column slices are fine; k and v
-        None: the layer caches nothing).  Queries and keys are RMS-normed per head (weight [dim], shared by the heads) or over the
-        whole projection (weight as wide as it), then the first rot_n dimensions of every head turn with the position (pairs of
-        neighbours; rope float [positions, 2, rot_n / 2] or None).  -> float queries [T, heads, vdim + dim] = [0 | q * scale];
-        writes the cache rows [v | k] of the step's tokens into pool [kv_heads, rows, vdim + dim]."""
+        None: the layer caches nothing; v may be k itself: values that are the projected keys).  q_b, k_b, v_b (one per channel) are added
+        first.  Queries and keys are RMS-normed per head (weight [dim], shared by the heads) or over the whole projection (weight as wide
+        as it), then the first rot_n dimensions of every head turn with the position (pairs of neighbours, or with `halves` (i, i + rot_n
+        / 2); rope float [positions, 2, rot_n / 2] or None).  -> float queries [T, heads, q_pad + dim] = [0 | q * scale *
+        head_scale[h]] (q_pad None: vdim); writes the cache rows [v | k] of the step's tokens into pool [kv_heads, rows, vdim + dim]."""
         T = q.size(0)
-        qf = torch.empty((T, heads, vdim + dim), dtype=torch.float32, device=q.device)
-        self._need(q_w, k_w, rope, pool, batch.slot, batch.pos)
+        q_pad = vdim if q_pad is None else int(q_pad)
+        qf = torch.empty((T, heads, q_pad + dim), dtype=torch.float32, device=q.device)
+        self._need(q_w, k_w, rope, pool, batch.slot, batch.pos, q_b, k_b, v_b, head_scale)
         assert q.stride(1) == 1 and q.size(1) == heads * dim and q_w.dtype == self.dtype and q_w.numel() == (dim if per_head else heads * dim)
         assert rope is None or (rope.dtype == torch.float32 and rope.size(-1) * 2 == rot_n and rot_n <= dim and rope.size(0) > batch.max_pos)
+        for b, n in ((q_b, heads * dim), (k_b, kv_heads * dim), (v_b, kv_heads * vdim)):
+            assert b is None or (b.dtype == self.dtype and b.numel() == n)
+        assert head_scale is None or (head_scale.dtype == torch.float32 and head_scale.numel() == heads)
         kp = [0, 0, 0, 0, 0, 0, 0]
         if k is not None:
             assert k.dtype == v.dtype == q.dtype and k.stride(1) == v.stride(1) == 1 and k.size(1) == kv_heads * dim
             assert v.size(1) == kv_heads * vdim and k_w.dtype == self.dtype and k_w.numel() == (dim if per_head else kv_heads * dim)
             assert pool.shape[0] == kv_heads and pool.shape[2] == vdim + dim and pool.dtype == self.dtype
             kp = [k.data_ptr(), k.stride(0), v.data_ptr(), v.stride(0), k_w.data_ptr(), pool.data_ptr(), pool.size(1)]
+        opt = [0 if b is None else b.data_ptr() for b in (q_b, k_b, v_b)]
         self.check(self.L.qsv_qk_norm_rope_prep(qf.data_ptr(), q.data_ptr(), q.stride(0), *kp[:4], dtype_code(q.dtype), heads, kv_heads,
                                                 dim, vdim, q_w.data_ptr(), kp[4], int(bool(per_head)), float(eps),
                                                 0 if rope is None else rope.data_ptr(), int(rot_n if rope is not None else 0),
-                                                float(scale), kp[5], kp[6], batch.slot.data_ptr(), batch.pos.data_ptr(), T, self.code,
+                                                float(scale), kp[5], kp[6], batch.slot.data_ptr(), batch.pos.data_ptr(), T, *opt,
+                                                int(bool(halves)), 0 if head_scale is None else head_scale.data_ptr(), q_pad, self.code,
                                                 self._s()), "qk_norm_rope_prep")
         return qf
 
@@ -382,6 +392,94 @@ class HipOps:
                                            max(n for _, _, n in batch.items), width, self.code, self._s()), "min_gru_scan")
         return out
 
+    # ---- norm after the sum, convolved mixer input, talking-heads attention, retention operands -----------------------------------------
+    def embed_rms_norm(self, tokens, table, w, eps):
+        """-> float x [T, D] = rms_norm(table[tokens]) * w."""
+        T, D = tokens.numel(), table.size(1)
+        x = torch.empty((T, D), dtype=torch.float32, device=table.device)
+        self._need(tokens, table, w)
+        self.check(self.L.qsv_embed_rms_norm(x.data_ptr(), table.data_ptr(), tokens.data_ptr(), w.data_ptr(), float(eps), T, D, self.code,
+                                             self._s()), "embed_rms_norm")
+        return x
+
+    def residual_conv(self, x, conv_w, hist, batch):
+        """-> [T, D] (storage type): x plus its causal convolution over time with per-channel taps conv_w float [taps, D]; hist: two-copy
+        state, the last taps - 1 rows of x of every sequence (None with one tap)."""
+        T, D = x.shape
+        h = torch.empty((T, D), dtype=self.dtype, device=x.device)
+        self._need(x, conv_w, hist)
+        assert x.dtype == torch.float32 and conv_w.dtype == torch.float32 and conv_w.size(1) == D
+        assert conv_w.size(0) == 1 or (hist.dtype == torch.float32 and hist.shape[1:] == (conv_w.size(0) - 1, D))
+        self.check(self.L.qsv_residual_conv(h.data_ptr(), x.data_ptr(), conv_w.data_ptr(), conv_w.size(0), 0 if hist is None else hist.data_ptr(),
+                                            batch.run_off.data_ptr(), batch.state_rd.data_ptr(), batch.state_wr.data_ptr(), T, D, self.code,
+                                            self._s()), "residual_conv")
+        return h
+
+    def scaled_add_rms_norm(self, x, y, alpha, w, eps, then_conv=None, batch=None, want_h=True):
+        """x <- rms_norm(alpha x + y) * w in place; -> x in the storage type (None without want_h).  then_conv = (conv_w, hist): -> what
+        `residual_conv` makes of the new x, in the same launch (steps in which every run is one token)."""
+        T, D = x.shape
+        h = torch.empty((T, D), dtype=self.dtype, device=x.device) if want_h else None
+        self._need(x, y, w)
+        assert x.dtype == torch.float32 and y.shape == x.shape and y.dtype == self.dtype and w.dtype == self.dtype and w.numel() == D
+        c = [0, 0, 0, 0, 0]
+        if then_conv is not None:
+            conv_w, hist = then_conv
+            self._need(conv_w, hist)
+            assert want_h and all(n == 1 for _, _, n in batch.items) and conv_w.dtype == torch.float32 and conv_w.size(1) == D
+            assert conv_w.size(0) == 1 or (hist.dtype == torch.float32 and hist.shape[1:] == (conv_w.size(0) - 1, D))
+            c = [conv_w.data_ptr(), conv_w.size(0), 0 if hist is None else hist.data_ptr(), batch.state_rd.data_ptr(), batch.state_wr.data_ptr()]
+        self.check(self.L.qsv_scaled_add_rms_norm(x.data_ptr(), 0 if h is None else h.data_ptr(), y.data_ptr(), float(alpha), w.data_ptr(),
+                                                  float(eps), *c, T, D, self.code, self._s()), "scaled_add_rms_norm")
+        return h
+
+    def rotate_qk(self, qkv, heads, dim, vdim, rope, rot_n, batch):
+        """qkv [T, >= heads * (2 dim + vdim)] = [q | k | v ..] -> float [T, heads * (2 dim + vdim)] with the first rot_n dimensions of every
+        q and k head turned by the position (halves layout)."""
+        T = qkv.size(0)
+        out = torch.empty((T, heads * (2 * dim + vdim)), dtype=torch.float32, device=qkv.device)
+        self._need(rope, batch.pos)
+        assert qkv.stride(1) == 1 and qkv.dtype == self.dtype and (rope is None or rope.size(0) > batch.max_pos)
+        self.check(self.L.qsv_rotate_qk(out.data_ptr(), qkv.data_ptr(), qkv.stride(0), heads, dim, vdim, 0 if rope is None else rope.data_ptr(),
+                                        int(rot_n if rope is not None else 0), batch.pos.data_ptr(), T, self.code, self._s()), "rotate_qk")
+        return out
+
+    def talking_attention(self, qf, pool, batch, talk, gate, vdim, page, cap=0.0, window=None, variant=0, key_splits=None, decode=None):
+        """qf float [T, H, dim] (scaled queries), pool [G, rows, vdim + dim] -> [T, H * vdim]: softmax weights per head (scores soft-capped
+        by cap tanh(. / cap) if cap > 0), mixed over the heads by talk [H, H], on each head's own values; head h times sigmoid(gate[t,
+        h]) (gate [T, H], a column slice is fine, or None).  variant 1: always the wave kernel.  decode: whether a workgroup serves
+        the heads of several key pools (None: where the step's sequences bring few tokens)."""
+        T, H, dim = qf.shape
+        G, R = pool.size(0), pool.size(2)
+        self._need(qf, pool, batch.block_table, batch.seq, batch.pos, talk)
+        assert R == vdim + dim and H % G == 0 and qf.dtype == torch.float32 and pool.dtype == self.dtype and talk.shape == (H, H)
+        assert talk.dtype == self.dtype and (gate is None or (gate.dtype == self.dtype and gate.stride(1) == 1 and gate.shape == (T, H)))
+        out = torch.empty((T, H * vdim), dtype=self.dtype, device=qf.device)
+        bt = batch.block_table
+        splits, pm = 1, None
+        if variant == 0 and self.L.qsv_talking_attention_mfma_ok(dim, vdim, page, self.code):
+            if decode is None:
+                decode = T <= 2 * len(batch.items)
+            kp = self.L.qsv_talking_attention_key_pools(H, G, dim, int(decode))
+            tiles = batch.tiles(self.L.qsv_talking_attention_tile_tokens(H, G, kp))
+            groups = tiles.size(0) * (G // kp)
+            span = min(batch.max_pos + 1, int(window)) if window else batch.max_pos + 1
+            splits = max(1, min(self.attention_split_target // max(groups, 1), span // 128, 32)) if key_splits is None else key_splits
+            po = torch.empty((splits, T, H, G, vdim), dtype=torch.float32, device=qf.device)
+            pm = torch.empty((splits, T, H, 2), dtype=torch.float32, device=qf.device)
+            self.check(self.L.qsv_talking_attention_mfma(po.data_ptr(), pm.data_ptr(), qf.data_ptr(), pool.data_ptr(), bt.data_ptr(), bt.stride(0),
+                                                         batch.pos.data_ptr(), tiles.data_ptr(), tiles.size(0), int(window or 0), T, H, G, dim,
+                                                         vdim, page, pool.stride(0), float(cap), kp, splits, self._s()), "talking_attention_mfma")
+        else:
+            po = torch.empty((1, T, H, G, vdim), dtype=torch.float32, device=qf.device)
+            self.check(self.L.qsv_talking_attention(po.data_ptr(), qf.data_ptr(), pool.data_ptr(), bt.data_ptr(), bt.stride(0),
+                                                    batch.seq.data_ptr(), batch.pos.data_ptr(), int(window or 0), T, H, G, dim, vdim, page,
+                                                    pool.stride(0), float(cap), self.code, self._s()), "talking_attention")
+        self.check(self.L.qsv_talking_mix(out.data_ptr(), po.data_ptr(), 0 if pm is None else pm.data_ptr(), talk.data_ptr(),
+                                          0 if gate is None else gate.data_ptr(), 0 if gate is None else gate.stride(0), splits, T, H, G, vdim,
+                                          self.code, self._s()), "talking_mix")
+        return out
+
     # ---- recurrences ----------------------------------------------------------------------------------------------------------
     def decay(self, z, bias, a_log, tau, heads, dim):
         """z [T, heads * dim] (storage type; a column slice is fine) -> float decays: a_log given: exp(-exp(a_log[h]) softplus(z +
@@ -402,7 +500,8 @@ class HipOps:
         T = proj.size(0)
         C, taps = conv_w.shape
         out = torch.empty((T, C), dtype=torch.float32, device=proj.device)
-        self._need(proj, conv_w, hist)
+        self._need(conv_w, hist)
+        assert proj.is_cuda and proj.stride(1) == 1 and off + C <= proj.size(1)
         assert conv_w.dtype == torch.float32 and hist.dtype == torch.float32 and hist.size(-1) == C and proj.dtype == self.dtype
         assert hist.size(1) == max(taps - 1, 1)
         self.check(self.L.qsv_conv_silu_unit(out.data_ptr(), proj.data_ptr(), proj.stride(0), off, C, taps, conv_w.data_ptr(),
@@ -414,13 +513,14 @@ class HipOps:
     def recurrent_scan(self, q, k, v, decay, beta, state, batch, heads, qk_heads, dim, vdim, q_scale, kscale=None, v_cols=None):
         """q, k [T, qk_heads * dim], v [T, heads * vdim] (float or storage type, column slices are fine), decay float [T, heads *
         dim], beta [T, heads] raw (before the sigmoid) or None, state float [slots, heads, dim, vdim] -> o float [T, heads, vdim].
-        decay of shape [T, heads]: one factor per head.  kscale float [T, heads]: multiplies k where it enters the state.
+        decay of shape [T, heads]: one factor per head; of shape [heads]: the same for every token.  kscale float [T, heads]: multiplies k where it enters the state.
         v_cols < vdim: v is [T, heads * v_cols] and the state's column v_cols is fed with ones (a normaliser), the rest with zeros."""
         T = q.size(0)
         o = torch.empty((T, heads, vdim), dtype=torch.float32, device=q.device)
         self._need(decay, state, kscale)
         assert q.dtype == k.dtype == v.dtype and q.stride(1) == k.stride(1) == v.stride(1) == 1
-        head_decay = decay.shape == (T, heads) and dim != 1
+        head_decay = 2 if decay.dim() == 1 else int(decay.shape == (T, heads) and dim != 1)
+        assert decay.dtype == torch.float32 and (decay.dim() != 1 or decay.numel() == heads)
         assert state.shape[1:] == (heads, dim, vdim) and state.dtype == torch.float32 and (head_decay or decay.shape == (T, heads * dim))
         assert kscale is None or (kscale.dtype == torch.float32 and kscale.shape == (T, heads))
         assert v.size(1) == heads * (v_cols or vdim)
@@ -430,7 +530,7 @@ class HipOps:
                                              0 if beta is None else beta.data_ptr(), 0 if beta is None else beta.stride(0),
                                              0 if beta is None else dtype_code(beta.dtype), state.data_ptr(), runs.data_ptr(),
                                              runs.size(0), max(n for _, _, n in batch.items), heads, qk_heads, dim, vdim,
-                                             float(q_scale), 0 if kscale is None else kscale.data_ptr(), int(head_decay),
+                                             float(q_scale), 0 if kscale is None else kscale.data_ptr(), head_decay,
                                              int(v_cols or 0), self._s()), "recurrent_scan")
         return o
 
@@ -641,7 +741,7 @@ class TorchOps:
         return (torch.cat([q_abs.transpose(0, 1).float(), qr], dim=-1) * scale).contiguous()
 
     def latent_attention(self, qf, pool, batch, window, rank, page, variant=0, key_splits=None, q_first=0, chunk=None, bias=None,
-                         keep_first=0, sink=None, pooled=None, pool_block=0):
+                         keep_first=0, sink=None, pooled=None, pool_block=0, slopes=None):
         T, H, R = qf.shape
         block_table, seq, pos = batch.block_table, batch.seq, batch.pos
         out = torch.empty((T, H, rank), dtype=self.dtype, device=qf.device)
@@ -665,6 +765,8 @@ class TorchOps:
                 s = qf[t, hs] @ rows.t()                                             # [per, n]
                 if bias is not None:
                     s = s + bias[hs][:, (p - j).clamp(max=bias.size(1) - 1)]
+                if slopes is not None:
+                    s = s - slopes[hs, None] * (p - j).float()
                 if extra is not None:                                                # blocks wholly before the window
                     first = torch.arange(max(0, p - window + 1) // pool_block, device=qf.device) * pool_block
                     more = extra[g][bt[int(seq[t]), first // page] * per_page + (first % page) // pool_block].float()
@@ -741,17 +843,26 @@ class TorchOps:
         a.copy_((torch.relu(a.float()) ** 2).to(a.dtype))
         return a
 
-    def qk_norm_rope_prep(self, q, k, v, heads, kv_heads, dim, vdim, q_w, k_w, per_head, eps, rope, rot_n, scale, pool, batch):
+    def qk_norm_rope_prep(self, q, k, v, heads, kv_heads, dim, vdim, q_w, k_w, per_head, eps, rope, rot_n, scale, pool, batch,
+                          q_b=None, k_b=None, v_b=None, halves=False, head_scale=None, q_pad=None):
         T = q.size(0)
+
+        def biased(u, b):
+            return u.float() if b is None else u.float() + b.float()
 
         def prep(u, w, n):
             u = self._rms(u.reshape(T, n, dim), w, eps) if per_head else self._rms(u, w, eps).view(T, n, dim)
-            return u if rope is None else _rotate(u, rope, batch.pos, rot_n)
+            if rope is None:
+                return u
+            return self._rotate_halves(u, rope, batch.pos, rot_n) if halves else _rotate(u, rope, batch.pos, rot_n)
 
         if k is not None:
-            rows = torch.cat([v.float().reshape(T, kv_heads, vdim), prep(k, k_w, kv_heads)], dim=-1)
+            rows = torch.cat([biased(v, v_b).reshape(T, kv_heads, vdim), prep(biased(k, k_b), k_w, kv_heads)], dim=-1)
             pool[:, batch.slot] = rows.transpose(0, 1).to(self.dtype)
-        return torch.cat([torch.zeros(T, heads, vdim, device=q.device), prep(q, q_w, heads) * scale], dim=-1).contiguous()
+        out = prep(biased(q, q_b), q_w, heads) * scale
+        if head_scale is not None:
+            out = out * head_scale[:, None]
+        return torch.cat([torch.zeros(T, heads, vdim if q_pad is None else q_pad, device=q.device), out], dim=-1).contiguous()
 
     def pool_blocks(self, pool, pooled, batch, block, page):
         per_page = (page + block - 1) // block
@@ -778,6 +889,51 @@ class TorchOps:
                 out[t] = S
             state[slot] = S
         return (out * g * torch.sigmoid(g)).to(self.dtype)
+
+    # ---- norm after the sum, convolved mixer input, talking-heads attention, retention operands -----------------------------------------
+    def embed_rms_norm(self, tokens, table, w, eps):
+        return self._rms(table[tokens.long()], w, eps)
+
+    def residual_conv(self, x, conv_w, hist, batch):
+        taps = conv_w.size(0)
+        out = torch.empty_like(x)
+        for slot, first, cnt in batch.items:
+            rd, wr = int(batch.state_rd[first]), int(batch.state_wr[first + cnt - 1])
+            past = hist[rd] if rd >= 0 and taps > 1 else torch.zeros((taps - 1, x.size(1)), device=x.device)
+            seq = torch.cat([past, x[first:first + cnt]])
+            out[first:first + cnt] = x[first:first + cnt] + sum(seq[j:j + cnt] * conv_w[j] for j in range(taps))
+            if taps > 1:
+                hist[wr] = seq[cnt:]
+        return out.to(self.dtype)
+
+    def scaled_add_rms_norm(self, x, y, alpha, w, eps, then_conv=None, batch=None, want_h=True):
+        x.copy_(self._rms(alpha * x + y.float(), w, eps))
+        if then_conv is not None:
+            return self.residual_conv(x, then_conv[0], then_conv[1], batch)
+        return x.to(self.dtype) if want_h else None
+
+    def rotate_qk(self, qkv, heads, dim, vdim, rope, rot_n, batch):
+        T = qkv.size(0)
+        qk, v = qkv[:, :2 * heads * dim].float().reshape(T, 2 * heads, dim), qkv[:, 2 * heads * dim:heads * (2 * dim + vdim)].float()
+        if rope is not None:
+            qk = self._rotate_halves(qk, rope, batch.pos, rot_n)
+        return torch.cat([qk.reshape(T, 2 * heads * dim), v], dim=-1)
+
+    def talking_attention(self, qf, pool, batch, talk, gate, vdim, page, cap=0.0, window=None, variant=0, key_splits=None, decode=None):
+        T, H, dim = qf.shape
+        G = pool.size(0)
+        per, bt = H // G, batch.block_table.long()
+        out = torch.empty((T, H, vdim), dtype=torch.float32, device=qf.device)
+        for t in range(T):
+            p = int(batch.pos[t])
+            j = torch.arange(max(0, p - int(window) + 1) if window else 0, p + 1, device=qf.device)
+            rows = pool[:, bt[int(batch.seq[t]), j // page] * page + j % page].float()                # [G, n, R]
+            s = torch.cat([qf[t, g * per:(g + 1) * per] @ rows[g, :, vdim:].t() for g in range(G)])       # [H, n]
+            w = talk.float() @ torch.softmax(cap * torch.tanh(s / cap) if cap > 0 else s, dim=-1)
+            out[t] = torch.cat([w[g * per:(g + 1) * per] @ rows[g, :, :vdim] for g in range(G)])
+        if gate is not None:
+            out = out * torch.sigmoid(gate.float())[:, :, None]
+        return out.reshape(T, H * vdim).to(self.dtype)
 
     # ---- recurrences ----------------------------------------------------------------------------------------------------------
     def decay(self, z, bias, a_log, tau, heads, dim):
@@ -818,7 +974,9 @@ class TorchOps:
             ones = torch.zeros((T, heads, vdim - v_cols), device=q.device)
             ones[..., 0] = 1.0
             vf = torch.cat([vf, ones], dim=-1)
-        g = decay[:, :, None].expand(T, heads, dim) if decay.shape == (T, heads) and dim != 1 else decay.view(T, heads, dim)
+        if decay.dim() == 1:
+            decay = decay.expand(T, heads)
+        g = decay[:, :, None].expand(T, heads, dim) if decay.shape == (T, heads) and dim != 1 else decay.reshape(T, heads, dim)
         bt = None if beta is None else torch.sigmoid(beta.float())
         o = torch.empty((T, heads, vdim), dtype=torch.float32, device=q.device)
         for slot, first, cnt in batch.items:

@@ -1,8 +1,9 @@
-"""Rotary position tables: plain, with YaRN frequency scaling, or with piecewise (wavelength-band) frequency scaling.
+"""Rotary position tables: plain, with linear or YaRN frequency scaling, or with piecewise (wavelength-band) frequency scaling.
 
 Rotation of pair i at position p by the angle a = p * f_i: (u cos a - v sin a, v cos a + u sin a), f_i = base^(-2i / dims).
 Which two dimensions form pair i is the kernels' business (neighbours 2i, 2i + 1, or halves i, i + dims / 2): the table holds
-cos and sin per (position, pair) and serves both.  With scaling {factor, original, fast, slow} (YaRN): the
+cos and sin per (position, pair) and serves both.  With scaling {factor} (linear): every f_i is divided by factor.  With scaling
+{factor, original, fast, slow} (YaRN): the
 dimension at which a wave makes t turns over the original context is c(t) = dims * ln(original / (2 pi t)) / (2 ln base);
 between lo = max(floor(c(fast)), 0) and hi = min(ceil(c(slow)), dims - 1) a linear ramp r_i blends the interpolated
 frequency f_i / factor (r = 1) with the plain one (r = 0), and cos and sin carry the magnitude 0.1 ln(factor) + 1.
@@ -40,6 +41,8 @@ class RotaryTable:
                     s = (orig / wavelength - low) / (high - low)
                     out.append((1.0 - s) * fi / factor + s * fi)
             f = torch.tensor(out, dtype=torch.float64)
+        elif scaling and "original" not in scaling:
+            f = f / float(scaling["factor"])
         elif scaling:
             factor, orig = float(scaling["factor"]), float(scaling["original"])
 

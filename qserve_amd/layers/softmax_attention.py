@@ -11,7 +11,8 @@ the softmax-weighted sum of the rows' first vdim elements is the output; one lau
 
 `NormedChunkAttention` is the position-free sibling on the same cache rows and kernel: queries and keys are RMS-normed over the
 whole projection, positions enter through a learned bias per (distance bucket, head) and through chunks that bound what a query
-sees, and the values may be blended with those an earlier layer computed for the same token.
+sees, and the values may be blended with those an earlier layer computed for the same token.  `SinkWindowAttention` is the windowed
+sibling with a sink, `TalkingHeadsAttention` the one whose weights are mixed across heads.
 """
 import math
 
@@ -135,14 +136,20 @@ class SinkWindowAttention:
       before i - window: the means of the block's cached keys and values (a second pool, ceil(page / P) rows per page, held by
       the page of the block's first position).
     * shared_kv: the layer has no keys and values of its own and reads the pools of another layer of the same head counts.
+    * tied_values: the layer has no value projection, a value is the projected key before its norm and rotation (vdim = dim).
+    * slopes (a number per head): slopes[h] * (i - j) is taken off the score of query i and key j (the sink gets none).
     Cache: per key / value head one pool of rows [v | k] (k after norm and rotation), as the row-attention kernels read them."""
 
     def __init__(self, ops, *, heads, kv_heads, dim, vdim, scale, eps, window, weights, norm="head", taps=None, rotary=None,
-                 keep_first=0, pool_block=None, shared_kv=False, page=64):
-        """weights: q [H dim, D], o [D, H vdim], q_norm, sink [H]; unless shared_kv: k [G dim, D], v [G vdim, D], k_norm; with
-        taps: q_conv [H dim, taps], k_conv, v_conv."""
+                 keep_first=0, pool_block=None, shared_kv=False, tied_values=False, slopes=None, page=64):
+        """weights: q [H dim, D], o [D, H vdim], q_norm, sink [H]; unless shared_kv: k [G dim, D], k_norm and, unless tied_values, v
+        [G vdim, D]; with taps: q_conv [H dim, taps], k_conv, v_conv."""
         if heads % kv_heads or norm not in ("head", "all") or not window or int(window) < 1:
             raise ValueError(f"attention: {heads} heads over {kv_heads}, norm {norm!r}, window {window}")
+        if tied_values and (shared_kv or taps or vdim != dim):
+            raise ValueError("attention: values tied to the keys need keys of their own, no convolution and vdim = dim")
+        if slopes is not None and (len(slopes) != heads or pool_block):
+            raise ValueError("attention: distance slopes are one per head and exclude pooled blocks")
         if shared_kv and (taps or pool_block):
             raise ValueError("attention: a layer that reads another layer's keys and values has no convolution or pooled blocks")
         if pool_block and keep_first:
@@ -159,13 +166,17 @@ class SinkWindowAttention:
         D = w["q"].size(1)
         expect = {"q": (heads * dim, D), "o": (D, heads * vdim), "sink": (heads,), "q_norm": (dim if self.per_head else heads * dim,)}
         if not shared_kv:
-            expect.update(k=(kv_heads * dim, D), v=(kv_heads * vdim, D), k_norm=(dim if self.per_head else kv_heads * dim,))
+            expect.update(k=(kv_heads * dim, D), k_norm=(dim if self.per_head else kv_heads * dim,))
+            if not tied_values:
+                expect.update(v=(kv_heads * vdim, D))
         if self.taps:
             expect.update(q_conv=(heads * dim, self.taps), k_conv=(kv_heads * dim, self.taps), v_conv=(kv_heads * vdim, self.taps))
         for k, shp in expect.items():
             if tuple(w[k].shape) != shp:
                 raise ValueError(f"attention weight {k}: shape {tuple(w[k].shape)}, expected {shp}")
-        self.w_in = (w["q"] if shared_kv else torch.cat([w["q"], w["k"], w["v"]], dim=0)).contiguous()
+        self.tied = bool(tied_values)
+        self.w_in = torch.cat([w["q"]] + ([] if shared_kv else [w["k"]] if tied_values else [w["k"], w["v"]]), dim=0).contiguous()
+        self.slopes = None if slopes is None else torch.tensor([float(v) for v in slopes], dtype=torch.float32, device=w["q"].device)
         self.w_o, self.q_norm, self.k_norm = w["o"].contiguous(), w["q_norm"].contiguous(), None if shared_kv else w["k_norm"].contiguous()
         self.sink = w["sink"].float().contiguous()
         self.conv = torch.cat([w["q_conv"], w["k_conv"], w["v_conv"]], dim=0).float().contiguous() if self.taps else None
@@ -190,6 +201,8 @@ class SinkWindowAttention:
             proj = proj.float() * self.conv[:, 0]
         q = proj[:, :H * d]
         k, v = (None, None) if self.shared_kv else (proj[:, H * d:(H + G) * d], proj[:, (H + G) * d:])
+        if self.tied:
+            v = k
         rope = self.rotary.reserve(batch.max_pos + 1) if self.rotary is not None else None
         pool = pools[0]
         qf = ops.qk_norm_rope_prep(q, k, v, H, G, d, dv, self.q_norm, self.k_norm, self.per_head, self.eps, rope,
@@ -199,5 +212,55 @@ class SinkWindowAttention:
             pooled = pools[1]
             ops.pool_blocks(pool, pooled, batch, self.pool_block, self.page)
         o = ops.latent_attention(qf, pool, batch, self.window, dv, self.page, q_first=dv, keep_first=self.keep_first, sink=self.sink,
-                                 pooled=pooled, pool_block=self.pool_block or 0)
+                                 slopes=self.slopes, pooled=pooled, pool_block=self.pool_block or 0)
         return linear(o.view(T, H * dv), self.w_o)
+
+
+def distance_slopes(heads):
+    """Slopes 2^(-8 (h + 1) / heads) of a linear distance bias."""
+    return [2.0 ** (-8.0 * (h + 1) / heads) for h in range(heads)]
+
+
+class TalkingHeadsAttention:
+    """Causal grouped-query attention with tied values whose softmax weights talk across heads.
+
+    q (H heads), k (G heads; head h reads key / value head h // (H / G)) have biases; a value is the projected key.  q and k are RMS-
+    normed per head (weights [dim], shared by the heads), then their first rotary.dims dimensions turn with the position (halves
+    layout).  score = q . k * scale * temp_h, soft-capped by softcap tanh(. / softcap) (softcap None: not); softmax over j <= i per head;
+    the heads' weights are mixed, w_h <- sum_g talk[h, g] w_g, and meet the values of head h's own pool; head h's output is multiplied
+    by sigmoid(W_g h)_h.  Cache: per key / value head one pool of rows [v | k] (k after norm and rotation)."""
+
+    takes_projection = True
+
+    def __init__(self, ops, *, heads, kv_heads, dim, scale, softcap, rotary, eps, weights, page=64):
+        """weights: q [H dim, D], q_b, k [G dim, D], k_b, q_norm, k_norm [dim], temp [H], talk [H, H], g [H, D], o [D, H dim]."""
+        if heads % kv_heads or (softcap is not None and not float(softcap) > 0.0):
+            raise ValueError(f"talking-heads attention: {heads} heads over {kv_heads}, soft cap {softcap}")
+        if rotary is not None and rotary.dims > dim:
+            raise ValueError(f"talking-heads attention: {rotary.dims} rotated dimensions in heads of {dim}")
+        self.ops, self.H, self.G, self.dim, self.scale, self.eps, self.page = ops, heads, kv_heads, dim, float(scale), float(eps), page
+        self.cap, self.rotary = float(softcap or 0.0), rotary
+        w = weights
+        D = w["q"].size(1)
+        for k, shp in {"q": (heads * dim, D), "q_b": (heads * dim,), "k": (kv_heads * dim, D), "k_b": (kv_heads * dim,), "q_norm": (dim,),
+                       "k_norm": (dim,), "temp": (heads,), "talk": (heads, heads), "g": (heads, D), "o": (D, heads * dim)}.items():
+            if tuple(w[k].shape) != shp:
+                raise ValueError(f"talking-heads attention weight {k}: shape {tuple(w[k].shape)}, expected {shp}")
+        from .recurrent import pad_rows
+        self.w_in, self.w_o = pad_rows(torch.cat([w["q"], w["k"], w["g"]], dim=0)), w["o"].contiguous()
+        self.q_b, self.k_b, self.q_norm, self.k_norm = (w[k].contiguous() for k in ("q_b", "k_b", "q_norm", "k_norm"))
+        self.temp, self.talk = w["temp"].float().contiguous(), w["talk"].contiguous()
+        self.cache_rows, self.state_specs = [(kv_heads, 2 * dim)], []
+
+    def __call__(self, h, batch, pools, states, proj=None):
+        """proj: h's product with w_in, where the caller has it already (a column slice is fine)."""
+        ops, H, G, d, pool = self.ops, self.H, self.G, self.dim, pools[0]
+        if proj is None:
+            proj = linear(h, self.w_in)
+        o_k, o_g = H * d, (H + G) * d
+        k = proj[:, o_k:o_g]
+        rope = self.rotary.reserve(batch.max_pos + 1) if self.rotary is not None else None
+        qf = ops.qk_norm_rope_prep(proj[:, :o_k], k, k, H, G, d, d, self.q_norm, self.k_norm, True, self.eps, rope,
+                                   self.rotary.dims if rope is not None else 0, self.scale, pool, batch, q_b=self.q_b, k_b=self.k_b,
+                                   v_b=self.k_b, halves=True, head_scale=self.temp, q_pad=0)
+        return linear(ops.talking_attention(qf, pool, batch, self.talk, proj[:, o_g:o_g + H], d, self.page, cap=self.cap), self.w_o)

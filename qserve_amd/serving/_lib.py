@@ -18,12 +18,22 @@ SIGNATURES = {
     "qsv_latent_prep": (_i, [_vp, _i64, _i, _i, _vp, _vp, _i, _i, _vp, _i, _i, _vp, _vp, _vp, _vp, _f, _i, _i, _vp]),
     "qsv_latent_query": (_i, [_vp, _vp, _vp, _vp, _vp, _f, _i, _i, _i, _i, _i, _i, _i, _vp]),
     "qsv_latent_attention": (_i, [_vp, _vp, _vp, _vp, _i, _vp, _vp, _i, _i, _i, _i, _i, _i, _i, _i64, _i, _vp, _i, _i, _vp, _vp, _i64, _i, _i,
-                                  _i, _i, _vp]),
+                                  _vp, _i, _i, _vp]),
     "qsv_pool_blocks": (_i, [_vp, _i64, _vp, _i64, _vp, _i, _vp, _vp, _i, _i, _i, _i, _i, _i, _i, _vp]),
     "qsv_latent_attention_tile_tokens": (_i, [_i]),
     "qsv_latent_attention_mfma_ok": (_i, [_i, _i, _i]),
     "qsv_latent_attention_mfma": (_i, [_vp, _vp, _vp, _vp, _i, _vp, _vp, _i, _i, _i, _i, _i, _i, _i, _vp, _vp, _i, _i, _i, _i64, _i, _vp,
-                                       _i, _i, _vp, _vp, _i64, _i, _i, _vp]),
+                                       _i, _i, _vp, _vp, _i64, _i, _i, _vp, _vp]),
+    "qsv_talking_attention_key_pools": (_i, [_i, _i, _i, _i]),
+    "qsv_talking_attention_tile_tokens": (_i, [_i, _i, _i]),
+    "qsv_talking_attention_mfma_ok": (_i, [_i, _i, _i, _i]),
+    "qsv_talking_attention": (_i, [_vp, _vp, _vp, _vp, _i, _vp, _vp, _i, _i, _i, _i, _i, _i, _i, _i64, _f, _i, _vp]),
+    "qsv_talking_attention_mfma": (_i, [_vp, _vp, _vp, _vp, _vp, _i, _vp, _vp, _i, _i, _i, _i, _i, _i, _i, _i, _i64, _f, _i, _i, _vp]),
+    "qsv_talking_mix": (_i, [_vp, _vp, _vp, _vp, _vp, _i64, _i, _i, _i, _i, _i, _i, _vp]),
+    "qsv_embed_rms_norm": (_i, [_vp, _vp, _vp, _vp, _f, _i, _i, _i, _vp]),
+    "qsv_residual_conv": (_i, [_vp, _vp, _vp, _i, _vp, _vp, _vp, _vp, _i, _i, _i, _vp]),
+    "qsv_scaled_add_rms_norm": (_i, [_vp, _vp, _vp, _f, _vp, _f, _vp, _i, _vp, _vp, _vp, _i, _i, _i, _vp]),
+    "qsv_rotate_qk": (_i, [_vp, _vp, _i64, _i, _i, _i, _vp, _i, _vp, _i, _i, _vp]),
     "qsv_sigmoid_gate": (_i, [_vp, _vp, _i64, _i, _i, _i, _vp]),
     "qsv_moe_route": (_i, [_vp, _vp, _vp, _vp, _vp, _i, _i, _i, _i, _i, _i, _i, _i, _vp, _i, _f, _i, _vp]),
     "qsv_moe_up": (_i, [_vp, _vp, _vp, _vp, _i, _i, _i, _i, _i, _f, _i, _i, _vp]),
@@ -46,7 +56,7 @@ SIGNATURES = {
     "qsv_min_gru_scan": (_i, [_vp, _vp, _i64, _i, _i, _i, _vp, _vp, _vp, _vp, _i, _i, _i, _i, _vp]),
     "qsv_add_normed_rms_norm": (_i, [_vp, _vp, _vp, _vp, _i, _vp, _i, _f, _i, _i, _i, _vp]),
     "qsv_qk_norm_rope_prep": (_i, [_vp, _vp, _i64, _vp, _i64, _vp, _i64, _i, _i, _i, _i, _i, _vp, _vp, _i, _f, _vp, _i, _f, _vp, _i64,
-                                   _vp, _vp, _i, _i, _vp]),
+                                   _vp, _vp, _i, _vp, _vp, _vp, _i, _vp, _i, _i, _vp]),
     "qsv_recurrent_scan": (_i, [_vp, _vp, _i64, _vp, _i64, _vp, _i64, _i, _vp, _vp, _i64, _i, _vp, _vp, _i, _i, _i, _i, _i, _i, _f, _vp,
                                 _i, _i, _vp]),
     "qsv_head_rms_gate": (_i, [_vp, _vp, _vp, _vp, _i64, _i, _f, _i, _i, _i, _i, _i, _vp, _i, _vp]),

@@ -96,11 +96,11 @@ def test_serve_argument_validation_without_gpu():
     assert L.qsv_moe_route(1, 1, 1, 1, None, 0, 4, 64, 8, 3, 4, 1, 0, None, 1, 1.0, 0, None) == 1  # top 3 of one kept group of 2
     assert b"experts" in L.qsv_last_error()
     assert L.qsv_moe_route(1, 1, 1, 1, None, 0, 4, 64, 8, 2, 4, 1, 2, None, 1, 1.0, 0, None) == 1  # unknown score function
-    assert L.qsv_latent_attention(1, 1, 1, 1, 4, 1, 1, 0, 4, 2, 1000, 1032, 64, 2, 0, 0, None, 0, 0, None, None, 0, 0, 0, 0, 1, None) == 1   # rows wider than 1024
-    assert L.qsv_latent_attention(1, 1, 1, 1, 4, 1, 1, 0, 4, 2, 64, 96, 64, 2, 0, -3, None, 0, 0, None, None, 0, 0, 0, 0, 1, None) == 1      # negative chunk
-    assert L.qsv_latent_attention(1, 1, 1, 1, 4, 1, 1, 0, 4, 2, 64, 96, 64, 2, 0, 0, 1, 0, 0, None, None, 0, 0, 0, 0, 1, None) == 1          # bias table without entries
-    assert L.qsv_latent_attention(1, 1, 1, 1, 4, 1, 1, 0, 4, 2, 64, 96, 64, 2, 0, 0, None, 0, 5, None, None, 0, 0, 0, 0, 1, None) == 1      # kept first positions without a window
-    assert L.qsv_latent_attention(1, 1, 1, 1, 4, 1, 1, 32, 4, 2, 64, 96, 64, 2, 0, 0, None, 0, 0, None, 1, 0, 12, 5, 0, 1, None) == 1       # five block rows of 12 positions do not cover a page of 64
+    assert L.qsv_latent_attention(1, 1, 1, 1, 4, 1, 1, 0, 4, 2, 1000, 1032, 64, 2, 0, 0, None, 0, 0, None, None, 0, 0, 0, None, 0, 1, None) == 1   # rows wider than 1024
+    assert L.qsv_latent_attention(1, 1, 1, 1, 4, 1, 1, 0, 4, 2, 64, 96, 64, 2, 0, -3, None, 0, 0, None, None, 0, 0, 0, None, 0, 1, None) == 1      # negative chunk
+    assert L.qsv_latent_attention(1, 1, 1, 1, 4, 1, 1, 0, 4, 2, 64, 96, 64, 2, 0, 0, 1, 0, 0, None, None, 0, 0, 0, None, 0, 1, None) == 1          # bias table without entries
+    assert L.qsv_latent_attention(1, 1, 1, 1, 4, 1, 1, 0, 4, 2, 64, 96, 64, 2, 0, 0, None, 0, 5, None, None, 0, 0, 0, None, 0, 1, None) == 1      # kept first positions without a window
+    assert L.qsv_latent_attention(1, 1, 1, 1, 4, 1, 1, 32, 4, 2, 64, 96, 64, 2, 0, 0, None, 0, 0, None, 1, 0, 12, 5, None, 0, 1, None) == 1       # five block rows of 12 positions do not cover a page of 64
     assert b"pooled" in L.qsv_last_error()
     assert L.qsv_latent_attention_mfma_ok(64, 80, 0) == 1 and L.qsv_latent_attention_mfma_ok(64, 80, 1) == 0
     assert L.qsv_latent_attention_mfma_ok(70, 70, 0) == 0
@@ -117,8 +117,18 @@ def test_serve_argument_validation_without_gpu():
     assert L.qsv_moe_up(1, 1, 1, 1, 1, 1, 8, 7, 2, 0.0, 4, 0, None) == 1                                      # gated units, odd rows
     assert L.qsv_moe_up(1, 1, 1, 1, 1, 1, 8, 8, 3, 0.0, 4, 0, None) == 1                                      # clamped units without a limit
     assert L.qsv_add_normed_rms_norm(1, 1, 1, None, 0, 1, 0, 1e-5, 2, 8, 0, None) == 1                        # an added sublayer output without its gain
-    assert L.qsv_qk_norm_rope_prep(1, 1, 64, None, 0, None, 0, 0, 2, 1, 32, 32, 1, None, 1, 1e-5, 1, 40, 1.0, None, 0, None, 1, 2, 0, None) == 1   # 40 rotated dimensions of 32
+    assert L.qsv_qk_norm_rope_prep(1, 1, 64, None, 0, None, 0, 0, 2, 1, 32, 32, 1, None, 1, 1e-5, 1, 40, 1.0, None, 0, None, 1, 2, None, None, None, 0, None, 32, 0, None) == 1   # 40 rotated dimensions of 32
     assert L.qsv_min_gru_scan(1, 1, 16, 0, 8, 16, 1, 1, 1, 1, 1, 1, 8, 0, None) == 1                            # the gate's columns lie outside the rows
+    assert L.qsv_latent_attention(1, 1, 1, 1, 4, 1, 1, 32, 4, 2, 64, 96, 64, 2, 0, 0, None, 0, 0, None, 1, 0, 16, 4, 1, 0, 1, None) == 1     # distance slopes with pooled blocks
+    assert [L.qsv_talking_attention_key_pools(*a) for a in ((8, 4, 64, 0), (8, 4, 64, 1), (32, 8, 128, 1), (32, 1, 64, 1))] == [1, 4, 4, 1]
+    assert [L.qsv_talking_attention_tile_tokens(*a) for a in ((8, 4, 1), (8, 4, 4), (40, 1, 1))] == [32, 8, 4]
+    assert L.qsv_talking_attention(1, 1, 1, 1, 4, 1, 1, 0, 4, 3, 2, 64, 64, 64, 0, 0.0, 0, None) == 1          # 3 heads over 2
+    assert L.qsv_talking_attention(1, 1, 1, 1, 4, 1, 1, 0, 4, 2, 2, 520, 64, 64, 0, 0.0, 0, None) == 1         # heads of 520 elements
+    assert L.qsv_talking_attention_mfma(1, 1, 1, 1, 1, 4, 1, 1, 1, 0, 4, 4, 4, 64, 64, 64, 0, 0.0, 3, 1, None) == 1     # 4 pools in groups of 3
+    assert L.qsv_talking_mix(1, 1, None, 1, None, 0, 2, 4, 4, 2, 64, 0, None) == 1                             # two key splits without their maxima
+    assert L.qsv_residual_conv(1, 1, 1, 3, None, 1, 1, 1, 2, 8, 0, None) == 1                                  # three taps without a history
+    assert L.qsv_scaled_add_rms_norm(1, None, 1, 2.0, 1, 1e-5, 1, 3, 1, 1, 1, 2, 8, 0, None) == 1              # a convolution without its output
+    assert L.qsv_rotate_qk(1, 1, 64, 2, 8, 8, 1, 10, 1, 2, 0, None) == 1                                       # 10 rotated dimensions of 8
     with pytest.raises(RuntimeError):
         check(L.qsv_embed(0, 1, 1, 1, 1, 8, 0, None), "embed")
 
@@ -128,6 +138,6 @@ def test_serving_package_does_not_need_the_w4a8_library():
     the serving kernels."""
     import subprocess
     import sys
-    code = ("import sys; import qserve_amd.serving, qserve_amd.models.vekalorn, qserve_amd.models.mumelix, qserve_amd.models.vepolix, qserve_amd.models.pemolorn, qserve_amd.serving.trace; "
+    code = ("import sys; import qserve_amd.serving, qserve_amd.models.vekalorn, qserve_amd.models.mumelix, qserve_amd.models.vepolix, qserve_amd.models.pemolorn, qserve_amd.models.sagupel, qserve_amd.serving.trace; "
             "bad = [m for m in sys.modules if m in ('qserve_amd._lib', 'qserve_amd.decode', 'qserve_backend')]; sys.exit(1 if bad else 0)")
     assert subprocess.run([sys.executable, "-c", code], cwd=ROOT).returncode == 0
