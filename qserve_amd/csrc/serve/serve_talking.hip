@@ -1,11 +1,13 @@
 // serve_talking.hip -- talking-heads attention over the paged cache: every head's softmax weights are mixed with the other heads'
 // before they meet the values,  out_h = sum_j (sum_g talk[h, g] w_g(j)) v_kv(h)(j).
 //
-// The mix is linear, so it is applied AFTER the sum over the keys: for every head g and every value pool k
+// Two forms.  Weights mixed before the sum ("two passes", up to 32 heads of up to 128 elements, bfloat16): the first launch finds every
+// head's maximum and sum, the second computes the scores again, normalises, mixes the heads' weights on the matrix cores and
+// multiplies each head's own values.  Its result is final but for the sum over key splits.
+//
+// Any sizes: the mix is linear, so it can come AFTER the sum over the keys, at the price of every head summing every pool's values:
 //   A[g, k] = sum_j w_g(j) v_k(j)           out_h = gate_h sum_g talk[h, g] A[g, kv(h)]
-// A score is computed once (its two exponentials are the dearest part of a visible pair: the soft cap's and the softmax's), no
-// weight ever leaves the registers, and contexts cut over workgroups merge as usual.  A is float; the last kernel merges the key
-// splits, normalises, mixes and gates in one pass.
+// A is float; the last kernel merges the key splits, normalises, mixes and gates in one pass.
 //
 // Scores: (qf . k), qf already scaled; cap > 0: cap tanh(. / cap).  With 0 < cap <= FIXED_CAP every score lies in [-cap, cap] and `cap`
 // itself serves as the softmax's maximum: no running maximum, no rescaling (e^(-2 cap) stays a normal float).
@@ -432,6 +434,329 @@ __global__ __launch_bounds__(NT) void talking_mix_kernel(T* __restrict__ out, co
     }
 }
 
+// ---- two passes: statistics, then mixed weights times values (matrix cores, bfloat16 storage) ----------------------------------------
+// A workgroup of eight waves serves a tile of up to 16 consecutive tokens of one sequence and ALL heads; wave w owns heads w HW .. +HW - 1.
+// Tiles of 32 keys; per tile
+//   scores   S^T = K Q^T per head, 16 keys at a time: A = key rows straight from the cache (registers, shared by the wave's heads of one
+//            pool; the next 16 rows are requested before the exponentials of these), B = the head's queries (registers)
+//   weights  e^(score) / sum from the first pass's (maximum, sum), as float16 times 2^10, to LDS as [key][token][head]
+//   mix      wave w takes four keys: talk [H x H] (A) times the weights of 16 tokens (B, contraction over the heads), result as
+//            bfloat16 to LDS as [head][token][key]
+//   values   O^T += V^T W^T per head: B = the mixed weights, A = the wave's value tile - copied straight into LDS of the wave's own
+//            while the scores are computed, transposed as it is read
+// two barriers a tile.  STATS: scores and sums only, no LDS.
+typedef _Float16 h8 __attribute__((ext_vector_type(8)));
+typedef _Float16 h4 __attribute__((ext_vector_type(4)));
+typedef __attribute__((address_space(1))) const void* gptr_t;
+typedef __attribute__((address_space(3))) void* lptr_t;
+constexpr int TT = 16;             // tokens of a tile
+constexpr int TW = 8;              // waves
+constexpr float LOG2E = 1.4426950408889634f;
+__host__ __device__ constexpr int two_pass_gk(int hw) { return TW * hw > 16 ? 32 : 16; }     // heads the mix contracts over, padded
+__host__ __device__ constexpr int two_pass_lds(int hw, int dt) {
+    return TW * dt * 2048 + 2 * (BN * TT * two_pass_gk(hw) + two_pass_gk(hw) * TT * BN);
+}
+
+template <int HW, int DT, bool STATS>
+__global__ __launch_bounds__(64 * TW, 2) void talking_two_pass_kernel(
+    bf16_t* __restrict__ out, float* __restrict__ part_o, float* __restrict__ part_ml, int Z1, const float* __restrict__ qf,
+    const bf16_t* __restrict__ pool, const int32_t* __restrict__ block_table, int table_stride, const int32_t* __restrict__ pos,
+    const int32_t* __restrict__ tiles, int window, int H, int G, int dim, int page, int64_t pool_stride, float cap,
+    const bf16_t* __restrict__ talk, const bf16_t* __restrict__ gate, int64_t gate_stride, int n_tokens) {
+    constexpr int GK = two_pass_gk(HW), HT = GK / 16, NV = 2 * DT, CT = 2 * DT, KPW = BN / TW;
+    extern __shared__ __attribute__((aligned(16))) unsigned char smem[];
+    const int tid = threadIdx.x, lane = tid & 63, w = __builtin_amdgcn_readfirstlane(tid >> 6), col = lane & 15, g4 = lane >> 4;
+    bf16_t* Vs = (bf16_t*)(smem + w * NV * 1024);                    // this wave's value tile: rows of dim, 16-byte pieces swizzled
+    _Float16* Ps = (_Float16*)(smem + TW * NV * 1024);               // [BN][TT][GK]
+    bf16_t* Ms = (bf16_t*)(Ps + BN * TT * GK);                       // [GK][TT][BN]
+
+    const int R = 2 * dim, per = H / G;
+    const int slot = tiles[3 * blockIdx.x], t0 = tiles[3 * blockIdx.x + 1], ntok = tiles[3 * blockIdx.x + 2];
+    const int32_t* bt = block_table + (size_t)slot * table_stride;
+    const bool row_ok = col < ntok;
+    const int t = t0 + (row_ok ? col : 0);
+    const int p_row = pos[t], p_first = pos[t0], p_last = pos[t0 + ntok - 1];
+    const int lo_row = window > 0 ? max(0, p_row - window + 1) : 0;
+    const int kstart = (window > 0 ? max(0, p_first - window + 1) : 0) / BN * BN;
+    const int lo_last = window > 0 ? max(0, p_last - window + 1) : 0;
+    const int nT = (p_last - kstart) / BN + 1;
+    const int Z = gridDim.y, z = blockIdx.y;
+    int kv[HW];                                          // key / value pools of the wave's heads (uniform)
+#pragma unroll
+    for (int i = 0; i < HW; ++i) kv[i] = min(w * HW + i, H - 1) / per;
+
+    v4u q[HW][DT];
+#pragma unroll
+    for (int i = 0; i < HW; ++i) {
+        const int h = w * HW + i;
+        const float* qrow = qf + ((size_t)t * H + min(h, H - 1)) * (size_t)dim;
+#pragma unroll
+        for (int s = 0; s < DT; ++s) {
+            const int e0 = 32 * s + 8 * g4;
+            float4 a = make_float4(0.f, 0.f, 0.f, 0.f), b = a;
+            if (row_ok && h < H && e0 < dim) {
+                a = *(const float4*)(qrow + e0);
+                b = *(const float4*)(qrow + e0 + 4);
+            }
+            q[i][s] = v4u{pack_bf2(a.x, a.y), pack_bf2(a.z, a.w), pack_bf2(b.x, b.y), pack_bf2(b.z, b.w)};
+        }
+    }
+    const bool fixed = cap > 0.f && cap <= FIXED_CAP;
+    const float c_in = cap > 0.f ? 2.0f * LOG2E / cap : 0.f, c_two = 2.0f * LOG2E * cap;
+    float m[HW], l[HW];                                  // STATS: running maximum and sum of this lane's keys; else: m = what comes off
+#pragma unroll
+    for (int i = 0; i < HW; ++i) {
+        l[i] = 0.f;
+        m[i] = fixed ? LOG2E * cap : -INFINITY;          // (maxima in units of log 2)
+        if (!STATS) {                                    // 2^(score - m) with m = maximum + log2(sum) - 10
+            const int h = min(w * HW + i, H - 1);
+            float M = -INFINITY, L = 0.f;
+            for (int zz = 0; zz < Z1; ++zz) M = fmaxf(M, part_ml[(((size_t)zz * n_tokens + t) * H + h) * 2]);
+            for (int zz = 0; zz < Z1; ++zz) {
+                const float* ml = part_ml + (((size_t)zz * n_tokens + t) * H + h) * 2;
+                L += __builtin_amdgcn_exp2f(ml[0] - M) * ml[1];
+            }
+            m[i] = M + __builtin_amdgcn_logf(L) - 10.0f;
+        }
+    }
+    v4f acc[STATS ? 1 : HW][STATS ? 1 : CT];
+    v4u tf[HT];                                          // talk as A operand: row h = 16 ht + col, columns 8 g4 .. (GK 32) or 4 g4 .. (GK 16)
+    const int pieces = dim / 8, inv_pieces = 65536 / pieces + 1;     // (p / pieces = p inv_pieces >> 16 for p < 512, pieces <= 16)
+    // 16-byte pieces of a row; piece c of row r lies at c ^ swizzle(r)
+    auto swizzle = [&](int row) { return pieces == 16 ? (row & 7) << 1 : pieces == 8 ? ((row >> 1) & 3) << 1 : 0; };
+    if (!STATS) {
+#pragma unroll
+        for (int i = 0; i < HW; ++i)
+#pragma unroll
+            for (int c = 0; c < CT; ++c) acc[i][c] = v4f{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+        for (int ht = 0; ht < HT; ++ht) {
+            const int h = 16 * ht + col;
+            unsigned u[4] = {0u, 0u, 0u, 0u};
+#pragma unroll
+            for (int e = 0; e < GK / 4; ++e) {
+                const int g = GK / 4 * g4 + e;
+                const _Float16 v = (_Float16)(h < H && g < H ? bf2f(talk[h * H + g]) : 0.f);
+                u[e / 2] |= (unsigned)__builtin_bit_cast(unsigned short, v) << (16 * (e & 1));
+            }
+            tf[ht] = v4u{u[0], u[1], u[2], u[3]};
+        }
+        if (TW * HW < GK)                                // heads that no wave owns: zero weights
+            for (int i = tid; i < BN * TT * (GK - TW * HW); i += 64 * TW) {
+                const int n = GK - TW * HW;
+                Ps[(i / n) * GK + TW * HW + i % n] = (_Float16)0.f;
+            }
+    }
+    v4u kr[DT];
+    auto tile_base = [&](int tile) {                     // 32 consecutive positions inside one page
+        const int k0 = kstart + tile * BN;
+        return pool + ((size_t)bt[k0 / page] * page + (size_t)(k0 % page)) * (size_t)R;
+    };
+    const int k_lane = col * R + dim + 8 * g4;
+    auto load_k = [&](const bf16_t* base, int g, int mt) {   // (rows past the last position exist in the page: their weights become zero)
+        const bf16_t* b = base + (size_t)g * (size_t)pool_stride + 16 * mt * R + k_lane;
+#pragma unroll
+        for (int s = 0; s < DT; ++s) kr[s] = 32 * s + 8 * g4 < dim ? *(const v4u*)(b + 32 * s) : v4u{0u, 0u, 0u, 0u};
+    };
+    auto copy_v = [&](const bf16_t* base, int g, int left) {  // (rows past the last position: the last one again, weight zero)
+        const bf16_t* b = base + (size_t)g * (size_t)pool_stride;
+        int ln = lane;
+        asm volatile("" : "+v"(ln));                     // (addresses made anew per tile: kept across tiles they would cost 16 registers)
+#pragma unroll
+        for (int i = 0; i < NV; ++i) {
+            if (16 * i >= dim) continue;                 // (uniform)
+            const int p = ln + 64 * i, r = p * inv_pieces >> 16, row = min(r, BN - 1), c = (p - r * pieces) ^ swizzle(row);
+            __builtin_amdgcn_global_load_lds((gptr_t)(b + min(row, left) * R + c * 8), (lptr_t)((unsigned char*)Vs + i * 1024), 16, 0, 0);
+        }
+    };
+    const bf16_t* base = pool;
+    if (z < nT) {
+        base = tile_base(z);
+        load_k(base, kv[0], 0);
+    }
+    for (int tile = z; tile < nT; tile += Z) {
+        const int k0 = kstart + tile * BN;
+        const bf16_t* next = tile + Z < nT ? tile_base(tile + Z) : nullptr;
+        if (!STATS) copy_v(base, kv[0], p_last - k0);
+        const bool whole = k0 + BN - 1 <= p_first && k0 >= lo_last;      // every token sees every key of the tile
+#pragma unroll
+        for (int mt = 0; mt < 2; ++mt) {
+            v4f sc[HW];
+#pragma unroll
+            for (int i = 0; i < HW; ++i) {
+                if (i > 0 && kv[i] != kv[i > 0 ? i - 1 : 0]) load_k(base, kv[i], mt);
+                sc[i] = v4f{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+                for (int s = 0; s < DT; ++s)
+                    sc[i] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(bf8, kr[s]), __builtin_bit_cast(bf8, q[i][s]), sc[i], 0, 0, 0);
+            }
+            if (mt == 0) load_k(base, kv[0], 1);
+            else if (next) load_k(next, kv[0], 0);
+            if (HW > 2) __builtin_amdgcn_sched_barrier(0);
+            const int key0 = k0 + 16 * mt + 4 * g4;
+            unsigned pk[4][HW > 1 ? HW / 2 : 1];         // four keys' weights of this lane's token: the wave's heads in pairs
+#pragma unroll
+            for (int i = 0; i < HW; ++i) {
+                float top = m[i];
+#pragma unroll
+                for (int r = 0; r < 4; ++r) {            // scores in units of log 2: cap tanh(s / cap) = cap - 2 cap / (2^(c_in s) + 1)
+                    float x = sc[i][r];
+                    if (cap > 0.f) x = LOG2E * cap - c_two * __builtin_amdgcn_rcpf(__builtin_amdgcn_exp2f(c_in * x) + 1.0f);
+                    else x *= LOG2E;
+                    if (!whole && !(key0 + r <= p_row && key0 + r >= lo_row)) x = -INFINITY;
+                    sc[i][r] = x;
+                    if (STATS && !fixed) top = fmaxf(top, x);
+                }
+                if (STATS && !fixed && top > m[i]) {
+                    l[i] *= __builtin_amdgcn_exp2f(m[i] - top);          // (first keys: 0 * 2^-inf)
+                    m[i] = top;
+                }
+#pragma unroll
+                for (int r = 0; r < 4; ++r) {
+                    const float pr = STATS && top == -INFINITY ? 0.f : __builtin_amdgcn_exp2f(sc[i][r] - m[i]);
+                    if (STATS) {
+                        l[i] += pr;
+                    } else {
+                        const unsigned u = __builtin_bit_cast(unsigned short, (_Float16)(w * HW + i < H ? pr : 0.f));
+                        if (i & 1) pk[r][i / 2] |= u << 16;
+                        else pk[r][i / 2] = u;
+                    }
+                }
+                if (HW > 2) __builtin_amdgcn_sched_barrier(0);
+            }
+            if (!STATS) {
+#pragma unroll
+                for (int r = 0; r < 4; ++r) {
+                    _Float16* dst = Ps + ((16 * mt + 4 * g4 + r) * TT + col) * GK + w * HW;
+                    if (HW == 4) *(v2u*)dst = v2u{pk[r][0], pk[r][HW > 2 ? 1 : 0]};
+                    else if (HW == 2) *(unsigned*)dst = pk[r][0];
+                    else *(unsigned short*)dst = (unsigned short)pk[r][0];
+                }
+            }
+        }
+        if (STATS) {
+            base = next;
+            continue;
+        }
+        __syncthreads();
+        // ---- mix: keys w KPW .. + KPW - 1 of the tile ----
+#pragma unroll
+        for (int ht = 0; ht < HT; ++ht) {
+            v4f mx[KPW];
+#pragma unroll
+            for (int j = 0; j < KPW; ++j) {
+                const _Float16* src = Ps + ((w * KPW + j) * TT + col) * GK + GK / 4 * g4;
+                const v4f zero = {0.f, 0.f, 0.f, 0.f};
+                if (GK == 32) {
+                    mx[j] = __builtin_amdgcn_mfma_f32_16x16x32_f16(__builtin_bit_cast(h8, tf[ht]), *(const h8*)src, zero, 0, 0, 0);
+                } else {
+                    const v2u a = {tf[ht][0], tf[ht][1]};
+                    mx[j] = __builtin_amdgcn_mfma_f32_16x16x16f16(__builtin_bit_cast(h4, a), *(const h4*)src, zero, 0, 0, 0);
+                }
+            }
+#pragma unroll
+            for (int r = 0; r < 4; ++r)
+                *(v2u*)(Ms + ((16 * ht + 4 * g4 + r) * TT + col) * BN + w * KPW) =
+                    v2u{pack_bf2(mx[0][r], mx[1][r]), pack_bf2(mx[2][r], mx[3][r])};
+            if (HT > 1) __builtin_amdgcn_sched_barrier(0);               // (registers: one 16-head block at a time)
+        }
+        __syncthreads();
+        // ---- values: k-slot (g4, e) <-> key 16 (e / 4) + 4 g4 + e % 4 ----
+        auto weights = [&](int i) {
+            const bf16_t* src = Ms + ((w * HW + i) * TT + col) * BN + 4 * g4;
+            const v2u a = *(const v2u*)src, b = *(const v2u*)(src + 16);
+            return __builtin_bit_cast(bf8, (v4u{a[0], a[1], b[0], b[1]}));
+        };
+        const int vr = 4 * g4 + (col >> 2), vsw = swizzle(vr);           // (rows vr and vr + 16 share a swizzle)
+        const bf16_t* vrow = Vs + vr * dim + ((col >> 1) & 1) * 8 + (col & 1) * 4;
+        auto values = [&](int c) {
+            const bf16_t* a = vrow + ((2 * c) ^ vsw) * 8;
+            const s4 a0 = __builtin_amdgcn_ds_read_tr16_b64_v4i16((lds_s4)a);
+            const s4 a1 = __builtin_amdgcn_ds_read_tr16_b64_v4i16((lds_s4)(a + 16 * dim));
+            const v2u u0 = __builtin_bit_cast(v2u, a0), u1 = __builtin_bit_cast(v2u, a1);
+            return __builtin_bit_cast(bf8, (v4u{u0[0], u0[1], u1[0], u1[1]}));
+        };
+        asm volatile("s_waitcnt vmcnt(0)" ::: "memory");                 // the value tile has landed (only this wave reads it)
+        constexpr int STEP = HW > 1 ? 2 : 1;             // two heads of one pool share a value fragment
+#pragma unroll
+        for (int i = 0; i < HW; i += STEP) {
+            const bool both = STEP == 2 && kv[i] == kv[i + STEP - 1];
+#pragma unroll
+            for (int half = 0; half < STEP; ++half) {
+                const int ii = i + half;
+                if (half == 1 && both) continue;         // (done with its neighbour)
+                if (ii > 0 && kv[ii] != kv[ii > 0 ? ii - 1 : 0]) {       // (uniform) another pool's values
+                    asm volatile("s_waitcnt lgkmcnt(0)" ::: "memory");
+                    copy_v(base, kv[ii], p_last - k0);
+                    asm volatile("s_waitcnt vmcnt(0)" ::: "memory");
+                }
+                const bf8 p0 = weights(ii), p1 = weights(both ? i + STEP - 1 : ii);
+#pragma unroll
+                for (int c = 0; c < CT; ++c) {
+                    if (16 * c >= dim) continue;         // (uniform)
+                    const bf8 a = values(c);
+                    acc[ii][c] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(a, p0, acc[ii][c], 0, 0, 0);
+                    if (STEP == 2 && half == 0 && both)
+                        acc[i + STEP - 1][c] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(a, p1, acc[i + STEP - 1][c], 0, 0, 0);
+                    if (HW > 2 && (c & 1) == 1) __builtin_amdgcn_sched_barrier(0);      // (registers: four fragments ahead at most)
+                }
+            }
+        }
+        asm volatile("s_waitcnt lgkmcnt(0)" ::: "memory");               // the value tile has been read: the next copy may start
+        base = next;
+    }
+    if (STATS) {
+#pragma unroll
+        for (int i = 0; i < HW; ++i) {
+            float M = m[i];
+            if (!fixed) {
+                M = fmaxf(M, __shfl_xor(M, 16, 64));
+                M = fmaxf(M, __shfl_xor(M, 32, 64));
+                l[i] = M == -INFINITY ? 0.f : l[i] * __builtin_amdgcn_exp2f(m[i] - M);
+            }
+            float L = l[i];
+            L += __shfl_xor(L, 16, 64);
+            L += __shfl_xor(L, 32, 64);
+            const int h = w * HW + i;
+            if (row_ok && h < H && g4 == 0) {
+                float* ml = part_ml + (((size_t)z * n_tokens + t) * H + h) * 2;
+                ml[0] = M;
+                ml[1] = L;
+            }
+        }
+        return;
+    }
+    if (!row_ok) return;
+#pragma unroll
+    for (int i = 0; i < HW; ++i) {
+        const int h = w * HW + i;
+        if (h >= H) continue;
+        const float f = 0.0009765625f * (Z == 1 && gate ? 1.0f / (1.0f + __expf(-bf2f(gate[(size_t)t * gate_stride + h]))) : 1.0f);
+#pragma unroll
+        for (int c = 0; c < CT; ++c) {
+            const int c0 = 16 * c + 4 * g4;
+            if (c0 >= dim) continue;                     // dim % 8 == 0: four values are inside or outside as a whole
+            const v4f o = acc[i][c] * f;
+            if (Z == 1) *(v2u*)(out + ((size_t)t * H + h) * (size_t)dim + c0) = v2u{pack_bf2(o[0], o[1]), pack_bf2(o[2], o[3])};
+            else *(v4f*)(part_o + (((size_t)z * n_tokens + t) * H + h) * (size_t)dim + c0) = o;
+        }
+    }
+}
+
+// out[t, h] = sigmoid(gate[t, h]) sum_z part_o[z, t, h]      (four elements per thread)
+__global__ __launch_bounds__(NT) void talking_sum_kernel(bf16_t* __restrict__ out, const float* __restrict__ part_o, const bf16_t* __restrict__ gate,
+                                                         int64_t gate_stride, int Z, int H, int dim, int64_t n) {
+    const int64_t i = ((int64_t)blockIdx.x * NT + threadIdx.x) * 4;
+    if (i >= n) return;
+    v4f a = *(const v4f*)(part_o + i);
+    for (int z = 1; z < Z; ++z) a += *(const v4f*)(part_o + (int64_t)z * n + i);
+    if (gate) {
+        const int64_t th = i / dim, t = th / H;
+        a *= 1.0f / (1.0f + __expf(-bf2f(gate[t * gate_stride + (th - t * H)])));
+    }
+    *(v2u*)(out + i) = v2u{pack_bf2(a[0], a[1]), pack_bf2(a[2], a[3])};
+}
+
 int pow2_heads(int n) {
     int hp = 1;
     while (hp < n && hp < 16) hp <<= 1;
@@ -551,4 +876,54 @@ extern "C" int qsv_talking_mix(void* out, const float* part_o, const float* part
                  hipLaunchKernelGGL(talking_mix_kernel<T>, dim3(n), dim3(NT), lds, (hipStream_t)stream, (T*)out, part_o, part_ml,
                                     (const T*)talk, (const T*)gate, gate_stride, key_splits, n, heads, kv_heads, vdim));
     return qsv_launch_status("qsv_talking_mix");
+}
+
+extern "C" int qsv_talking_two_pass_tile_tokens(void) { return TT; }
+extern "C" int qsv_talking_two_pass_ok(int heads, int kv_heads, int dim, int vdim, int page, int dtype) {
+    return dtype == QSV_BF16 && heads > 0 && heads <= 32 && kv_heads > 0 && heads % kv_heads == 0 && dim == vdim && dim > 0 && dim % 8 == 0 &&
+           dim <= 128 && page % BN == 0;
+}
+extern "C" int qsv_talking_two_pass(void* out, float* part_o, float* part_ml, const float* qf, const void* pool, const int32_t* block_table,
+                                    int table_stride, const int32_t* pos, const int32_t* tiles, int n_tiles, int window, int n_tokens,
+                                    int heads, int kv_heads, int dim, int page, int64_t pool_stride, float cap, const void* talk,
+                                    const void* gate, int64_t gate_stride, int stat_splits, int key_splits, void* stream) {
+    QSV_REQUIRE(out && part_ml && qf && pool && block_table && pos && tiles && talk, "qsv_talking_two_pass: null argument");
+    QSV_REQUIRE(qsv_talking_two_pass_ok(heads, kv_heads, dim, dim, page, QSV_BF16) && n_tiles >= 0 && n_tokens >= 0 && table_stride > 0 &&
+                    window >= 0 && pool_stride % 8 == 0 && pool_stride >= 0 && cap >= 0.f && (!gate || gate_stride >= heads),
+                "qsv_talking_two_pass: sizes not supported (%d heads over %d of %d, page %d)", heads, kv_heads, dim, page);
+    QSV_REQUIRE(stat_splits >= 1 && stat_splits <= 64 && key_splits >= 1 && key_splits <= 64 && (key_splits == 1 || part_o),
+                "qsv_talking_two_pass: %d / %d key splits", stat_splits, key_splits);
+    if (n_tiles == 0) return QSV_OK;
+    hipStream_t st_ = (hipStream_t)stream;
+#define QSV_TP(HW, DT)                                                                                                              \
+    do {                                                                                                                            \
+        const int lds = two_pass_lds(HW, DT);                                                                                       \
+        const hipError_t e = hipFuncSetAttribute((const void*)talking_two_pass_kernel<HW, DT, false>,                               \
+                                                 hipFuncAttributeMaxDynamicSharedMemorySize, lds);                                  \
+        QSV_REQUIRE(e == hipSuccess, "qsv_talking_two_pass: %s", hipGetErrorString(e));                                             \
+        hipLaunchKernelGGL((talking_two_pass_kernel<HW, DT, true>), dim3(n_tiles, stat_splits), dim3(64 * TW), 0, st_, (bf16_t*)out, \
+                           part_o, part_ml, 0, qf, (const bf16_t*)pool, block_table, table_stride, pos, tiles, window, heads, kv_heads, \
+                           dim, page, pool_stride, cap, (const bf16_t*)talk, (const bf16_t*)gate, gate_stride, n_tokens);            \
+        hipLaunchKernelGGL((talking_two_pass_kernel<HW, DT, false>), dim3(n_tiles, key_splits), dim3(64 * TW), lds, st_, (bf16_t*)out, \
+                           part_o, part_ml, stat_splits, qf, (const bf16_t*)pool, block_table, table_stride, pos, tiles, window, heads, \
+                           kv_heads, dim, page, pool_stride, cap, (const bf16_t*)talk, (const bf16_t*)gate, gate_stride, n_tokens);  \
+    } while (0)
+#define QSV_TP_DT(HW)                      \
+    do {                                   \
+        if (dim <= 64) QSV_TP(HW, 2);      \
+        else QSV_TP(HW, 4);                \
+    } while (0)
+    if (heads <= 8) QSV_TP_DT(1);
+    else if (heads <= 16) QSV_TP_DT(2);
+    else QSV_TP_DT(4);
+#undef QSV_TP
+#undef QSV_TP_DT
+    if (key_splits > 1) {
+        const int rc = qsv_launch_status("qsv_talking_two_pass");
+        if (rc != QSV_OK) return rc;
+        const int64_t n = (int64_t)n_tokens * heads * dim;
+        hipLaunchKernelGGL(talking_sum_kernel, dim3((unsigned)((n / 4 + NT - 1) / NT)), dim3(NT), 0, st_, (bf16_t*)out, part_o, (const bf16_t*)gate,
+                           gate_stride, key_splits, heads, dim, n);
+    }
+    return qsv_launch_status("qsv_talking_two_pass");
 }

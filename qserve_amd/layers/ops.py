@@ -444,11 +444,14 @@ class HipOps:
                                         int(rot_n if rope is not None else 0), batch.pos.data_ptr(), T, self.code, self._s()), "rotate_qk")
         return out
 
+    talking_split_targets = (512, 512)  # workgroups the two passes should at least have (few tiles: the keys are cut over several)
+
     def talking_attention(self, qf, pool, batch, talk, gate, vdim, page, cap=0.0, window=None, variant=0, key_splits=None, decode=None):
         """qf float [T, H, dim] (scaled queries), pool [G, rows, vdim + dim] -> [T, H * vdim]: softmax weights per head (scores soft-capped
         by cap tanh(. / cap) if cap > 0), mixed over the heads by talk [H, H], on each head's own values; head h times sigmoid(gate[t,
-        h]) (gate [T, H], a column slice is fine, or None).  variant 1: always the wave kernel.  decode: whether a workgroup serves
-        the heads of several key pools (None: where the step's sequences bring few tokens)."""
+        h]) (gate [T, H], a column slice is fine, or None).  variant: 0 = weights mixed before the sum (two passes) where the kernel takes
+        the sizes, else 2; 2 = mixed after the sum on the matrix cores where they take the sizes, else 1; 1 = the wave kernel.
+        decode (variant 2): whether a workgroup serves the heads of several key pools (None: where the sequences bring few tokens)."""
         T, H, dim = qf.shape
         G, R = pool.size(0), pool.size(2)
         self._need(qf, pool, batch.block_table, batch.seq, batch.pos, talk)
@@ -457,13 +460,24 @@ class HipOps:
         out = torch.empty((T, H * vdim), dtype=self.dtype, device=qf.device)
         bt = batch.block_table
         splits, pm = 1, None
-        if variant == 0 and self.L.qsv_talking_attention_mfma_ok(dim, vdim, page, self.code):
+        span = min(batch.max_pos + 1, int(window)) if window else batch.max_pos + 1
+        if variant == 0 and self.L.qsv_talking_two_pass_ok(H, G, dim, vdim, page, self.code):
+            tiles = batch.tiles(self.L.qsv_talking_two_pass_tile_tokens())
+            n = tiles.size(0)
+            s1, s2 = (max(1, min(t // max(n, 1), span // 128, 32)) for t in self.talking_split_targets) if key_splits is None else (key_splits,) * 2
+            pm = torch.empty((s1, T, H, 2), dtype=torch.float32, device=qf.device)
+            po = torch.empty((s2, T, H, vdim), dtype=torch.float32, device=qf.device) if s2 > 1 else None
+            self.check(self.L.qsv_talking_two_pass(out.data_ptr(), 0 if po is None else po.data_ptr(), pm.data_ptr(), qf.data_ptr(), pool.data_ptr(),
+                                                   bt.data_ptr(), bt.stride(0), batch.pos.data_ptr(), tiles.data_ptr(), n, int(window or 0), T, H,
+                                                   G, dim, page, pool.stride(0), float(cap), talk.data_ptr(), 0 if gate is None else gate.data_ptr(),
+                                                   0 if gate is None else gate.stride(0), s1, s2, self._s()), "talking_two_pass")
+            return out
+        if variant != 1 and self.L.qsv_talking_attention_mfma_ok(dim, vdim, page, self.code):
             if decode is None:
                 decode = T <= 2 * len(batch.items)
             kp = self.L.qsv_talking_attention_key_pools(H, G, dim, int(decode))
             tiles = batch.tiles(self.L.qsv_talking_attention_tile_tokens(H, G, kp))
             groups = tiles.size(0) * (G // kp)
-            span = min(batch.max_pos + 1, int(window)) if window else batch.max_pos + 1
             splits = max(1, min(self.attention_split_target // max(groups, 1), span // 128, 32)) if key_splits is None else key_splits
             po = torch.empty((splits, T, H, G, vdim), dtype=torch.float32, device=qf.device)
             pm = torch.empty((splits, T, H, 2), dtype=torch.float32, device=qf.device)

@@ -4,6 +4,7 @@
     python bench.py --design mumelix  [--design-sizes w2048,w4096] [--steps K] [--warmup W]     beside Vekalorn
     python bench.py --design vepolix  [--design-sizes w2048,w4096] [--steps K] [--warmup W]     beside Mumelix
     python bench.py --design pemolorn [--design-sizes w2048,w4096] [--steps K] [--warmup W]     beside Mumelix
+    python bench.py --design sagupel  [--design-sizes w2048,w4096] [--steps K] [--warmup W]     beside Mumelix
 
 Per size (random weights, 4 layers, vocabulary 32000): prompt phase = 8 prompts x 1024 tokens in one step through
 Engine.execute; decoding = 64 sequences at context 1024, one token each per step.  Beside them the Llama-style W4A8KV4
@@ -79,7 +80,7 @@ class OpTimer:
              "moe_route", "moe_experts", "embed_streams", "hc_read", "hc_write", "dyt_sum_rows", "rms_pair_mean", "glu",
              "attention_prep", "rotate_heads", "decay", "conv_silu_unit", "recurrent_scan", "head_rms_gate", "embed_sinusoid",
              "add_rms_norm", "rms_norm_rows", "normed_attention_prep", "max_gates", "add_normed_rms_norm", "qk_norm_rope_prep", "pool_blocks",
-             "min_gru_scan", "relu_sq")
+             "min_gru_scan", "relu_sq", "embed_rms_norm", "residual_conv", "scaled_add_rms_norm", "rotate_qk", "talking_attention")
 
     def __init__(self, ops):
         self.ops, self.events, self.calls, self.on = ops, [], [], False
@@ -94,7 +95,7 @@ class OpTimer:
         import importlib
         return [importlib.import_module("qserve_amd." + m) for m in
                 ("layers.latent_attention", "layers.moe", "layers.recurrent", "layers.softmax_attention", "models.vekalorn",
-                 "models.mumelix", "models.vepolix", "models.pemolorn")]
+                 "models.mumelix", "models.vepolix", "models.pemolorn", "models.sagupel")]
 
     def _wrap(self, name, fn):
         def timed(*a, **k):
@@ -347,7 +348,8 @@ def bench_mumelix(name, s, dev, steps, warmup):
         want = [k * L + L - 1 for k in range(BP)]
         if i == BP:                                          # one step with events around every launch
             ops_pre, _ = timer.step(lambda: eng.execute(items, want))
-            rep_pre = {k: timer.replay(k, 3) for k in ("latent_attention", "hc_read", "hc_write")}
+            rep_pre = {k: timer.replay(k, 3) for k in ("latent_attention", "hc_read", "hc_write", "attention_prep", "conv_silu_unit", "head_rms_gate",
+                                                      "rms_pair_mean")}
             continue
         torch.cuda.synchronize()
         t0 = time.perf_counter()
@@ -683,6 +685,144 @@ def bench_pemolorn(name, s, dev, steps, warmup):
     return out
 
 
+# ---- Sagupel ----------------------------------------------------------------------------------------------------------------
+SAGUPEL_WINDOW = 512
+
+
+def sagupel_config(s, m):
+    """Mumelix's sizes in Sagupel's layers: retention with its gated linear attention's heads, the talking-heads attention with its
+    attention's heads and cache rows beside the same delta rule, sloped window attention with those heads; dense clamped units of the
+    active expert width."""
+    mlp = {"kind": "dense", "ff": s["top"] * s["ff"], "limit": 7.0}
+    H, d = m["g_heads"], m["g_dim"]
+    r = {"type": "retention", "mlp": mlp, "mixer": {"heads": H, "dim": d, "vdim": m["g_vdim"], "decay": [1.0 - 2.0 ** -(5 + h % 8) for h in range(H)],
+                                                    "rot": {"base": 10000.0, "dims": d}}}
+    att = {"heads": m["a_heads"], "kv_heads": m["a_kv"], "dim": m["a_dim"], "vdim": m["a_dim"], "scale": 1.0 / math.sqrt(m["a_dim"])}
+    left = dict(att, softcap=30.0, rot={"base": 500000.0, "dims": m["rot"], "scaling": {"factor": 8.0}})
+    right = {"heads": m["d_heads"], "kv_heads": m["d_kv"], "dim": m["d_dim"], "vdim": m["d_vdim"], "conv": m["taps"]}
+    p = {"type": "parallel", "mlp": mlp, "mixer": {"left": left, "right": right}}
+    a = {"type": "attention", "mlp": mlp, "mixer": dict(att, mask={"size": SAGUPEL_WINDOW})}
+    return {"architecture": "Sagupel", "width": s["width"], "vocab": VOCAB, "norm": {"eps": 1e-5}, "postln_alpha": 3.0,
+            "canon": {"taps": m["taps"]}, "layers": [r, p, a, p][:LAYERS]}
+
+
+def sagupel_weights(cfg, dev, seed=0):
+    g = torch.Generator(device=dev).manual_seed(seed)
+    D, V, taps = cfg["width"], cfg["vocab"], cfg["canon"]["taps"]
+
+    def mat(o, i, s=1.0):
+        return (torch.randn((o, i), device=dev, generator=g) * (s / math.sqrt(i))).bfloat16()
+
+    def vec(n, mean=1.0, s=0.1):
+        return (mean + s * torch.randn((n,), device=dev, generator=g)).bfloat16()
+
+    W = {"embed": mat(V, D), "embed.norm": vec(D), "final.norm": vec(D)}
+    for i, L in enumerate(cfg["layers"]):
+        p, x = f"l{i}.", L["mixer"]
+        W.update({p + "norm1": vec(D), p + "norm2": vec(D), p + "canon1": mat(D, taps)})
+        q = p + "mix."
+        if L["type"] == "retention":
+            H, d, dv = x["heads"], x["dim"], x["vdim"]
+            W.update({q + "q": mat(H * d, D), q + "k": mat(H * d, D), q + "v": mat(H * dv, D), q + "g": mat(H * dv, D), q + "o": mat(D, H * dv)})
+        elif L["type"] == "attention":
+            H, G, d = x["heads"], x["kv_heads"], x["dim"]
+            W.update({q + "q": mat(H * d, D), q + "k": mat(G * d, D), q + "o": mat(D, H * d), q + "q.norm": vec(d), q + "k.norm": vec(d),
+                      q + "sink": vec(H, 0.0, 1.0)})
+        else:
+            a, b, q = x["left"], x["right"], p + "mix.left."
+            H, G, d = a["heads"], a["kv_heads"], a["dim"]
+            W.update({q + "q": mat(H * d, D), q + "q.b": vec(H * d, 0.0), q + "k": mat(G * d, D), q + "k.b": vec(G * d, 0.0), q + "q.norm": vec(d),
+                      q + "k.norm": vec(d), q + "temp": vec(H), q + "talk": (torch.eye(H, device=dev) + 0.1 * mat(H, H).float()).bfloat16(),
+                      q + "g": mat(H, D), q + "o": mat(D, H * d), q + "out": vec(D)})
+            H, G, d, dv, n, q = b["heads"], b["kv_heads"], b["dim"], b["vdim"], b["conv"], p + "mix.right."
+            W.update({q + "q": mat(G * d, D), q + "k": mat(G * d, D), q + "v": mat(H * dv, D), q + "q.conv": mat(G * d, n), q + "k.conv": mat(G * d, n),
+                      q + "v.conv": mat(H * dv, n), q + "b": mat(H, D), q + "A_log": vec(H, -1.0, 0.5), q + "norm": vec(dv), q + "a": mat(H, D),
+                      q + "dt_bias": vec(H, -1.0, 1.0), q + "g": mat(H * dv, D), q + "o": mat(D, H * dv), q + "out": vec(D)})
+        ff, q = L["mlp"]["ff"], p + "mlp."
+        W[q + "gate"], W[q + "up"], W[q + "down"] = mat(ff, D), mat(ff, D), mat(D, ff)
+    return W
+
+
+def bench_sagupel(name, s, dev, steps, warmup):
+    from ..models.sagupel import Sagupel
+    from .engine import Engine
+    m = MUMELIX[name]
+    cfg = sagupel_config(s, m)
+    NB, L, BP = 64, 1024, 8
+    eng = Engine(Sagupel, cfg, sagupel_weights(cfg, dev), dtype="bfloat16", device=dev, max_tokens=NB * (L + 384), max_seqs=NB)
+    timer = OpTimer(eng.ops)
+    g = torch.Generator().manual_seed(1)
+    prompts = [torch.randint(0, VOCAB, (L,), generator=g).tolist() for _ in range(NB)]
+    slots = [eng.open_sequence() for _ in range(NB)]
+    stateless = ("talking_attention", "latent_attention", "scaled_add_rms_norm", "qk_norm_rope_prep", "rotate_qk", "rms_pair_mean", "head_rms_gate",
+                 "glu", "residual_conv", "conv_silu_unit")     # (the convolutions write the same history again; the scan advances its state)
+    pre_ms, ops_pre, rep_pre = [], None, {}
+    for i in range(0, NB, BP):
+        items = [(slots[j], prompts[j]) for j in range(i, i + BP)]
+        want = [k * L + L - 1 for k in range(BP)]
+        if i == BP:                                          # one step with events around every launch
+            ops_pre, _ = timer.step(lambda: eng.execute(items, want))
+            rep_pre = {k: timer.replay(k, 3) for k in stateless}
+            continue
+        torch.cuda.synchronize()
+        t0 = time.perf_counter()
+        eng.execute(items, want)
+        torch.cuda.synchronize()
+        if i > 0:
+            pre_ms.append((time.perf_counter() - t0) * 1e3)
+    pre = sorted(pre_ms)[len(pre_ms) // 2]
+    nxt = [[int(torch.randint(0, VOCAB, (1,), generator=g))] for _ in range(NB)]
+    want = list(range(NB))
+
+    def decode():
+        eng.execute([(slots[j], nxt[j]) for j in range(NB)], want)
+
+    dec_eager = timed(decode, steps, warmup)
+    ops_dec, dec_events_ms = timer.step(decode)
+    rep_dec = {k: timer.replay(k, 20) for k in ("talking_attention", "latent_attention", "qk_norm_rope_prep", "glu", "head_rms_gate", "conv_silu_unit")}
+    eng.decode_graphs = True
+    dec = timed(decode, steps, warmup)
+    graph_ok = any(v is not False for v in eng._graphs.values()) and bool(eng._graphs)
+    ctx = eng.cache.length[slots[0]]
+    T, D = BP * L, s["width"]
+    kinds = [x["type"] for x in cfg["layers"]]
+    n_par, n_att, n_ret = kinds.count("parallel"), kinds.count("attention"), kinds.count("retention")
+    H, R, W_ = m["a_heads"], 2 * m["a_dim"], SAGUPEL_WINDOW
+    pairs = BP * sum(p + 1 for p in range(L))
+    # useful work per visible pair: q.k and p.v of every head, and the mix of the heads' weights
+    talk_flops = n_par * pairs * H * (R + H) * 2.0
+    talk_pre = talk_flops / (rep_pre["talking_attention"] * 1e-3) / 1e12
+    talk_dec = n_par * NB * ctx * m["a_kv"] * R * 2.0 / (rep_dec["talking_attention"] * 1e-3) / 1e9
+    att_flops = n_att * BP * sum(min(p + 1, W_) for p in range(L)) * H * R * 2.0
+    att_pre = att_flops / (rep_pre["latent_attention"] * 1e-3) / 1e12
+    att_dec = n_att * NB * min(ctx, W_) * m["a_kv"] * R * 2.0 / (rep_dec["latent_attention"] * 1e-3) / 1e9
+    # recurrences: 5 (retention) / 7 (delta rule) float operations per state element and token; decoding moves the state twice
+    el = n_ret * m["g_heads"] * m["g_dim"] * m["g_vdim"], n_par * m["d_heads"] * m["d_dim"] * m["d_vdim"]
+    scan_pre = T * (5.0 * el[0] + 7.0 * el[1]) / (ops_pre["recurrent_scan"] * 1e-3) / 1e12
+    scan_dec = NB * (el[0] + el[1]) * 4.0 * 2 / (ops_dec["recurrent_scan"] * 1e-3) / 1e9
+    # residual kernel: per sublayer the float stream in and out, the sublayer's output in; one cast out per layer (the second norm's
+    # reader is the convolution, which reads the float stream and writes one row)
+    res_bytes = T * LAYERS * (2 * (8.0 * D + 2.0 * D) + 2.0 * D)
+    res_pre = res_bytes / (rep_pre["scaled_add_rms_norm"] * 1e-3) / 1e9
+    conv_pre = T * LAYERS * (4.0 * D + 2.0 * D) / (rep_pre["residual_conv"] * 1e-3) / 1e9
+    out = dict(model=f"Sagupel-{name}", sizes=m, prefill_tokens_per_s=T / pre * 1e3, prefill_ms=pre, decode_tokens_per_s=NB / dec * 1e3,
+               decode_ms=dec, decode_from_hipgraph=graph_ok, decode_ms_eager=dec_eager, decode_ms_gpu_events=dec_events_ms, context=ctx,
+               prefill_ops_ms=ops_pre, decode_ops_ms=ops_dec, prefill_kernels_ms=rep_pre, decode_kernels_ms=rep_dec,
+               roofline=dict(prefill_talking_attention_tflops=talk_pre, prefill_talking_attention_frac_bf16_peak=talk_pre / BF16_PEAK_TFLOPS,
+                             decode_talking_attention_gbs=talk_dec, decode_talking_attention_frac_hbm=talk_dec / HBM_PEAK_GBS,
+                             prefill_window_attention_tflops=att_pre, prefill_window_attention_frac_bf16_peak=att_pre / BF16_PEAK_TFLOPS,
+                             decode_window_attention_gbs=att_dec, decode_window_attention_frac_hbm=att_dec / HBM_PEAK_GBS,
+                             prefill_recurrence_tflops=scan_pre, prefill_recurrence_frac_fp32_valu_peak=scan_pre / FP32_VALU_PEAK_TFLOPS,
+                             decode_recurrence_gbs=scan_dec, decode_recurrence_frac_hbm=scan_dec / HBM_PEAK_GBS,
+                             prefill_residual_kernel_gbs=res_pre, prefill_residual_kernel_frac_hbm=res_pre / HBM_PEAK_GBS,
+                             prefill_input_conv_gbs=conv_pre, prefill_input_conv_frac_hbm=conv_pre / HBM_PEAK_GBS))
+    for sl in slots:
+        eng.close_sequence(sl)
+    del eng
+    torch.cuda.empty_cache()
+    return out
+
+
 def main(args, helpers):
     dev = "cuda:0"
     torch.cuda.set_device(0)
@@ -692,12 +832,15 @@ def main(args, helpers):
         build.build(verbose=False)
     steps, warmup = min(args.steps, 32), min(args.warmup, 8)
     for name in args.design_sizes.split(","):
-        if args.design in ("mumelix", "vepolix", "pemolorn") and name not in MUMELIX:      # (sizes that differ in a Vekalorn-only constant)
+        if args.design in ("mumelix", "vepolix", "pemolorn", "sagupel") and name not in MUMELIX:      # (sizes that differ in a Vekalorn-only constant)
             continue
         s = SIZES[name]
         line = {"design": args.design, "size": name, "sizes": s, "layers": LAYERS, "vocab": VOCAB, "dtype": "bf16",
                 "data": "synthetic", "workload": "prefill 8 x 1024 tokens in one step; decode 64 sequences at context 1024"}
-        if args.design == "pemolorn":
+        if args.design == "sagupel":
+            line["sagupel"] = bench_sagupel(name, s, dev, steps, warmup)
+            line["mumelix"] = bench_mumelix(name, s, dev, steps, warmup)
+        elif args.design == "pemolorn":
             line["pemolorn"] = bench_pemolorn(name, s, dev, steps, warmup)
             line["mumelix"] = bench_mumelix(name, s, dev, steps, warmup)
         elif args.design == "vepolix":

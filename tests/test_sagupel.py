@@ -349,7 +349,9 @@ def test_talking_attention_forms(backend, dtype, tol):
     ops = make_ops(backend, dtype, dev)
     g = torch.Generator().manual_seed(4)
     for H, G, d, L, nq, cap, window, gated in ((8, 4, 16, 200, 1, 3.0, None, True), (8, 4, 16, 200, 37, 3.0, None, True), (6, 2, 8, 300, 5, 0.0, 70, False),
-                                               (6, 6, 48, 130, 66, 45.0, None, True), (4, 1, 64, 520, 1, 20.0, None, True), (18, 1, 8, 90, 3, 1.0, 33, True)):
+                                               (6, 6, 48, 130, 66, 45.0, None, True), (4, 1, 64, 520, 1, 20.0, None, True), (18, 1, 8, 90, 3, 1.0, 33, True),
+                                               (32, 8, 128, 200, 20, 30.0, None, True), (16, 4, 128, 170, 33, 0.0, None, True),
+                                               (12, 6, 72, 300, 18, 60.0, 100, False), (32, 32, 16, 140, 17, 2.0, None, True), (21, 7, 40, 97, 16, 8.0, None, True)):
         cache, slot, k, v = _talking_case(g, H, G, d, L, dev, dtype)
         q = torch.randn(nq, H, d, generator=g).bfloat16().double()
         talk, gate = torch.randn(H, H, generator=g).bfloat16().double(), torch.randn(nq, H, generator=g).bfloat16().double()
@@ -366,7 +368,7 @@ def test_talking_attention_forms(backend, dtype, tol):
         b.seq, b.block_table = torch.full((nq,), slot, dtype=torch.int32, device=dev), cache.block_table()
         forms = [dict(), dict(variant=1)]
         if backend == "hip":
-            forms += [dict(key_splits=s, decode=m) for s in (1, 3) for m in (False, True)]
+            forms += [dict(key_splits=s) for s in (1, 2, 5)] + [dict(variant=2, key_splits=s, decode=m) for s in (1, 3) for m in (False, True)]
         for kw in forms:
             out = ops.talking_attention(q.float().to(dev), cache.pools[0], b, talk.to(dtype).to(dev), gate.to(dtype).to(dev) if gated else None,
                                         d, 64, cap=cap, window=window, **kw)
