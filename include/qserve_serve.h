@@ -166,13 +166,14 @@ int qsv_talking_attention_mfma(float* part_o, float* part_ml, const float* qf, c
                                int key_splits, void* stream);
 /* Up to 32 heads of up to 128 elements (vdim = dim), bfloat16: the weights are normalised and mixed before they meet the values, in two
  * launches over the keys (statistics: part_ml float [stat_splits, T, heads, 2]; then the output, for key_splits > 1 through part_o float
- * [key_splits, T, heads, dim]).  tiles of at most qsv_talking_two_pass_tile_tokens() tokens; out: [T, heads, dim], the storage type. */
+ * [key_splits, T, heads, dim]).  scores (float [T, heads, score_stride], score_stride a multiple of 32 above every position; NULL: none):
+ * the first launch leaves the scores there and the second reads them instead of queries and keys (few tokens).  tiles of at most qsv_talking_two_pass_tile_tokens() tokens; out: [T, heads, dim], the storage type. */
 int qsv_talking_two_pass_tile_tokens(void);
 int qsv_talking_two_pass_ok(int heads, int kv_heads, int dim, int vdim, int page, int dtype);
 int qsv_talking_two_pass(void* out, float* part_o, float* part_ml, const float* qf, const void* pool, const int32_t* block_table,
                          int table_stride, const int32_t* pos, const int32_t* tiles, int n_tiles, int window, int n_tokens, int heads,
                          int kv_heads, int dim, int page, int64_t pool_stride, float cap, const void* talk, const void* gate,
-                         int64_t gate_stride, int stat_splits, int key_splits, void* stream);
+                         int64_t gate_stride, int stat_splits, int key_splits, float* scores, int score_stride, void* stream);
 int qsv_talking_mix(void* out, const float* part_o, const float* part_ml, const void* talk, const void* gate, int64_t gate_stride,
                     int key_splits, int n_tokens, int heads, int kv_heads, int vdim, int dtype, void* stream);
 

@@ -444,7 +444,9 @@ __global__ __launch_bounds__(NT) void talking_mix_kernel(T* __restrict__ out, co
 //            bfloat16 to LDS as [head][token][key]
 //   values   O^T += V^T W^T per head: B = the mixed weights, A = the wave's value tile - copied straight into LDS of the wave's own
 //            while the scores are computed, transposed as it is read
-// two barriers a tile.  STATS: scores and sums only, no LDS.
+// two barriers a tile.  MODE 1 (first pass): scores and sums only, no LDS; with `scores` it also leaves the scores (in units of log 2,
+// invisible pairs -inf) for the second pass, which then (MODE 2) reads neither queries nor keys: steps of few tokens, whose cost is
+// reading the cache.
 typedef _Float16 h8 __attribute__((ext_vector_type(8)));
 typedef _Float16 h4 __attribute__((ext_vector_type(4)));
 typedef __attribute__((address_space(1))) const void* gptr_t;
@@ -457,12 +459,14 @@ __host__ __device__ constexpr int two_pass_lds(int hw, int dt) {
     return TW * dt * 2048 + 2 * (BN * TT * two_pass_gk(hw) + two_pass_gk(hw) * TT * BN);
 }
 
-template <int HW, int DT, bool STATS>
+template <int HW, int DT, int MODE>
 __global__ __launch_bounds__(64 * TW, 2) void talking_two_pass_kernel(
     bf16_t* __restrict__ out, float* __restrict__ part_o, float* __restrict__ part_ml, int Z1, const float* __restrict__ qf,
     const bf16_t* __restrict__ pool, const int32_t* __restrict__ block_table, int table_stride, const int32_t* __restrict__ pos,
     const int32_t* __restrict__ tiles, int window, int H, int G, int dim, int page, int64_t pool_stride, float cap,
-    const bf16_t* __restrict__ talk, const bf16_t* __restrict__ gate, int64_t gate_stride, int n_tokens) {
+    const bf16_t* __restrict__ talk, const bf16_t* __restrict__ gate, int64_t gate_stride, int n_tokens, float* __restrict__ scores,
+    int score_stride) {
+    constexpr bool STATS = MODE == 1, KEYS = MODE != 2;
     constexpr int GK = two_pass_gk(HW), HT = GK / 16, NV = 2 * DT, CT = 2 * DT, KPW = BN / TW;
     extern __shared__ __attribute__((aligned(16))) unsigned char smem[];
     const int tid = threadIdx.x, lane = tid & 63, w = __builtin_amdgcn_readfirstlane(tid >> 6), col = lane & 15, g4 = lane >> 4;
@@ -471,7 +475,11 @@ __global__ __launch_bounds__(64 * TW, 2) void talking_two_pass_kernel(
     bf16_t* Ms = (bf16_t*)(Ps + BN * TT * GK);                       // [GK][TT][BN]
 
     const int R = 2 * dim, per = H / G;
-    const int slot = tiles[3 * blockIdx.x], t0 = tiles[3 * blockIdx.x + 1], ntok = tiles[3 * blockIdx.x + 2];
+    // workgroups go round the XCDs: neighbouring tiles (one sequence's) on one XCD, whose L2 then holds that sequence's rows; the last tile
+    // of a run (the most keys) first
+    const int per_xcd = gridDim.x / 8, in_order = (int)blockIdx.x < 8 * per_xcd ? (blockIdx.x & 7) * per_xcd + (blockIdx.x >> 3) : blockIdx.x;
+    const int32_t* tl = tiles + 3 * (gridDim.x - 1 - in_order);
+    const int slot = tl[0], t0 = tl[1], ntok = tl[2];
     const int32_t* bt = block_table + (size_t)slot * table_stride;
     const bool row_ok = col < ntok;
     const int t = t0 + (row_ok ? col : 0);
@@ -485,9 +493,9 @@ __global__ __launch_bounds__(64 * TW, 2) void talking_two_pass_kernel(
 #pragma unroll
     for (int i = 0; i < HW; ++i) kv[i] = min(w * HW + i, H - 1) / per;
 
-    v4u q[HW][DT];
+    v4u q[KEYS ? HW : 1][DT];
 #pragma unroll
-    for (int i = 0; i < HW; ++i) {
+    for (int i = 0; i < (KEYS ? HW : 0); ++i) {
         const int h = w * HW + i;
         const float* qrow = qf + ((size_t)t * H + min(h, H - 1)) * (size_t)dim;
 #pragma unroll
@@ -572,7 +580,7 @@ __global__ __launch_bounds__(64 * TW, 2) void talking_two_pass_kernel(
     const bf16_t* base = pool;
     if (z < nT) {
         base = tile_base(z);
-        load_k(base, kv[0], 0);
+        if (KEYS) load_k(base, kv[0], 0);
     }
     for (int tile = z; tile < nT; tile += Z) {
         const int k0 = kstart + tile * BN;
@@ -584,14 +592,20 @@ __global__ __launch_bounds__(64 * TW, 2) void talking_two_pass_kernel(
             v4f sc[HW];
 #pragma unroll
             for (int i = 0; i < HW; ++i) {
+                if (!KEYS) {
+                    sc[i] = *(const v4f*)(scores + ((size_t)t * H + min(w * HW + i, H - 1)) * (size_t)score_stride + k0 + 16 * mt + 4 * g4);
+                    continue;
+                }
                 if (i > 0 && kv[i] != kv[i > 0 ? i - 1 : 0]) load_k(base, kv[i], mt);
                 sc[i] = v4f{0.f, 0.f, 0.f, 0.f};
 #pragma unroll
                 for (int s = 0; s < DT; ++s)
-                    sc[i] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(bf8, kr[s]), __builtin_bit_cast(bf8, q[i][s]), sc[i], 0, 0, 0);
+                    sc[i] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(bf8, kr[s]), __builtin_bit_cast(bf8, q[KEYS ? i : 0][s]), sc[i], 0, 0, 0);
             }
-            if (mt == 0) load_k(base, kv[0], 1);
-            else if (next) load_k(next, kv[0], 0);
+            if (KEYS) {
+                if (mt == 0) load_k(base, kv[0], 1);
+                else if (next) load_k(next, kv[0], 0);
+            }
             if (HW > 2) __builtin_amdgcn_sched_barrier(0);
             const int key0 = k0 + 16 * mt + 4 * g4;
             unsigned pk[4][HW > 1 ? HW / 2 : 1];         // four keys' weights of this lane's token: the wave's heads in pairs
@@ -600,6 +614,7 @@ __global__ __launch_bounds__(64 * TW, 2) void talking_two_pass_kernel(
                 float top = m[i];
 #pragma unroll
                 for (int r = 0; r < 4; ++r) {            // scores in units of log 2: cap tanh(s / cap) = cap - 2 cap / (2^(c_in s) + 1)
+                    if (!KEYS) continue;
                     float x = sc[i][r];
                     if (cap > 0.f) x = LOG2E * cap - c_two * __builtin_amdgcn_rcpf(__builtin_amdgcn_exp2f(c_in * x) + 1.0f);
                     else x *= LOG2E;
@@ -607,6 +622,8 @@ __global__ __launch_bounds__(64 * TW, 2) void talking_two_pass_kernel(
                     sc[i][r] = x;
                     if (STATS && !fixed) top = fmaxf(top, x);
                 }
+                if (STATS && scores && row_ok && w * HW + i < H)         // (uniform but for the row)
+                    *(v4f*)(scores + ((size_t)t * H + w * HW + i) * (size_t)score_stride + key0) = sc[i];
                 if (STATS && !fixed && top > m[i]) {
                     l[i] *= __builtin_amdgcn_exp2f(m[i] - top);          // (first keys: 0 * 2^-inf)
                     m[i] = top;
@@ -886,27 +903,34 @@ extern "C" int qsv_talking_two_pass_ok(int heads, int kv_heads, int dim, int vdi
 extern "C" int qsv_talking_two_pass(void* out, float* part_o, float* part_ml, const float* qf, const void* pool, const int32_t* block_table,
                                     int table_stride, const int32_t* pos, const int32_t* tiles, int n_tiles, int window, int n_tokens,
                                     int heads, int kv_heads, int dim, int page, int64_t pool_stride, float cap, const void* talk,
-                                    const void* gate, int64_t gate_stride, int stat_splits, int key_splits, void* stream) {
+                                    const void* gate, int64_t gate_stride, int stat_splits, int key_splits, float* scores, int score_stride,
+                                    void* stream) {
     QSV_REQUIRE(out && part_ml && qf && pool && block_table && pos && tiles && talk, "qsv_talking_two_pass: null argument");
     QSV_REQUIRE(qsv_talking_two_pass_ok(heads, kv_heads, dim, dim, page, QSV_BF16) && n_tiles >= 0 && n_tokens >= 0 && table_stride > 0 &&
                     window >= 0 && pool_stride % 8 == 0 && pool_stride >= 0 && cap >= 0.f && (!gate || gate_stride >= heads),
                 "qsv_talking_two_pass: sizes not supported (%d heads over %d of %d, page %d)", heads, kv_heads, dim, page);
     QSV_REQUIRE(stat_splits >= 1 && stat_splits <= 64 && key_splits >= 1 && key_splits <= 64 && (key_splits == 1 || part_o),
                 "qsv_talking_two_pass: %d / %d key splits", stat_splits, key_splits);
+    QSV_REQUIRE(!scores || (score_stride > 0 && score_stride % BN == 0), "qsv_talking_two_pass: score rows of %d keys", score_stride);
     if (n_tiles == 0) return QSV_OK;
     hipStream_t st_ = (hipStream_t)stream;
-#define QSV_TP(HW, DT)                                                                                                              \
+#define QSV_TP_RUN(HW, DT, MODE, SPLITS, LDS)                                                                                       \
+    hipLaunchKernelGGL((talking_two_pass_kernel<HW, DT, MODE>), dim3(n_tiles, SPLITS), dim3(64 * TW), LDS, st_, (bf16_t*)out, part_o, \
+                       part_ml, stat_splits, qf, (const bf16_t*)pool, block_table, table_stride, pos, tiles, window, heads, kv_heads, dim, \
+                       page, pool_stride, cap, (const bf16_t*)talk, (const bf16_t*)gate, gate_stride, n_tokens, scores, score_stride)
+#define QSV_TP_MAIN(HW, DT, MODE)                                                                                                   \
     do {                                                                                                                            \
         const int lds = two_pass_lds(HW, DT);                                                                                       \
-        const hipError_t e = hipFuncSetAttribute((const void*)talking_two_pass_kernel<HW, DT, false>,                               \
+        const hipError_t e = hipFuncSetAttribute((const void*)talking_two_pass_kernel<HW, DT, MODE>,                                \
                                                  hipFuncAttributeMaxDynamicSharedMemorySize, lds);                                  \
         QSV_REQUIRE(e == hipSuccess, "qsv_talking_two_pass: %s", hipGetErrorString(e));                                             \
-        hipLaunchKernelGGL((talking_two_pass_kernel<HW, DT, true>), dim3(n_tiles, stat_splits), dim3(64 * TW), 0, st_, (bf16_t*)out, \
-                           part_o, part_ml, 0, qf, (const bf16_t*)pool, block_table, table_stride, pos, tiles, window, heads, kv_heads, \
-                           dim, page, pool_stride, cap, (const bf16_t*)talk, (const bf16_t*)gate, gate_stride, n_tokens);            \
-        hipLaunchKernelGGL((talking_two_pass_kernel<HW, DT, false>), dim3(n_tiles, key_splits), dim3(64 * TW), lds, st_, (bf16_t*)out, \
-                           part_o, part_ml, stat_splits, qf, (const bf16_t*)pool, block_table, table_stride, pos, tiles, window, heads, \
-                           kv_heads, dim, page, pool_stride, cap, (const bf16_t*)talk, (const bf16_t*)gate, gate_stride, n_tokens);  \
+        QSV_TP_RUN(HW, DT, 1, stat_splits, 0);                                                                                      \
+        QSV_TP_RUN(HW, DT, MODE, key_splits, lds);                                                                                  \
+    } while (0)
+#define QSV_TP(HW, DT)                               \
+    do {                                             \
+        if (scores) QSV_TP_MAIN(HW, DT, 2);          \
+        else QSV_TP_MAIN(HW, DT, 0);                 \
     } while (0)
 #define QSV_TP_DT(HW)                      \
     do {                                   \
@@ -918,6 +942,8 @@ extern "C" int qsv_talking_two_pass(void* out, float* part_o, float* part_ml, co
     else QSV_TP_DT(4);
 #undef QSV_TP
 #undef QSV_TP_DT
+#undef QSV_TP_MAIN
+#undef QSV_TP_RUN
     if (key_splits > 1) {
         const int rc = qsv_launch_status("qsv_talking_two_pass");
         if (rc != QSV_OK) return rc;

@@ -444,14 +444,16 @@ class HipOps:
                                         int(rot_n if rope is not None else 0), batch.pos.data_ptr(), T, self.code, self._s()), "rotate_qk")
         return out
 
-    talking_split_targets = (512, 512)  # workgroups the two passes should at least have (few tiles: the keys are cut over several)
+    talking_score_bytes = 1 << 30       # the most memory kept scores may take
+    talking_split_targets = (512, 256)  # workgroups the two passes should at least have (few tiles: the keys are cut over several)
 
     def talking_attention(self, qf, pool, batch, talk, gate, vdim, page, cap=0.0, window=None, variant=0, key_splits=None, decode=None):
         """qf float [T, H, dim] (scaled queries), pool [G, rows, vdim + dim] -> [T, H * vdim]: softmax weights per head (scores soft-capped
         by cap tanh(. / cap) if cap > 0), mixed over the heads by talk [H, H], on each head's own values; head h times sigmoid(gate[t,
         h]) (gate [T, H], a column slice is fine, or None).  variant: 0 = weights mixed before the sum (two passes) where the kernel takes
         the sizes, else 2; 2 = mixed after the sum on the matrix cores where they take the sizes, else 1; 1 = the wave kernel.
-        decode (variant 2): whether a workgroup serves the heads of several key pools (None: where the sequences bring few tokens)."""
+        decode: the form for few tokens per sequence (None: chosen): the first of two passes keeps the scores, or (variant 2) a workgroup
+        serves the heads of several key pools."""
         T, H, dim = qf.shape
         G, R = pool.size(0), pool.size(2)
         self._need(qf, pool, batch.block_table, batch.seq, batch.pos, talk)
@@ -467,10 +469,15 @@ class HipOps:
             s1, s2 = (max(1, min(t // max(n, 1), span // 128, 32)) for t in self.talking_split_targets) if key_splits is None else (key_splits,) * 2
             pm = torch.empty((s1, T, H, 2), dtype=torch.float32, device=qf.device)
             po = torch.empty((s2, T, H, vdim), dtype=torch.float32, device=qf.device) if s2 > 1 else None
+            # few tokens per sequence: keys are read once, their scores kept (a fraction of the cache's bytes) for the second pass
+            ctx = (batch.max_pos + 32) // 32 * 32
+            keep = T * H * ctx * 4 <= self.talking_score_bytes and (T <= 2 * len(batch.items) if decode is None else decode)
+            sc = torch.empty((T, H, ctx), dtype=torch.float32, device=qf.device) if keep else None
             self.check(self.L.qsv_talking_two_pass(out.data_ptr(), 0 if po is None else po.data_ptr(), pm.data_ptr(), qf.data_ptr(), pool.data_ptr(),
                                                    bt.data_ptr(), bt.stride(0), batch.pos.data_ptr(), tiles.data_ptr(), n, int(window or 0), T, H,
                                                    G, dim, page, pool.stride(0), float(cap), talk.data_ptr(), 0 if gate is None else gate.data_ptr(),
-                                                   0 if gate is None else gate.stride(0), s1, s2, self._s()), "talking_two_pass")
+                                                   0 if gate is None else gate.stride(0), s1, s2, 0 if sc is None else sc.data_ptr(),
+                                                   ctx, self._s()), "talking_two_pass")
             return out
         if variant != 1 and self.L.qsv_talking_attention_mfma_ok(dim, vdim, page, self.code):
             if decode is None:

@@ -31,7 +31,8 @@ SIGNATURES = {
     "qsv_talking_attention_mfma": (_i, [_vp, _vp, _vp, _vp, _vp, _i, _vp, _vp, _i, _i, _i, _i, _i, _i, _i, _i, _i64, _f, _i, _i, _vp]),
     "qsv_talking_two_pass_tile_tokens": (_i, []),
     "qsv_talking_two_pass_ok": (_i, [_i, _i, _i, _i, _i, _i]),
-    "qsv_talking_two_pass": (_i, [_vp, _vp, _vp, _vp, _vp, _vp, _i, _vp, _vp, _i, _i, _i, _i, _i, _i, _i, _i64, _f, _vp, _vp, _i64, _i, _i, _vp]),
+    "qsv_talking_two_pass": (_i, [_vp, _vp, _vp, _vp, _vp, _vp, _i, _vp, _vp, _i, _i, _i, _i, _i, _i, _i, _i64, _f, _vp, _vp, _i64, _i, _i, _vp, _i,
+                                  _vp]),
     "qsv_talking_mix": (_i, [_vp, _vp, _vp, _vp, _vp, _i64, _i, _i, _i, _i, _i, _i, _vp]),
     "qsv_embed_rms_norm": (_i, [_vp, _vp, _vp, _vp, _f, _i, _i, _i, _vp]),
     "qsv_residual_conv": (_i, [_vp, _vp, _vp, _i, _vp, _vp, _vp, _vp, _i, _i, _i, _vp]),

@@ -368,7 +368,7 @@ def test_talking_attention_forms(backend, dtype, tol):
         b.seq, b.block_table = torch.full((nq,), slot, dtype=torch.int32, device=dev), cache.block_table()
         forms = [dict(), dict(variant=1)]
         if backend == "hip":
-            forms += [dict(key_splits=s) for s in (1, 2, 5)] + [dict(variant=2, key_splits=s, decode=m) for s in (1, 3) for m in (False, True)]
+            forms += [dict(key_splits=s, decode=m) for s in (1, 2, 5) for m in (False, True)] + [dict(variant=2, key_splits=s, decode=m) for s in (1, 3) for m in (False, True)]
         for kw in forms:
             out = ops.talking_attention(q.float().to(dev), cache.pools[0], b, talk.to(dtype).to(dev), gate.to(dtype).to(dev) if gated else None,
                                         d, 64, cap=cap, window=window, **kw)
