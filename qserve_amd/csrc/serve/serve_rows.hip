@@ -536,7 +536,9 @@ extern "C" int qsv_add_normed_rms_norm(float* x, void* h, const void* y, const v
 // q_b / k_b / v_b (each may be NULL) are added to the projections first; the pairs are neighbours or, with `halves`, (i, i + rot_n / 2);
 // head_scale (may be NULL) multiplies the common scale; a query row starts with q_pad zeros.  One workgroup per token.  Statistics: per head a wave's sum over `dim`; over the projection a workgroup sum.  The rotation works
 // on normed values staged in LDS (a pair's two values may sit in different threads).  Dynamic LDS: (heads + kv_heads) * dim floats.
-template <typename T, typename TI>
+// VEC (every size, stride and address a multiple of four elements, dim <= 256): four elements per lane, dim / 4 lanes (rounded up to a
+// power of two, `lph`) per head for the per-head statistics, 16-byte stores.
+template <typename T, typename TI, bool VEC>
 __global__ __launch_bounds__(NT) void qk_norm_rope_prep_kernel(float* __restrict__ qf, const TI* __restrict__ q, int64_t q_stride,
                                                                const TI* __restrict__ k, int64_t k_stride, const TI* __restrict__ v,
                                                                int64_t v_stride, int H, int G, int dim, int vdim,
@@ -546,8 +548,8 @@ __global__ __launch_bounds__(NT) void qk_norm_rope_prep_kernel(float* __restrict
                                                                const int64_t* __restrict__ slot, const int32_t* __restrict__ pos,
                                                                const T* __restrict__ q_b, const T* __restrict__ k_b,
                                                                const T* __restrict__ v_b, int halves,
-                                                               const float* __restrict__ head_scale, int q_pad) {
-    extern __shared__ float sm[];
+                                                               const float* __restrict__ head_scale, int q_pad, int lph) {
+    extern __shared__ __attribute__((aligned(16))) float sm[];
     __shared__ float red[NT / 64 + 1];
     const size_t t = blockIdx.x;
     const int lane = threadIdx.x & 63, wv = threadIdx.x >> 6;
@@ -555,7 +557,29 @@ __global__ __launch_bounds__(NT) void qk_norm_rope_prep_kernel(float* __restrict
     float* nq = sm;                                    // [NH][dim]
     const TI* qrow = q + t * q_stride;
     const TI* krow = k ? k + t * k_stride : nullptr;
-    if (per_head) {
+    if (VEC && per_head) {
+        const int e = (lane & (lph - 1)) * 4;
+        for (int h0 = threadIdx.x / lph; h0 - lane / lph < NH; h0 += NT / lph) {      // (a wave stays together: its lanes exchange sums)
+            const bool ok = h0 < NH && e < dim, isq = h0 < H;
+            const int hh = isq ? h0 : h0 - H;
+            float4 u = make_float4(0.f, 0.f, 0.f, 0.f);
+            if (ok) {
+                u = ld4v(isq ? qrow : krow, (size_t)hh * dim + e);
+                const T* bias = isq ? q_b : k_b;
+                if (bias) {
+                    const float4 b = ld4v(bias, (size_t)hh * dim + e);
+                    u.x += b.x; u.y += b.y; u.z += b.z; u.w += b.w;
+                }
+            }
+            float s = u.x * u.x + u.y * u.y + u.z * u.z + u.w * u.w;
+            for (int o = lph >> 1; o > 0; o >>= 1) s += __shfl_xor(s, o, 64);
+            const float inv = 1.0f / sqrtf(s / (float)dim + eps);
+            if (ok) {
+                const float4 g = ld4v(isq ? q_w : k_w, e);
+                *(float4*)(nq + h0 * dim + e) = make_float4(u.x * (inv * g.x), u.y * (inv * g.y), u.z * (inv * g.z), u.w * (inv * g.w));
+            }
+        }
+    } else if (per_head) {
         for (int hh = wv; hh < NH; hh += NT / 64) {
             const bool isq = hh < H;
             const TI* src = isq ? qrow + (size_t)hh * dim : krow + (size_t)(hh - H) * dim;
@@ -606,6 +630,36 @@ __global__ __launch_bounds__(NT) void qk_norm_rope_prep_kernel(float* __restrict
         __syncthreads();
     }
     const int RQ = q_pad + dim, R = vdim + dim;
+    if (VEC) {
+        const int q4 = RQ >> 2, r4 = R >> 2;
+        for (int idx = threadIdx.x; idx < H * q4; idx += NT) {
+            const int h = idx / q4, c = (idx - h * q4) * 4;
+            float4 v = make_float4(0.f, 0.f, 0.f, 0.f);
+            if (c >= q_pad) {
+                v = *(const float4*)(nq + h * dim + c - q_pad);
+                const float f = head_scale ? scale * head_scale[h] : scale;
+                v.x *= f; v.y *= f; v.z *= f; v.w *= f;
+            }
+            st4v(qf, t * H * (size_t)RQ + (size_t)idx * 4, v);
+        }
+        if (!k) return;
+        const size_t row = (size_t)slot[t];
+        for (int idx = threadIdx.x; idx < G * r4; idx += NT) {
+            const int g = idx / r4, c = (idx - g * r4) * 4;
+            float4 u;
+            if (c < vdim) {
+                u = ld4v(v + t * v_stride, (size_t)g * vdim + c);
+                if (v_b) {
+                    const float4 b = ld4v(v_b, (size_t)g * vdim + c);
+                    u.x += b.x; u.y += b.y; u.z += b.z; u.w += b.w;
+                }
+            } else {
+                u = *(const float4*)(nq + (H + g) * dim + c - vdim);
+            }
+            st4v(pool, ((size_t)g * pool_rows + row) * R + c, u);
+        }
+        return;
+    }
     for (int idx = threadIdx.x; idx < H * RQ; idx += NT) {
         const int h = idx / RQ, c = idx - h * RQ;
         qf[t * H * (size_t)RQ + idx] = c < q_pad ? 0.f : nq[h * dim + c - q_pad] * (head_scale ? scale * head_scale[h] : scale);
@@ -635,14 +689,26 @@ extern "C" int qsv_qk_norm_rope_prep(float* qf, const void* q, int64_t q_stride,
     const size_t lds = (size_t)(heads + kv_heads) * dim * 4;
     QSV_REQUIRE(lds <= 64 * 1024, "qsv_qk_norm_rope_prep: %d + %d heads of %d do not fit the workgroup's LDS", heads, kv_heads, dim);
     if (n == 0) return QSV_OK;
-#define QSV_QKP(TI)                                                                                                              \
+    // four elements at a time where everything is aligned to that
+    const size_t el = qkv_dtype == QSV_F32 ? 4 : 2, es = dtype == QSV_F32 ? 4 : 2;
+    auto al = [](const void* p, size_t size) { return (uintptr_t)p % (4 * size) == 0; };
+    const bool vec = dim % 4 == 0 && vdim % 4 == 0 && q_pad % 4 == 0 && dim <= 256 && q_stride % 4 == 0 && al(q, el) && al(q_w, es) && al(q_b, es) &&
+                     (!k || (k_stride % 4 == 0 && v_stride % 4 == 0 && al(k, el) && al(v, el) && al(k_w, es) && al(k_b, es) && al(v_b, es) && al(pool, es)));
+    int lph = 1;
+    while (lph * 4 < dim) lph <<= 1;
+#define QSV_QKP(TI, VEC)                                                                                                         \
     QSV_DISPATCH(dtype, "qsv_qk_norm_rope_prep",                                                                                 \
-                 hipLaunchKernelGGL((qk_norm_rope_prep_kernel<T, TI>), dim3(n), dim3(NT), lds, (hipStream_t)stream, qf, (const TI*)q, \
+                 hipLaunchKernelGGL((qk_norm_rope_prep_kernel<T, TI, VEC>), dim3(n), dim3(NT), lds, (hipStream_t)stream, qf, (const TI*)q, \
                                     q_stride, (const TI*)k, k_stride, (const TI*)v, v_stride, heads, kv_heads, dim, vdim,          \
                                     (const T*)q_w, (const T*)k_w, per_head, eps, rope, rot_n, scale, (T*)pool, pool_rows, slot, pos,  \
-                                    (const T*)q_b, (const T*)k_b, (const T*)v_b, halves, head_scale, q_pad))
-    if (qkv_dtype == QSV_F32) QSV_QKP(float);
-    else QSV_QKP(bf16_t);
+                                    (const T*)q_b, (const T*)k_b, (const T*)v_b, halves, head_scale, q_pad, lph))
+    if (vec) {
+        if (qkv_dtype == QSV_F32) QSV_QKP(float, true);
+        else QSV_QKP(bf16_t, true);
+    } else {
+        if (qkv_dtype == QSV_F32) QSV_QKP(float, false);
+        else QSV_QKP(bf16_t, false);
+    }
 #undef QSV_QKP
     return qsv_launch_status("qsv_qk_norm_rope_prep");
 }
@@ -723,12 +789,64 @@ __global__ __launch_bounds__(NT) void residual_conv_kernel(T* __restrict__ h, co
         for (int c = threadIdx.x; c < D; c += NT) conv_tail1(h, x, cv, t, i, rd, wr, D, c, x[t * D + c]);
     }
 }
+// The same for PAST = taps - 1 known and widths of multiples of four: a workgroup walks CONV_TB consecutive tokens of four channels per
+// thread, the last PAST rows in registers - every row is read once (and PAST more at a block's start); all CONV_TB rows are requested
+// at once.  Rows of another run in the registers are replaced by the run's history (or zeros).
+constexpr int CONV_TB = 8;
+template <typename T, int PAST>
+__global__ __launch_bounds__(NT) void residual_conv_rows_kernel(T* __restrict__ h, const float* __restrict__ x, ConvState cv, int n, int D) {
+    const int c = ((int)blockIdx.y * NT + (int)threadIdx.x) * 4;
+    if (c >= D) return;
+    const int t0 = (int)blockIdx.x * CONV_TB, cnt = min(CONV_TB, n - t0);
+    float4 w[PAST + 1], r[CONV_TB + PAST];               // r[PAST + k]: row t0 + k
+#pragma unroll
+    for (int j = 0; j <= PAST; ++j) w[j] = ld4v(cv.w, (size_t)j * D + c);
+#pragma unroll
+    for (int k = 0; k < CONV_TB + PAST; ++k) r[k] = ld4v(x, (size_t)min(max(t0 - PAST + k, 0), n - 1) * D + c);
+#pragma unroll
+    for (int k = 0; k < CONV_TB; ++k) {
+        if (k >= cnt) continue;
+        const size_t t = (size_t)(t0 + k);
+        const int i = cv.run_off[t], wr = cv.wr[t];      // (uniform over the workgroup)
+        float4 u[PAST + 1];                              // u[d]: the input d tokens back
+#pragma unroll
+        for (int d = 0; d <= PAST; ++d) u[d] = r[PAST + k - d];
+        if (i < PAST) {
+            const int rd = cv.rd[t];
+#pragma unroll
+            for (int d = 1; d <= PAST; ++d)
+                if (d > i) u[d] = conv_in4(x, cv, t, i, rd, d, D, c);
+        }
+        float4 a = u[0];
+#pragma unroll
+        for (int d = 0; d <= PAST; ++d) {
+            const float4 wd = w[PAST - d];
+            a.x += wd.x * u[d].x; a.y += wd.y * u[d].y; a.z += wd.z * u[d].z; a.w += wd.w * u[d].w;
+        }
+        st4v(h, t * D + c, a);
+        if (wr >= 0) {
+#pragma unroll
+            for (int d = 0; d < PAST; ++d) st4v(cv.hist, ((size_t)wr * PAST + (PAST - 1 - d)) * D + c, u[d]);
+        }
+    }
+}
 extern "C" int qsv_residual_conv(void* h, const float* x, const float* w, int taps, float* hist, const int32_t* run_off,
                                  const int32_t* state_rd, const int32_t* state_wr, int n, int D, int dtype, void* stream) {
     QSV_REQUIRE(h && x && w && run_off && state_rd && state_wr && n >= 0 && D > 0 && taps >= 1 && (taps == 1 || hist),
                 "qsv_residual_conv: bad arguments");
     if (n == 0) return QSV_OK;
     const ConvState cv = {w, hist, run_off, state_rd, state_wr, taps - 1};
+    if (D % 4 == 0 && taps >= 2 && taps <= 4 && n >= 2 * CONV_TB && D <= 65535 * NT * 4) {
+        const dim3 grid((n + CONV_TB - 1) / CONV_TB, (D / 4 + NT - 1) / NT);
+#define QSV_RCR(P)                                                                                                          \
+    QSV_DISPATCH(dtype, "qsv_residual_conv",                                                                                \
+                 hipLaunchKernelGGL((residual_conv_rows_kernel<T, P>), grid, dim3(NT), 0, (hipStream_t)stream, (T*)h, x, cv, n, D))
+        if (taps == 2) QSV_RCR(1);
+        else if (taps == 3) QSV_RCR(2);
+        else QSV_RCR(3);
+#undef QSV_RCR
+        return qsv_launch_status("qsv_residual_conv");
+    }
     if (D % 4 == 0)
         QSV_DISPATCH(dtype, "qsv_residual_conv",
                      hipLaunchKernelGGL((residual_conv_kernel<T, true>), dim3(n), dim3(NT), 0, (hipStream_t)stream, (T*)h, x, cv, D));

@@ -195,39 +195,76 @@ __global__ __launch_bounds__(NT) void dyt_sum_rows_kernel(T* __restrict__ out, c
 }
 
 // out[t] = (a[t] / rms(a[t]) * wa + b[t] / rms(b[t]) * wb) / 2
-template <typename T>
+template <typename T, bool VEC>
 __global__ __launch_bounds__(NT) void rms_pair_mean_kernel(T* __restrict__ out, const T* __restrict__ a, const T* __restrict__ wa,
                                                            const T* __restrict__ b, const T* __restrict__ wb, float eps, int D) {
     __shared__ float red[NT / 64 + 1];
     const size_t t = blockIdx.x;
     float sa = 0.f, sb = 0.f;
-    for (int i = threadIdx.x; i < D; i += NT) {
-        const float u = ld(a, t * D + i), v = ld(b, t * D + i);
-        sa += u * u;
-        sb += v * v;
+    if (VEC) {                                                           // D % 4 == 0
+        for (int i = threadIdx.x * 4; i < D; i += NT * 4) {
+            float u[4], v[4];
+            ld4t(a, t * D + i, u);
+            ld4t(b, t * D + i, v);
+#pragma unroll
+            for (int j = 0; j < 4; ++j) {
+                sa += u[j] * u[j];
+                sb += v[j] * v[j];
+            }
+        }
+    } else {
+        for (int i = threadIdx.x; i < D; i += NT) {
+            const float u = ld(a, t * D + i), v = ld(b, t * D + i);
+            sa += u * u;
+            sb += v * v;
+        }
     }
     const float ia = 1.0f / sqrtf(block_sum<NT>(sa, red) / (float)D + eps);
     const float ib = 1.0f / sqrtf(block_sum<NT>(sb, red) / (float)D + eps);
+    if (VEC) {
+        for (int i = threadIdx.x * 4; i < D; i += NT * 4) {
+            float u[4], v[4], wu[4], wv[4], y[4];
+            ld4t(a, t * D + i, u);
+            ld4t(b, t * D + i, v);
+            ld4t(wa, i, wu);
+            ld4t(wb, i, wv);
+#pragma unroll
+            for (int j = 0; j < 4; ++j) y[j] = 0.5f * (u[j] * ia * wu[j] + v[j] * ib * wv[j]);
+            st4t(out, t * D + i, y);
+        }
+        return;
+    }
     for (int i = threadIdx.x; i < D; i += NT)
         st(out, t * D + i, 0.5f * (ld(a, t * D + i) * ia * ld(wa, i) + ld(b, t * D + i) * ib * ld(wb, i)));
 }
 
 // out[r, f] = act(a[r, 2f]) * a[r, 2f + 1];  act 0: silu, 1: gelu in its tanh form, 0.5 z (1 + tanh(sqrt(2 / pi) (z + 0.044715 z^3)));
 // act 2: g = min(gate, limit), u = clamp(up, -limit, limit) -> g sigmoid(1.702 g) (u + 1)
-template <typename T>
+__device__ __forceinline__ float glu_unit(float g, float u, int act, float limit) {
+    if (act == 2) {
+        g = fminf(g, limit);
+        u = fminf(fmaxf(u, -limit), limit);
+        return g / (1.0f + expf(-1.702f * g)) * (u + 1.0f);
+    }
+    const float ag = act == 0 ? g / (1.0f + expf(-g)) : 0.5f * g * (1.0f + tanhf(0.7978845608028654f * (g + 0.044715f * g * g * g)));
+    return ag * u;
+}
+template <typename T, bool VEC>
 __global__ __launch_bounds__(NT) void glu_kernel(T* __restrict__ out, const T* __restrict__ a, int ff, int act, float limit) {
     const size_t r = blockIdx.x;
-    for (int f = threadIdx.x; f < ff; f += NT) {
-        float g = ld(a, (r * ff + f) * 2), u = ld(a, (r * ff + f) * 2 + 1);
-        if (act == 2) {
-            g = fminf(g, limit);
-            u = fminf(fmaxf(u, -limit), limit);
-            st(out, r * ff + f, g / (1.0f + expf(-1.702f * g)) * (u + 1.0f));
-            continue;
+    if (VEC) {                                                           // ff % 4 == 0: four units per thread and pass
+        for (int f = threadIdx.x * 4; f < ff; f += NT * 4) {
+            float p[4], q[4];
+            ld4t(a, (r * ff + f) * 2, p);
+            ld4t(a, (r * ff + f) * 2 + 4, q);
+            const float y[4] = {glu_unit(p[0], p[1], act, limit), glu_unit(p[2], p[3], act, limit), glu_unit(q[0], q[1], act, limit),
+                                glu_unit(q[2], q[3], act, limit)};
+            st4t(out, r * ff + f, y);
         }
-        const float ag = act == 0 ? g / (1.0f + expf(-g)) : 0.5f * g * (1.0f + tanhf(0.7978845608028654f * (g + 0.044715f * g * g * g)));
-        st(out, r * ff + f, ag * u);
+        return;
     }
+    for (int f = threadIdx.x; f < ff; f += NT)
+        st(out, r * ff + f, glu_unit(ld(a, (r * ff + f) * 2), ld(a, (r * ff + f) * 2 + 1), act, limit));
 }
 }  // namespace
 
@@ -290,16 +327,27 @@ extern "C" int qsv_rms_pair_mean(void* out, const void* a, const void* wa, const
                                  int dtype, void* stream) {
     QSV_REQUIRE(out && a && wa && b && wb && n >= 0 && D > 0, "qsv_rms_pair_mean: bad arguments");
     if (n == 0) return QSV_OK;
-    QSV_DISPATCH(dtype, "qsv_rms_pair_mean",
-                 hipLaunchKernelGGL(rms_pair_mean_kernel<T>, dim3(n), dim3(NT), 0, (hipStream_t)stream, (T*)out, (const T*)a,
-                                    (const T*)wa, (const T*)b, (const T*)wb, eps, D));
+    if (D % 4 == 0)
+        QSV_DISPATCH(dtype, "qsv_rms_pair_mean",
+                     hipLaunchKernelGGL((rms_pair_mean_kernel<T, true>), dim3(n), dim3(NT), 0, (hipStream_t)stream, (T*)out, (const T*)a,
+                                        (const T*)wa, (const T*)b, (const T*)wb, eps, D));
+    else
+        QSV_DISPATCH(dtype, "qsv_rms_pair_mean",
+                     hipLaunchKernelGGL((rms_pair_mean_kernel<T, false>), dim3(n), dim3(NT), 0, (hipStream_t)stream, (T*)out, (const T*)a,
+                                        (const T*)wa, (const T*)b, (const T*)wb, eps, D));
     return qsv_launch_status("qsv_rms_pair_mean");
 }
 
 extern "C" int qsv_glu(void* out, const void* a, int n_rows, int ff, int act, float limit, int dtype, void* stream) {
     QSV_REQUIRE(out && a && n_rows >= 0 && ff > 0 && (act == 0 || act == 1 || (act == 2 && limit > 0.f)), "qsv_glu: bad arguments");
     if (n_rows == 0) return QSV_OK;
-    QSV_DISPATCH(dtype, "qsv_glu",
-                 hipLaunchKernelGGL(glu_kernel<T>, dim3(n_rows), dim3(NT), 0, (hipStream_t)stream, (T*)out, (const T*)a, ff, act, limit));
+    if (ff % 4 == 0)
+        QSV_DISPATCH(dtype, "qsv_glu",
+                     hipLaunchKernelGGL((glu_kernel<T, true>), dim3(n_rows), dim3(NT), 0, (hipStream_t)stream, (T*)out, (const T*)a, ff, act,
+                                        limit));
+    else
+        QSV_DISPATCH(dtype, "qsv_glu",
+                     hipLaunchKernelGGL((glu_kernel<T, false>), dim3(n_rows), dim3(NT), 0, (hipStream_t)stream, (T*)out, (const T*)a, ff, act,
+                                        limit));
     return qsv_launch_status("qsv_glu");
 }

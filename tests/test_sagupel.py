@@ -178,7 +178,7 @@ def test_mixer_input_convolution_carries_its_last_rows(backend):
     dev = device_of(backend)
     ops = make_ops(backend, torch.float32, dev)
     g = torch.Generator().manual_seed(2)
-    for D, taps, cuts in ((10, 3, [1, 2, 3, 9]), (72, 4, [5]), (6, 2, [1, 2, 3]), (300, 5, [2, 3, 4, 30]), (12, 1, [4, 5]), (8, 6, [1, 2, 3, 4, 5, 6, 7])):
+    for D, taps, cuts in ((10, 3, [1, 2, 3, 9]), (72, 4, [5]), (40, 3, [1, 3, 20]), (12, 2, []), (1040, 4, [16]), (6, 2, [1, 2, 3]), (300, 5, [2, 3, 4, 30]), (12, 1, [4, 5]), (8, 6, [1, 2, 3, 4, 5, 6, 7])):
         T = 33
         x = torch.randn(T, D, generator=g)
         w = torch.randn(D, taps, generator=g)
