@@ -19,7 +19,9 @@ LIB = os.path.join(HERE, "libqserve_amd.so")
 SOURCES = ["lib.hip", "gemm_w4a8.hip", "gemm_w4a8_lds.hip", "gemm_w4a8_tiled.hip", "gemm_w4a8_wide.hip", "gemm_w4a8_ring.hip", "gemm_w8a8.hip", "attention.hip", "attention_mfma.hip", "attention_mfma8.hip", "flash_prefill.hip", "fused_small.hip", "direct_allreduce.hip"]
 ARCH = "gfx950"
 FLAGS = ["-O3", "-std=c++17", "-fPIC", f"--offload-arch={ARCH}", "-Wall", "-Wno-unused-function",
-         "-Wno-unused-variable", "-Wno-unused-but-set-variable"]
+         "-Wno-unused-variable", "-Wno-unused-but-set-variable",
+         # packed-FP32 instructions off: a float result must not depend on how the compiler pairs operations
+         "-Xclang", "-target-feature", "-Xclang", "-packed-fp32-ops"]
 
 
 def hipcc():
@@ -82,8 +84,7 @@ SERVE_BUILD = os.path.join(HERE, "_build_serve")
 SERVE_LIB = os.path.join(HERE, "libqserve_serve.so")
 SERVE_SOURCES = ["serve_rows.hip", "serve_attention.hip", "serve_attention_mfma.hip", "serve_moe.hip", "serve_moe_gemm.hip",
                  "serve_streams.hip", "serve_recurrent.hip", "serve_talking.hip"]
-# packed-FP32 instructions off: the kernels' float statistics must not depend on how the compiler pairs them
-SERVE_FLAGS = FLAGS + ["-Xclang", "-target-feature", "-Xclang", "-packed-fp32-ops"]
+SERVE_FLAGS = FLAGS
 
 
 def serve_stale():

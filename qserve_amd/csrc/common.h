@@ -79,7 +79,11 @@ __device__ __forceinline__ float epi_per_chn(int acc, float ws, float sa, float 
 #pragma clang fp contract(off)
     float t = (float)acc * ws;
     const float u = wz * ss;
-    if (fma) return __builtin_fmaf(t, sa, -u);
+    if (fma) {
+        float r = __builtin_fmaf(t, sa, -u);
+        asm("" : "+v"(r));                       // a float of its own: fused with the caller's cast (fma_mixlo) it would be rounded only once
+        return r;
+    }
     t = t * sa;
     return t - u;
 }
