@@ -126,6 +126,9 @@ def test_serve_argument_validation_without_gpu():
     assert L.qsv_talking_attention(1, 1, 1, 1, 4, 1, 1, 0, 4, 2, 2, 520, 64, 64, 0, 0.0, 0, None) == 1         # heads of 520 elements
     assert L.qsv_talking_attention_mfma(1, 1, 1, 1, 1, 4, 1, 1, 1, 0, 4, 4, 4, 64, 64, 64, 0, 0.0, 3, 1, None) == 1     # 4 pools in groups of 3
     assert L.qsv_talking_mix(1, 1, None, 1, None, 0, 2, 4, 4, 2, 64, 0, None) == 1                             # two key splits without their maxima
+    assert [L.qsv_talking_two_pass_ok(*a) for a in ((32, 8, 128, 128, 64, 0), (33, 3, 64, 64, 64, 0), (8, 2, 136, 136, 64, 0), (8, 2, 64, 64, 64, 1))] == [1, 0, 0, 0]
+    assert L.qsv_talking_two_pass(1, None, 1, 1, 1, 1, 4, 1, 1, 1, 0, 4, 4, 2, 64, 64, 0, 0.0, 1, None, 0, 1, 2, None, 0, None) == 1   # two key splits without a workspace
+    assert L.qsv_talking_two_pass(1, 1, 1, 1, 1, 1, 4, 1, 1, 1, 0, 4, 4, 2, 64, 64, 0, 0.0, 1, None, 0, 1, 2, 1, 40, None) == 1         # score rows that are no multiple of a tile
     assert L.qsv_residual_conv(1, 1, 1, 3, None, 1, 1, 1, 2, 8, 0, None) == 1                                  # three taps without a history
     assert L.qsv_scaled_add_rms_norm(1, None, 1, 2.0, 1, 1e-5, 1, 3, 1, 1, 1, 2, 8, 0, None) == 1              # a convolution without its output
     assert L.qsv_rotate_qk(1, 1, 64, 2, 8, 8, 1, 10, 1, 2, 0, None) == 1                                       # 10 rotated dimensions of 8
