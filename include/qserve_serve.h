@@ -31,6 +31,12 @@ int qsv_embed_sinusoid(float* x, const void* table, const int32_t* tokens, const
  * (h == NULL: the sum only). */
 int qsv_add_rms_norm(float* x, void* h, const void* a, const void* b, const void* c, const void* w, float eps, int n_tokens,
                      int width, int dtype, void* stream);
+/* x[t] += sa a[t] + sb b[t] + sc c[t] (a, b, c storage type, each may be NULL; scales per coordinate, storage type, NULL: ones), then with n =
+ * x[t] / sqrt(mean(x[t]^2) + eps): h0[t] = n * g0 and h1[t] = n * g1 in the storage type (float gains per coordinate; h1 may be NULL; h0 NULL: the
+ * sum only).  tokens != NULL: x[t] starts as table[tokens[t]]. */
+int qsv_scaled_sum_rms_norms(float* x, void* h0, void* h1, const void* a, const void* sa, const void* b, const void* sb, const void* c,
+                             const void* sc, const float* g0, const float* g1, const int32_t* tokens, const void* table, float eps,
+                             int n_tokens, int width, int dtype, void* stream);
 /* Sublayers between two norms: x[t] += rms_norm(y[t]) * w_post (y == NULL: nothing added), then h[t] = rms_norm(x[t]) * w_next in
  * the storage type (h == NULL: the sum only).  A weight is one gain for all coordinates (its *_wide flag 0) or one per coordinate. */
 int qsv_add_normed_rms_norm(float* x, void* h, const void* y, const void* w_post, int post_wide, const void* w_next, int next_wide,
@@ -42,12 +48,14 @@ int qsv_add_normed_rms_norm(float* x, void* h, const void* y, const void* w_post
  *   pool[g, slot[t]] = [ v[t, g] | k'[t, g] ]              [kv_heads, pool_rows, vdim + dim]     (k == NULL: nothing is written)
  * Options (NULL / 0: none): q_b, k_b, v_b (storage type, one per projected channel) are added to the projections before anything else;
  * halves: pair i = dimensions i and i + rot_n / 2; head_scale (float [heads]) multiplies `scale`; a query row starts with q_pad zeros
- * (above: q_pad = vdim).  v may be k's own columns (values that are the projected keys). */
-int qsv_qk_norm_rope_prep(float* qf, const void* q, int64_t q_stride, const void* k, int64_t k_stride, const void* v,
+ * (above: q_pad = vdim).  v may be k's own columns (values that are the projected keys).  q_w = k_w = NULL (per head): no weights.  rot_gain >
+ * 0: the norm follows the rotation (per head, no weights), rot_gain = the square of the magnitude that rope's cos and sin carry.  q_store:
+ * the query rows leave in the storage type. */
+int qsv_qk_norm_rope_prep(void* qf, const void* q, int64_t q_stride, const void* k, int64_t k_stride, const void* v,
                           int64_t v_stride, int qkv_dtype, int heads, int kv_heads, int dim, int vdim, const void* q_w,
                           const void* k_w, int per_head, float eps, const float* rope, int rot_n, float scale, void* pool,
                           int64_t pool_rows, const int64_t* slot, const int32_t* pos, int n_tokens, const void* q_b, const void* k_b,
-                          const void* v_b, int halves, const float* head_scale, int q_pad, int dtype, void* stream);
+                          const void* v_b, int halves, const float* head_scale, int q_pad, float rot_gain, int q_store, int dtype, void* stream);
 /* x[t] = rms_norm(table[tokens[t]]) * w    (float) */
 int qsv_embed_rms_norm(float* x, const void* table, const int32_t* tokens, const void* w, float eps, int n_tokens, int width, int dtype,
                        void* stream);
@@ -64,8 +72,8 @@ int qsv_scaled_add_rms_norm(float* x, void* h, const void* y, float alpha, const
  * dimensions of every q and k head turned by the position, halves layout (rope as above, NULL with rot_n = 0). */
 int qsv_rotate_qk(float* out, const void* qkv, int64_t stride, int heads, int dim, int vdim, const float* rope, int rot_n,
                   const int32_t* pos, int n_tokens, int dtype, void* stream);
-/* out[r] = rms_norm(x[rows[r]]) * w in the storage type (rows == NULL: row r). */
-int qsv_rms_norm_rows(void* out, const float* x, const int32_t* rows, const void* w, float eps, int n_rows, int width, int dtype,
+/* out[r] = rms_norm(x[rows[r]]) * w in the storage type (rows == NULL: row r); w of the storage type or float (w_dtype). */
+int qsv_rms_norm_rows(void* out, const float* x, const int32_t* rows, const void* w, int w_dtype, float eps, int n_rows, int width, int dtype,
                       void* stream);
 /* Queries and keys RMS-normed over the whole projection (all heads at once), values optionally blended, cache rows written:
  *   qf[t, h]         = [ 0 (vdim) | (q[t] / rms(q[t]) * q_w)[h] * scale ]          float [T, heads, vdim + dim]
@@ -202,9 +210,11 @@ int qsv_moe_route(int32_t* idx, float* weight, const void* h, const void* router
  * `limit` is read by this activation only.  Expert indices >= n_experts name identity experts (output = input): the up kernels
  * skip their slots and the down / combine kernels add weight * h[t] for them. */
 #define QSV_ACT_CLAMPED_GLU 3
+/* Weights on the expert's input: with in_weight != NULL (float, per slot t * top_k + k) an up product works on in_weight * input, and the
+ * down / combine kernels take weight == NULL (ones). */
 /* act[t, k] = activation(up[idx[t, k]] . h[t])     up: [E, ff, width] -> act [T, top_k, ff or ff / 2] (storage type). */
 int qsv_moe_up(void* act, const void* h, const void* up, const int32_t* idx, int n_tokens, int top_k, int width, int ff,
-               int activation, float limit, int n_experts, int dtype, void* stream);
+               int activation, float limit, int n_experts, const float* in_weight, int dtype, void* stream);
 
 /* y[t] = sum_k weight[t, k] * down[idx[t, k]] . act[t, k]     down: [E, width, ff] -> y [T, width] (storage type). */
 int qsv_moe_down(void* y, const void* act, const void* down, const int32_t* idx, const float* weight, int n_tokens,
@@ -219,14 +229,14 @@ int qsv_moe_down(void* y, const void* act, const void* down, const int32_t* idx,
  * s in [offsets[e], offsets[e + 1]) of every expert e; W [n_experts, rows, K]; act = one of QSV_ACT_* (QSV_ACT_GLU: out is
  * rows / 2 wide).  Every weight is read once per launch.  K a multiple of 8, at most 4096. */
 int qsv_expert_rows(void* out, const void* X, const int64_t* x_index, int div, const void* W, const int64_t* offsets,
-                    int n_experts, int rows, int K, int act, float limit, void* stream);
+                    int n_experts, int rows, int K, int act, float limit, const float* in_weight, void* stream);
 /* Grouped expert product on the bf16 matrix cores (prompt phase): the same out[s, n] for work tiles (expert, first sorted slot,
  * slots <= qsv_grouped_gemm_tile_slots()) listed in tiles int32 [n_tiles, 3]; K a multiple of qsv_grouped_gemm_k_step(), n_rows
  * a multiple of 4, n_tiles <= 65535.  act: QSV_ACT_* (QSV_ACT_GLU: out is n_rows / 2 wide). */
 int qsv_grouped_gemm_tile_slots(void);
 int qsv_grouped_gemm_k_step(void);
 int qsv_grouped_gemm(void* out, const void* X, const int64_t* x_index, int div, const void* W, const int32_t* tiles,
-                     int n_tiles, int n_rows, int K, int act, float limit, void* stream);
+                     int n_tiles, int n_rows, int K, int act, float limit, const float* in_weight, void* stream);
 int qsv_gather_rows(void* out, const void* src, const int64_t* order, int div, int n_rows, int width, int dtype, void* stream);
 int qsv_relu_sq(void* a, int64_t n, int dtype, void* stream);
 /* (idx != NULL: slots with idx[t, k] >= n_experts take h[t] in place of a sorted row) */
@@ -258,7 +268,25 @@ int qsv_rms_pair_mean(void* out, const void* a, const void* wa, const void* b, c
 #define QSV_GLU_SILU 0
 #define QSV_GLU_GELU_TANH 1
 #define QSV_GLU_CLAMPED 2   /* g = min(gate, limit), u = clamp(up, -limit, limit): g sigmoid(1.702 g) (u + 1) */
-int qsv_glu(void* out, const void* a, int n_rows, int ff, int act, float limit, int dtype, void* stream);
+/* row_scale != NULL: row r of a is multiplied by row_scale[scale_index ? scale_index[r] : r] first. */
+int qsv_glu(void* out, const void* a, int n_rows, int ff, int act, float limit, const float* row_scale, const int64_t* scale_index,
+            int dtype, void* stream);
+
+/* ---- attention with two key maps over the same values, and what feeds it (serve_differential.hip) ------------------------------ */
+/* A causal convolution over time on every channel of a projection row q (q_channels) | k (kv_heads * key_width) | v (kv_heads * vdim): y_t =
+ * sum_j w[j, c] u_(t - (taps - 1) + j), w float [taps, channels].  History: the projected rows, as in qsv_residual_conv.
+ *   q[t]             = y * scale * (temp_every > 0 ? 1 + temp_coef ln(floor((pos[t] + 1) / temp_every) + 1) : 1)    [T, q_channels], storage type
+ *   pool[g, slot[t]] = [ v'[t, g] | k'[t, g] ]      [kv_heads, pool_rows, vdim + key_width]     (kv_heads == 0: queries only) */
+int qsv_conv_heads_cache(void* q, void* pool, int64_t pool_rows, const void* proj, int64_t stride, const float* w, int taps, float* hist,
+                         const int32_t* run_off, const int32_t* state_rd, const int32_t* state_wr, const int64_t* slot, const int32_t* pos,
+                         int q_channels, int kv_heads, int key_width, int vdim, float scale, float temp_coef, double temp_every, int n_tokens,
+                         int dtype, void* stream);
+/* q [T, H, 2, dim] (scaled), cache rows [v (vdim) | k_1 (dim) | k_2 (dim)] in G pools (head h reads pool h / (H / G)), keys 0 .. pos[t]:
+ * a_m = softmax(q_m . k_m) v, o = a_1 - lambda a_2, out[t, h] = o / sqrt(mean(o^2) + eps) * out_scale * sigmoid(gate[t, h]) (gate NULL: no
+ * gate); [T, H, vdim].  Any sizes up to dim 512 and vdim 1024. */
+int qsv_diff_attention(void* out, const void* q, const void* pool, const int32_t* block_table, int table_stride, const int32_t* seq,
+                       const int32_t* pos, int n_tokens, int H, int G, int dim, int vdim, int page, int64_t pool_stride, float lambda,
+                       float out_scale, float eps, const void* gate, int64_t gate_stride, int dtype, void* stream);
 
 /* ---- matrix-state recurrences and the attention beside them (serve_recurrent.hip) ------------------------------------------- */
 /* out[t, c] (float, [T, heads * dim]) = a_log ? exp(-exp(a_log[c / dim]) * softplus(z[t, c] + bias[c]))

@@ -83,7 +83,7 @@ SERVE_CSRC = os.path.join(CSRC, "serve")
 SERVE_BUILD = os.path.join(HERE, "_build_serve")
 SERVE_LIB = os.path.join(HERE, "libqserve_serve.so")
 SERVE_SOURCES = ["serve_rows.hip", "serve_attention.hip", "serve_attention_mfma.hip", "serve_moe.hip", "serve_moe_gemm.hip",
-                 "serve_streams.hip", "serve_recurrent.hip", "serve_talking.hip"]
+                 "serve_streams.hip", "serve_recurrent.hip", "serve_talking.hip", "serve_differential.hip"]
 SERVE_FLAGS = FLAGS
 
 

@@ -178,7 +178,8 @@ __device__ __forceinline__ float glu(float g, float u, float limit) {
 // One workgroup per (token, chosen expert): act = relu(up_e . h)^2 (or the gated unit).  Dynamic LDS: D floats.  ff: weight rows.
 template <typename T, int ACT>
 __global__ __launch_bounds__(NT) void moe_up_kernel(T* __restrict__ act, const T* __restrict__ h, const T* __restrict__ up,
-                                                    const int32_t* __restrict__ idx, int top_k, int D, int ff, float limit, int n_experts) {
+                                                    const int32_t* __restrict__ idx, int top_k, int D, int ff, float limit, int n_experts,
+                                                        const float* __restrict__ in_weight) {
     extern __shared__ float xs[];
     const size_t slot = blockIdx.x;
     if (idx[slot] >= n_experts) return;                      // an identity expert: the down kernel adds the input itself
@@ -187,6 +188,7 @@ __global__ __launch_bounds__(NT) void moe_up_kernel(T* __restrict__ act, const T
     for (int i = threadIdx.x; i < D; i += NT) xs[i] = ld(h, t * D + i);
     __syncthreads();
     const T* W = up + (size_t)idx[slot] * ff * D;
+    const float iw = in_weight ? in_weight[slot] : 1.0f;     // the expert works on iw * h
     if (ACT == ACT_GLU) {
         for (int f = w; f < ff / 2; f += NW) {
             const T* r = W + (size_t)(2 * f) * D;
@@ -197,7 +199,7 @@ __global__ __launch_bounds__(NT) void moe_up_kernel(T* __restrict__ act, const T
             }
             d = wave_sum(d);
             e = wave_sum(e);
-            if (lane == 0) st(act, slot * (ff / 2) + f, glu(d, e, limit));
+            if (lane == 0) st(act, slot * (ff / 2) + f, glu(iw * d, iw * e, limit));
         }
         return;
     }
@@ -206,7 +208,7 @@ __global__ __launch_bounds__(NT) void moe_up_kernel(T* __restrict__ act, const T
         float d = 0.f;
         for (int i = lane; i < D; i += 64) d += ld(r, i) * xs[i];
         d = wave_sum(d);
-        if (lane == 0) st(act, slot * ff + f, relu_sq(d));
+        if (lane == 0) st(act, slot * ff + f, relu_sq(iw * d));
     }
 }
 
@@ -224,13 +226,13 @@ __global__ __launch_bounds__(NT) void moe_down_kernel(T* __restrict__ y, const T
         float total = 0.f;
         for (int k = 0; k < top_k; ++k) {
             if (idx[t * top_k + k] >= n_experts) {           // identity expert
-                total += weight[t * top_k + k] * ld(h, t * D + d);
+                total += (weight ? weight[t * top_k + k] : 1.0f) * ld(h, t * D + d);
                 continue;
             }
             const T* r = down + ((size_t)idx[t * top_k + k] * D + d) * ff;
             float v = 0.f;
             for (int i = lane; i < ff; i += 64) v += ld(r, i) * as[k * ff + i];
-            total += weight[t * top_k + k] * wave_sum(v);
+            total += (weight ? weight[t * top_k + k] : 1.0f) * wave_sum(v);
         }
         if (lane == 0) st(y, t * D + d, total);
     }
@@ -242,7 +244,8 @@ constexpr int ROWS = 4;      // output rows a wave works on at once
 
 template <typename T, int ACT>
 __global__ __launch_bounds__(NT) void moe_up_vec_kernel(T* __restrict__ act, const T* __restrict__ h, const T* __restrict__ up,
-                                                        const int32_t* __restrict__ idx, int top_k, int D, int ff, float limit, int n_experts) {
+                                                        const int32_t* __restrict__ idx, int top_k, int D, int ff, float limit, int n_experts,
+                                                        const float* __restrict__ in_weight) {
     extern __shared__ float xs[];
     const size_t slot = blockIdx.x;
     if (idx[slot] >= n_experts) return;                      // an identity expert: the down kernel adds the input itself
@@ -251,6 +254,7 @@ __global__ __launch_bounds__(NT) void moe_up_vec_kernel(T* __restrict__ act, con
     for (int i = threadIdx.x; i < D; i += NT) xs[i] = ld(h, t * D + i);
     __syncthreads();
     const T* W = up + (size_t)idx[slot] * ff * D;
+    const float iw = in_weight ? in_weight[slot] : 1.0f;     // the expert works on iw * h
     for (int f0 = w * ROWS; f0 < ff; f0 += NW * ROWS) {
         float acc[ROWS] = {0.f, 0.f, 0.f, 0.f};
         for (int c = lane * 8; c < D; c += 64 * 8) {
@@ -269,7 +273,7 @@ __global__ __launch_bounds__(NT) void moe_up_vec_kernel(T* __restrict__ act, con
         }
         float d[ROWS];
 #pragma unroll
-        for (int r = 0; r < ROWS; ++r) d[r] = wave_sum(acc[r]);
+        for (int r = 0; r < ROWS; ++r) d[r] = iw * wave_sum(acc[r]);
         if (lane == 0) {
             if (ACT == ACT_GLU) {                               // (ROWS and ff are even: a pair never straddles two waves)
 #pragma unroll
@@ -296,7 +300,7 @@ __global__ __launch_bounds__(NT) void moe_down_vec_kernel(T* __restrict__ y, con
     for (int d0 = w * ROWS; d0 < D; d0 += NW * ROWS) {
         float acc[ROWS] = {0.f, 0.f, 0.f, 0.f};
         for (int k = 0; k < top_k; ++k) {
-            const float wk = weight[t * top_k + k];
+            const float wk = weight ? weight[t * top_k + k] : 1.0f;
             if (idx[t * top_k + k] >= n_experts) {           // identity expert: lane 0's share carries the input (the rest add zero)
                 if (lane == 0) {
 #pragma unroll
@@ -339,7 +343,8 @@ typedef __bf16 bf2 __attribute__((ext_vector_type(2)));
 template <int KI, int ACT>
 __global__ __launch_bounds__(NT) void expert_rows_kernel(bf16_t* __restrict__ out, const bf16_t* __restrict__ X,
                                                          const int64_t* __restrict__ x_index, int div, const bf16_t* __restrict__ W,
-                                                         const int64_t* __restrict__ offsets, int rows, int K, float limit) {
+                                                         const int64_t* __restrict__ offsets, int rows, int K, float limit,
+                                                         const float* __restrict__ in_weight) {
     const int e = blockIdx.y;
     const int64_t s0 = offsets[e], s1 = offsets[e + 1];
     if (s0 == s1) return;                                                   // nobody chose this expert
@@ -387,6 +392,11 @@ __global__ __launch_bounds__(NT) void expert_rows_kernel(bf16_t* __restrict__ ou
                 float d[ROWS];
 #pragma unroll
                 for (int r = 0; r < ROWS; ++r) d[r] = wave_sum(acc[r]);
+                if (in_weight) {                                            // the expert works on weight * input
+                    const float iw = in_weight[x_index ? x_index[sb + j] : sb + j];
+#pragma unroll
+                    for (int r = 0; r < ROWS; ++r) d[r] *= iw;
+                }
                 if (lane == 0) {
                     if (ACT == ACT_GLU) {
 #pragma unroll
@@ -420,7 +430,7 @@ __global__ __launch_bounds__(NT) void relu_sq_kernel(T* __restrict__ a, size_t n
         st(a, i, v * v);
     }
 }
-// y[t] = sum_k weight[t, k] * ys[inv[t top_k + k]]
+// y[t] = sum_k weight[t, k] * ys[inv[t top_k + k]]   (weight NULL: ones)
 template <typename T>
 __global__ __launch_bounds__(NT) void moe_combine_kernel(T* __restrict__ y, const T* __restrict__ ys, const int64_t* __restrict__ inv,
                                                          const float* __restrict__ weight, int top_k, int D,
@@ -430,7 +440,7 @@ __global__ __launch_bounds__(NT) void moe_combine_kernel(T* __restrict__ y, cons
         float a = 0.f;
         for (int k = 0; k < top_k; ++k) {
             const bool same = idx && idx[t * top_k + k] >= n_experts;       // an identity expert's slot has no sorted row
-            a += weight[t * top_k + k] * (same ? ld(h, t * D + c) : ld(ys, (size_t)inv[t * top_k + k] * D + c));
+            a += (weight ? weight[t * top_k + k] : 1.0f) * (same ? ld(h, t * D + c) : ld(ys, (size_t)inv[t * top_k + k] * D + c));
         }
         st(y, t * D + c, a);
     }
@@ -449,7 +459,7 @@ extern "C" int qsv_gather_rows(void* out, const void* src, const int64_t* order,
 // out[s, r] = act(W[e][r, :] . X[x_index ? x_index[s] / div : s, :]) for the sorted slots s in [offsets[e], offsets[e + 1]) of every
 // expert e; W [E, rows, K] bfloat16, act: 0 nothing, 1 relu^2, 2 gated unit (row pairs; out is rows / 2 wide).  K % 8 == 0, K <= 4096.
 extern "C" int qsv_expert_rows(void* out, const void* X, const int64_t* x_index, int div, const void* W, const int64_t* offsets,
-                               int n_experts, int rows, int K, int act, float limit, void* stream) {
+                               int n_experts, int rows, int K, int act, float limit, const float* in_weight, void* stream) {
     QSV_REQUIRE(out && X && W && offsets && n_experts > 0 && rows > 0 && div > 0, "qsv_expert_rows: bad arguments");
     QSV_REQUIRE(act == ACT_NONE || act == ACT_RELU_SQ || ((act == ACT_GLU || act == QSV_ACT_CLAMPED_GLU) && rows % 2 == 0),
                 "qsv_expert_rows: activation %d", act);
@@ -463,13 +473,13 @@ extern "C" int qsv_expert_rows(void* out, const void* X, const int64_t* x_index,
     do {                                                                                                                     \
         if (act == ACT_RELU_SQ)                                                                                              \
             hipLaunchKernelGGL((expert_rows_kernel<KI, ACT_RELU_SQ>), grid, block, 0, (hipStream_t)stream, (bf16_t*)out,         \
-                               (const bf16_t*)X, x_index, div, (const bf16_t*)W, offsets, rows, K, limit);                          \
+                               (const bf16_t*)X, x_index, div, (const bf16_t*)W, offsets, rows, K, limit, in_weight);                          \
         else if (act == ACT_GLU)                                                                                             \
             hipLaunchKernelGGL((expert_rows_kernel<KI, ACT_GLU>), grid, block, 0, (hipStream_t)stream, (bf16_t*)out,             \
-                               (const bf16_t*)X, x_index, div, (const bf16_t*)W, offsets, rows, K, limit);                          \
+                               (const bf16_t*)X, x_index, div, (const bf16_t*)W, offsets, rows, K, limit, in_weight);                          \
         else                                                                                                                 \
             hipLaunchKernelGGL((expert_rows_kernel<KI, ACT_NONE>), grid, block, 0, (hipStream_t)stream, (bf16_t*)out,            \
-                               (const bf16_t*)X, x_index, div, (const bf16_t*)W, offsets, rows, K, limit);                          \
+                               (const bf16_t*)X, x_index, div, (const bf16_t*)W, offsets, rows, K, limit, in_weight);                          \
     } while (0)
     if (K <= 512) QSV_ER(1);
     else if (K <= 1024) QSV_ER(2);
@@ -488,7 +498,7 @@ extern "C" int qsv_relu_sq(void* a, int64_t n, int dtype, void* stream) {
 }
 extern "C" int qsv_moe_combine(void* y, const void* ys, const int64_t* inv, const float* weight, int n, int top_k, int D,
                                const int32_t* idx, const void* h, int n_experts, int dtype, void* stream) {
-    QSV_REQUIRE(y && ys && inv && weight && n >= 0 && top_k > 0 && D > 0 && (!idx || h), "qsv_moe_combine: bad arguments");
+    QSV_REQUIRE(y && ys && inv && n >= 0 && top_k > 0 && D > 0 && (!idx || h), "qsv_moe_combine: bad arguments");
     if (n == 0) return QSV_OK;
     QSV_DISPATCH(dtype, "qsv_moe_combine",
                  hipLaunchKernelGGL(moe_combine_kernel<T>, dim3(n), dim3(NT), 0, (hipStream_t)stream, (T*)y, (const T*)ys, inv,
@@ -514,7 +524,7 @@ extern "C" int qsv_moe_route(int32_t* idx, float* weight, const void* h, const v
 }
 
 extern "C" int qsv_moe_up(void* act, const void* h, const void* up, const int32_t* idx, int n, int top_k, int D, int ff,
-                          int activation, float limit, int n_experts, int dtype, void* stream) {
+                          int activation, float limit, int n_experts, const float* in_weight, int dtype, void* stream) {
     QSV_REQUIRE(act && h && up && idx && n >= 0 && top_k > 0 && D > 0 && ff > 0 && n_experts > 0, "qsv_moe_up: bad arguments");
     QSV_REQUIRE(activation == ACT_RELU_SQ || ((activation == ACT_GLU || activation == QSV_ACT_CLAMPED_GLU) && ff % 2 == 0),
                 "qsv_moe_up: activation %d over %d rows", activation, ff);
@@ -526,7 +536,7 @@ extern "C" int qsv_moe_up(void* act, const void* h, const void* up, const int32_
 #define QSV_UP(KERNEL, ACT)                                                                                                  \
     QSV_DISPATCH(dtype, "qsv_moe_up",                                                                                        \
                  hipLaunchKernelGGL((KERNEL<T, ACT>), dim3(n * top_k), dim3(NT), (size_t)D * 4, (hipStream_t)stream, (T*)act,   \
-                                    (const T*)h, (const T*)up, idx, top_k, D, ff, limit, n_experts))
+                                    (const T*)h, (const T*)up, idx, top_k, D, ff, limit, n_experts, in_weight))
     if (D % 8 == 0) {
         if (activation == ACT_GLU) QSV_UP(moe_up_vec_kernel, ACT_GLU);
         else QSV_UP(moe_up_vec_kernel, ACT_RELU_SQ);
@@ -540,7 +550,7 @@ extern "C" int qsv_moe_up(void* act, const void* h, const void* up, const int32_
 
 extern "C" int qsv_moe_down(void* y, const void* act, const void* down, const int32_t* idx, const float* weight, int n,
                             int top_k, int D, int ff, const void* h, int n_experts, int dtype, void* stream) {
-    QSV_REQUIRE(y && act && down && idx && weight && h && n >= 0 && top_k > 0 && D > 0 && ff > 0 && n_experts > 0,
+    QSV_REQUIRE(y && act && down && idx && h && n >= 0 && top_k > 0 && D > 0 && ff > 0 && n_experts > 0,
                 "qsv_moe_down: bad arguments");
     QSV_REQUIRE((size_t)top_k * ff * 4 <= 64 * 1024, "qsv_moe_down: %d x %d activations do not fit the workgroup's LDS", top_k, ff);
     if (n == 0) return QSV_OK;

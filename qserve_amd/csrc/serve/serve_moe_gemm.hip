@@ -31,7 +31,7 @@ template <int ACT>
 __global__ __launch_bounds__(256, 2) void grouped_gemm_kernel(bf16_t* __restrict__ out, const bf16_t* __restrict__ X,
                                                            const int64_t* __restrict__ x_index, int div,
                                                            const bf16_t* __restrict__ W, const int32_t* __restrict__ tiles, int N,
-                                                           int K, float limit) {
+                                                           int K, float limit, const float* __restrict__ in_weight) {
     __shared__ __attribute__((aligned(16))) bf16_t As[BNW * LS];
     __shared__ __attribute__((aligned(16))) bf16_t Bs[BS * LS];
     const int tid = threadIdx.x, lane = tid & 63, w = tid >> 6;
@@ -105,11 +105,13 @@ __global__ __launch_bounds__(256, 2) void grouped_gemm_kernel(bf16_t* __restrict
     for (int nt = 0; nt < BS / 16; ++nt) {
         const int sl = 16 * nt + col;
         if (sl >= ns) continue;
+        float iw = 1.0f;                                            // the expert works on iw * input
+        if (in_weight) iw = in_weight[x_index ? x_index[s_first + sl] : s_first + sl];
 #pragma unroll
         for (int mt = 0; mt < MT; ++mt) {
             const int n = n0 + 16 * MT * w + 16 * mt + 4 * g4;
             if (n >= N) continue;                                   // N % 4 == 0: the four rows are inside together
-            v4f v = acc[mt][nt];
+            v4f v = acc[mt][nt] * iw;
             if (ACT == 2) {
                 float u0, u1;
                 if (limit > 0.f) {                                  // clamped units: g sigmoid(1.702 g) (u + 1) (uniform over the launch)
@@ -142,7 +144,7 @@ __global__ __launch_bounds__(256, 2) void grouped_gemm_kernel(bf16_t* __restrict
 extern "C" int qsv_grouped_gemm_tile_slots(void) { return BS; }
 extern "C" int qsv_grouped_gemm_k_step(void) { return KS; }
 extern "C" int qsv_grouped_gemm(void* out, const void* X, const int64_t* x_index, int div, const void* W, const int32_t* tiles,
-                                int n_tiles, int N, int K, int act, float limit, void* stream) {
+                                int n_tiles, int N, int K, int act, float limit, const float* in_weight, void* stream) {
     QSV_REQUIRE(out && X && W && tiles && div > 0 && n_tiles >= 0, "qsv_grouped_gemm: bad arguments");
     QSV_REQUIRE(N > 0 && N % 4 == 0 && K > 0 && K % KS == 0, "qsv_grouped_gemm: N %d (a multiple of 4), K %d (a multiple of 64)", N, K);
     QSV_REQUIRE(n_tiles <= 65535, "qsv_grouped_gemm: %d tiles (at most 65535 per launch)", n_tiles);
@@ -154,7 +156,7 @@ extern "C" int qsv_grouped_gemm(void* out, const void* X, const int64_t* x_index
     const dim3 grid((N + BNW - 1) / BNW, n_tiles), block(256);
 #define QSV_GG(ACT)                                                                                                          \
     hipLaunchKernelGGL(grouped_gemm_kernel<ACT>, grid, block, 0, (hipStream_t)stream, (bf16_t*)out, (const bf16_t*)X, x_index, div, \
-                       (const bf16_t*)W, tiles, N, K, limit)
+                       (const bf16_t*)W, tiles, N, K, limit, in_weight)
     if (act == QSV_ACT_RELU_SQ) QSV_GG(1);
     else if (act == QSV_ACT_GLU) QSV_GG(2);
     else QSV_GG(0);

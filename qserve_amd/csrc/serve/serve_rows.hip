@@ -341,9 +341,104 @@ extern "C" int qsv_add_rms_norm(float* x, void* h, const void* a, const void* b,
     return qsv_launch_status("qsv_add_rms_norm");
 }
 
+// ---- x += s0 a + s1 b + s2 c (element-wise scales); h0 = rms_norm(x) * g0, h1 = rms_norm(x) * g1 -------------------------------------------
+// The parallel layer with a norm of its own for each side: one statistic, two gains (float, one per coordinate).  tokens: x starts as the
+// embedding row.  a, b, c (storage type), their scales and h1 may be NULL; h0 == NULL: the sum only.
+struct ScaledParts {
+    const void *y[3], *s[3];
+};
+template <typename T, int VPT>
+__global__ __launch_bounds__(NT) void scaled_sum_rms_norms_vec_kernel(float* __restrict__ x, T* __restrict__ h0, T* __restrict__ h1, ScaledParts p,
+                                                                      const float* __restrict__ g0, const float* __restrict__ g1,
+                                                                      const int32_t* __restrict__ tokens, const T* __restrict__ table, float eps, int D) {
+    __shared__ float red[NT / 64 + 1];
+    const size_t t = blockIdx.x;
+    float4 v[VPT];
+    float s = 0.f;
+#pragma unroll
+    for (int k = 0; k < VPT; ++k) {
+        const int i = (threadIdx.x + k * NT) * 4;
+        if (i >= D) continue;
+        v[k] = tokens ? ld4v(table, (size_t)tokens[t] * D + i) : ld4v(x, t * D + i);
+        float4 y = make_float4(0.f, 0.f, 0.f, 0.f);
+#pragma unroll
+        for (int j = 0; j < 3; ++j)
+            if (p.y[j]) {
+                const float4 z = ld4v((const T*)p.y[j], t * D + i);
+                const float4 f = p.s[j] ? ld4v((const T*)p.s[j], i) : make_float4(1.f, 1.f, 1.f, 1.f);
+                y.x += f.x * z.x; y.y += f.y * z.y; y.z += f.z * z.z; y.w += f.w * z.w;
+            }
+        v[k].x += y.x; v[k].y += y.y; v[k].z += y.z; v[k].w += y.w;
+        st4v(x, t * D + i, v[k]);
+        s += v[k].x * v[k].x + v[k].y * v[k].y + v[k].z * v[k].z + v[k].w * v[k].w;
+    }
+    if (!h0) return;
+    const float inv = 1.0f / sqrtf(block_sum<NT>(s, red) / (float)D + eps);
+#pragma unroll
+    for (int k = 0; k < VPT; ++k) {
+        const int i = (threadIdx.x + k * NT) * 4;
+        if (i >= D) continue;
+        const float4 n = make_float4(v[k].x * inv, v[k].y * inv, v[k].z * inv, v[k].w * inv);
+        const float4 a = ld4v(g0, i);
+        st4v(h0, t * D + i, make_float4(n.x * a.x, n.y * a.y, n.z * a.z, n.w * a.w));
+        if (h1) {
+            const float4 b = ld4v(g1, i);
+            st4v(h1, t * D + i, make_float4(n.x * b.x, n.y * b.y, n.z * b.z, n.w * b.w));
+        }
+    }
+}
 template <typename T>
+__global__ __launch_bounds__(NT) void scaled_sum_rms_norms_kernel(float* __restrict__ x, T* __restrict__ h0, T* __restrict__ h1, ScaledParts p,
+                                                                  const float* __restrict__ g0, const float* __restrict__ g1,
+                                                                  const int32_t* __restrict__ tokens, const T* __restrict__ table, float eps, int D) {
+    __shared__ float red[NT / 64 + 1];
+    const size_t t = blockIdx.x;
+    float s = 0.f;
+    for (int i = threadIdx.x; i < D; i += NT) {
+        float v = tokens ? ld(table, (size_t)tokens[t] * D + i) : x[t * D + i], y = 0.f;
+#pragma unroll
+        for (int j = 0; j < 3; ++j)
+            if (p.y[j]) y += (p.s[j] ? ld((const T*)p.s[j], i) : 1.f) * ld((const T*)p.y[j], t * D + i);
+        v += y;
+        x[t * D + i] = v;
+        s += v * v;
+    }
+    if (!h0) return;
+    const float inv = 1.0f / sqrtf(block_sum<NT>(s, red) / (float)D + eps);
+    for (int i = threadIdx.x; i < D; i += NT) {
+        const float n = x[t * D + i] * inv;              // (this thread's own writes)
+        st(h0, t * D + i, n * g0[i]);
+        if (h1) st(h1, t * D + i, n * g1[i]);
+    }
+}
+extern "C" int qsv_scaled_sum_rms_norms(float* x, void* h0, void* h1, const void* a, const void* sa, const void* b, const void* sb, const void* c,
+                                        const void* sc, const float* g0, const float* g1, const int32_t* tokens, const void* table, float eps,
+                                        int n, int D, int dtype, void* stream) {
+    QSV_REQUIRE(x && n >= 0 && D > 0 && (!h0 || g0) && (!h1 || (h0 && g1)) && (!tokens || table), "qsv_scaled_sum_rms_norms: bad arguments");
+    if (n == 0) return QSV_OK;
+    const ScaledParts p = {{a, b, c}, {sa, sb, sc}};
+    const int vecs = (D / 4 + NT - 1) / NT;
+#define QSV_SSN(V)                                                                                                                 \
+    QSV_DISPATCH(dtype, "qsv_scaled_sum_rms_norms",                                                                                \
+                 hipLaunchKernelGGL((scaled_sum_rms_norms_vec_kernel<T, V>), dim3(n), dim3(NT), 0, (hipStream_t)stream, x, (T*)h0, (T*)h1, p, g0, \
+                                    g1, tokens, (const T*)table, eps, D))
+    if (D % 4 == 0 && vecs <= 8) {
+        if (vecs <= 1) QSV_SSN(1);
+        else if (vecs <= 2) QSV_SSN(2);
+        else if (vecs <= 4) QSV_SSN(4);
+        else QSV_SSN(8);
+    } else {
+        QSV_DISPATCH(dtype, "qsv_scaled_sum_rms_norms",
+                     hipLaunchKernelGGL(scaled_sum_rms_norms_kernel<T>, dim3(n), dim3(NT), 0, (hipStream_t)stream, x, (T*)h0, (T*)h1, p, g0, g1,
+                                        tokens, (const T*)table, eps, D));
+    }
+#undef QSV_SSN
+    return qsv_launch_status("qsv_scaled_sum_rms_norms");
+}
+
+template <typename T, typename TW>
 __global__ __launch_bounds__(NT) void rms_norm_rows_kernel(T* __restrict__ out, const float* __restrict__ x,
-                                                           const int32_t* __restrict__ rows, const T* __restrict__ w, float eps,
+                                                           const int32_t* __restrict__ rows, const TW* __restrict__ w, float eps,
                                                            int D) {
     __shared__ float red[NT / 64 + 1];
     const size_t r = blockIdx.x;
@@ -353,13 +448,17 @@ __global__ __launch_bounds__(NT) void rms_norm_rows_kernel(T* __restrict__ out, 
     const float inv = 1.0f / sqrtf(block_sum<NT>(s, red) / (float)D + eps);
     for (int i = threadIdx.x; i < D; i += NT) st(out, r * D + i, xr[i] * inv * ld(w, i));
 }
-extern "C" int qsv_rms_norm_rows(void* out, const float* x, const int32_t* rows, const void* w, float eps, int n, int D, int dtype,
-                                 void* stream) {
-    QSV_REQUIRE(out && x && w && n >= 0 && D > 0, "qsv_rms_norm_rows: bad arguments");
+extern "C" int qsv_rms_norm_rows(void* out, const float* x, const int32_t* rows, const void* w, int w_dtype, float eps, int n, int D,
+                                 int dtype, void* stream) {
+    QSV_REQUIRE(out && x && w && n >= 0 && D > 0 && (w_dtype == dtype || w_dtype == QSV_F32), "qsv_rms_norm_rows: bad arguments");
     if (n == 0) return QSV_OK;
-    QSV_DISPATCH(dtype, "qsv_rms_norm_rows",
-                 hipLaunchKernelGGL(rms_norm_rows_kernel<T>, dim3(n), dim3(NT), 0, (hipStream_t)stream, (T*)out, x, rows, (const T*)w,
-                                    eps, D));
+    if (w_dtype == QSV_F32)
+        QSV_DISPATCH(dtype, "qsv_rms_norm_rows",
+                     hipLaunchKernelGGL((rms_norm_rows_kernel<T, float>), dim3(n), dim3(NT), 0, (hipStream_t)stream, (T*)out, x, rows,
+                                        (const float*)w, eps, D));
+    else
+        hipLaunchKernelGGL((rms_norm_rows_kernel<bf16_t, bf16_t>), dim3(n), dim3(NT), 0, (hipStream_t)stream, (bf16_t*)out, x, rows,
+                           (const bf16_t*)w, eps, D);
     return qsv_launch_status("qsv_rms_norm_rows");
 }
 
@@ -535,6 +634,9 @@ extern "C" int qsv_add_normed_rms_norm(float* x, void* h, const void* y, const v
 // ---- query / key norms (per head or over the projection), rotated pairs, cache write -----------------------------------------------
 // q_b / k_b / v_b (each may be NULL) are added to the projections first; the pairs are neighbours or, with `halves`, (i, i + rot_n / 2);
 // head_scale (may be NULL) multiplies the common scale; a query row starts with q_pad zeros.  One workgroup per token.  Statistics: per head a wave's sum over `dim`; over the projection a workgroup sum.  The rotation works
+// (rot_gain > 0, per-head norms only: the norm follows the rotation - its statistic is taken before it, the rotated dimensions weighted by
+// rot_gain, the square of the magnitude cos and sin carry, and the turned values are scaled; no weights: q_w, k_w NULL; q_out: the queries
+// leave in the storage type)
 // on normed values staged in LDS (a pair's two values may sit in different threads).  Dynamic LDS: (heads + kv_heads) * dim floats.
 // VEC (every size, stride and address a multiple of four elements, dim <= 256): four elements per lane, dim / 4 lanes (rounded up to a
 // power of two, `lph`) per head for the per-head statistics, 16-byte stores.
@@ -548,7 +650,8 @@ __global__ __launch_bounds__(NT) void qk_norm_rope_prep_kernel(float* __restrict
                                                                const int64_t* __restrict__ slot, const int32_t* __restrict__ pos,
                                                                const T* __restrict__ q_b, const T* __restrict__ k_b,
                                                                const T* __restrict__ v_b, int halves,
-                                                               const float* __restrict__ head_scale, int q_pad, int lph) {
+                                                               const float* __restrict__ head_scale, int q_pad, int lph,
+                                                               float rot_gain, T* __restrict__ q_out) {
     extern __shared__ __attribute__((aligned(16))) float sm[];
     __shared__ float red[NT / 64 + 1];
     const size_t t = blockIdx.x;
@@ -571,11 +674,16 @@ __global__ __launch_bounds__(NT) void qk_norm_rope_prep_kernel(float* __restrict
                     u.x += b.x; u.y += b.y; u.z += b.z; u.w += b.w;
                 }
             }
-            float s = u.x * u.x + u.y * u.y + u.z * u.z + u.w * u.w;
+            float s;
+            if (rot_gain > 0.f)
+                s = (e < rot_n ? rot_gain : 1.f) * u.x * u.x + (e + 1 < rot_n ? rot_gain : 1.f) * u.y * u.y +
+                    (e + 2 < rot_n ? rot_gain : 1.f) * u.z * u.z + (e + 3 < rot_n ? rot_gain : 1.f) * u.w * u.w;
+            else
+                s = u.x * u.x + u.y * u.y + u.z * u.z + u.w * u.w;
             for (int o = lph >> 1; o > 0; o >>= 1) s += __shfl_xor(s, o, 64);
             const float inv = 1.0f / sqrtf(s / (float)dim + eps);
             if (ok) {
-                const float4 g = ld4v(isq ? q_w : k_w, e);
+                const float4 g = q_w ? ld4v(isq ? q_w : k_w, e) : make_float4(1.f, 1.f, 1.f, 1.f);
                 *(float4*)(nq + h0 * dim + e) = make_float4(u.x * (inv * g.x), u.y * (inv * g.y), u.z * (inv * g.z), u.w * (inv * g.w));
             }
         }
@@ -590,10 +698,10 @@ __global__ __launch_bounds__(NT) void qk_norm_rope_prep_kernel(float* __restrict
             for (int e = lane; e < dim; e += 64) {
                 const float u = ld(src, e) + (bias ? ld(bias, b0 + e) : 0.f);
                 nq[hh * dim + e] = u;
-                s += u * u;
+                s += (rot_gain > 0.f && e < rot_n ? rot_gain : 1.f) * u * u;
             }
             const float inv = 1.0f / sqrtf(wave_sum(s) / (float)dim + eps);
-            for (int e = lane; e < dim; e += 64) nq[hh * dim + e] *= inv * ld(w, e);
+            for (int e = lane; e < dim; e += 64) nq[hh * dim + e] *= q_w ? inv * ld(w, e) : inv;
         }
     } else {
         float s = 0.f;
@@ -640,7 +748,8 @@ __global__ __launch_bounds__(NT) void qk_norm_rope_prep_kernel(float* __restrict
                 const float f = head_scale ? scale * head_scale[h] : scale;
                 v.x *= f; v.y *= f; v.z *= f; v.w *= f;
             }
-            st4v(qf, t * H * (size_t)RQ + (size_t)idx * 4, v);
+            if (q_out) st4v(q_out, t * H * (size_t)RQ + (size_t)idx * 4, v);
+            else st4v(qf, t * H * (size_t)RQ + (size_t)idx * 4, v);
         }
         if (!k) return;
         const size_t row = (size_t)slot[t];
@@ -662,7 +771,9 @@ __global__ __launch_bounds__(NT) void qk_norm_rope_prep_kernel(float* __restrict
     }
     for (int idx = threadIdx.x; idx < H * RQ; idx += NT) {
         const int h = idx / RQ, c = idx - h * RQ;
-        qf[t * H * (size_t)RQ + idx] = c < q_pad ? 0.f : nq[h * dim + c - q_pad] * (head_scale ? scale * head_scale[h] : scale);
+        const float qv = c < q_pad ? 0.f : nq[h * dim + c - q_pad] * (head_scale ? scale * head_scale[h] : scale);
+        if (q_out) st(q_out, t * H * (size_t)RQ + idx, qv);
+        else qf[t * H * (size_t)RQ + idx] = qv;
     }
     if (!k) return;
     const size_t dst = (size_t)slot[t];
@@ -673,13 +784,17 @@ __global__ __launch_bounds__(NT) void qk_norm_rope_prep_kernel(float* __restrict
            c < vdim ? ld(vrow, g * vdim + c) + (v_b ? ld(v_b, g * vdim + c) : 0.f) : nq[(H + g) * dim + c - vdim]);
     }
 }
-extern "C" int qsv_qk_norm_rope_prep(float* qf, const void* q, int64_t q_stride, const void* k, int64_t k_stride, const void* v,
+extern "C" int qsv_qk_norm_rope_prep(void* qf, const void* q, int64_t q_stride, const void* k, int64_t k_stride, const void* v,
                                      int64_t v_stride, int qkv_dtype, int heads, int kv_heads, int dim, int vdim, const void* q_w,
                                      const void* k_w, int per_head, float eps, const float* rope, int rot_n, float scale, void* pool,
                                      int64_t pool_rows, const int64_t* slot, const int32_t* pos, int n, const void* q_b, const void* k_b,
-                                     const void* v_b, int halves, const float* head_scale, int q_pad, int dtype, void* stream) {
-    QSV_REQUIRE(qf && q && q_w && pos, "qsv_qk_norm_rope_prep: null argument");
-    QSV_REQUIRE(!k || (v && k_w && pool && slot), "qsv_qk_norm_rope_prep: keys without values, weight, pool or rows");
+                                     const void* v_b, int halves, const float* head_scale, int q_pad, float rot_gain, int q_store,
+                                     int dtype, void* stream) {
+    QSV_REQUIRE(qf && q && pos, "qsv_qk_norm_rope_prep: null argument");
+    QSV_REQUIRE(!k || (v && pool && slot && !k_w == !q_w), "qsv_qk_norm_rope_prep: keys without values, weight, pool or rows");
+    QSV_REQUIRE(q_w || per_head, "qsv_qk_norm_rope_prep: a norm over the projection without its weight");
+    QSV_REQUIRE(!(rot_gain > 0.f) || (per_head && !q_w), "qsv_qk_norm_rope_prep: a norm behind the rotation is per head and has no weight");
+    if (!rope) rot_n = 0;
     QSV_REQUIRE(heads > 0 && kv_heads > 0 && dim > 0 && vdim > 0 && n >= 0 && q_pad >= 0 && q_stride >= (int64_t)heads * dim &&
                     (!k || (k_stride >= (int64_t)kv_heads * dim && v_stride >= (int64_t)kv_heads * vdim)),
                 "qsv_qk_norm_rope_prep: bad sizes");
@@ -698,10 +813,11 @@ extern "C" int qsv_qk_norm_rope_prep(float* qf, const void* q, int64_t q_stride,
     while (lph * 4 < dim) lph <<= 1;
 #define QSV_QKP(TI, VEC)                                                                                                         \
     QSV_DISPATCH(dtype, "qsv_qk_norm_rope_prep",                                                                                 \
-                 hipLaunchKernelGGL((qk_norm_rope_prep_kernel<T, TI, VEC>), dim3(n), dim3(NT), lds, (hipStream_t)stream, qf, (const TI*)q, \
+                 hipLaunchKernelGGL((qk_norm_rope_prep_kernel<T, TI, VEC>), dim3(n), dim3(NT), lds, (hipStream_t)stream, q_store ? nullptr : (float*)qf, (const TI*)q, \
                                     q_stride, (const TI*)k, k_stride, (const TI*)v, v_stride, heads, kv_heads, dim, vdim,          \
                                     (const T*)q_w, (const T*)k_w, per_head, eps, rope, rot_n, scale, (T*)pool, pool_rows, slot, pos,  \
-                                    (const T*)q_b, (const T*)k_b, (const T*)v_b, halves, head_scale, q_pad, lph))
+                                    (const T*)q_b, (const T*)k_b, (const T*)v_b, halves, head_scale, q_pad, lph, rot_gain,              \
+                                    q_store ? (T*)qf : nullptr))
     if (vec) {
         if (qkv_dtype == QSV_F32) QSV_QKP(float, true);
         else QSV_QKP(bf16_t, true);

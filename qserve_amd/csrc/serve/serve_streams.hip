@@ -238,7 +238,7 @@ __global__ __launch_bounds__(NT) void rms_pair_mean_kernel(T* __restrict__ out, 
         st(out, t * D + i, 0.5f * (ld(a, t * D + i) * ia * ld(wa, i) + ld(b, t * D + i) * ib * ld(wb, i)));
 }
 
-// out[r, f] = act(a[r, 2f]) * a[r, 2f + 1];  act 0: silu, 1: gelu in its tanh form, 0.5 z (1 + tanh(sqrt(2 / pi) (z + 0.044715 z^3)));
+// out[r, f] = act(s a[r, 2f]) * s a[r, 2f + 1] with s = row_scale[scale_index ? scale_index[r] : r] (row_scale NULL: 1);  act 0: silu, 1: gelu in its tanh form, 0.5 z (1 + tanh(sqrt(2 / pi) (z + 0.044715 z^3)));
 // act 2: g = min(gate, limit), u = clamp(up, -limit, limit) -> g sigmoid(1.702 g) (u + 1)
 __device__ __forceinline__ float glu_unit(float g, float u, int act, float limit) {
     if (act == 2) {
@@ -250,21 +250,23 @@ __device__ __forceinline__ float glu_unit(float g, float u, int act, float limit
     return ag * u;
 }
 template <typename T, bool VEC>
-__global__ __launch_bounds__(NT) void glu_kernel(T* __restrict__ out, const T* __restrict__ a, int ff, int act, float limit) {
+__global__ __launch_bounds__(NT) void glu_kernel(T* __restrict__ out, const T* __restrict__ a, int ff, int act, float limit,
+                                                 const float* __restrict__ row_scale, const int64_t* __restrict__ scale_index) {
     const size_t r = blockIdx.x;
+    const float rs = row_scale ? row_scale[scale_index ? (size_t)scale_index[r] : r] : 1.0f;
     if (VEC) {                                                           // ff % 4 == 0: four units per thread and pass
         for (int f = threadIdx.x * 4; f < ff; f += NT * 4) {
             float p[4], q[4];
             ld4t(a, (r * ff + f) * 2, p);
             ld4t(a, (r * ff + f) * 2 + 4, q);
-            const float y[4] = {glu_unit(p[0], p[1], act, limit), glu_unit(p[2], p[3], act, limit), glu_unit(q[0], q[1], act, limit),
-                                glu_unit(q[2], q[3], act, limit)};
+            const float y[4] = {glu_unit(rs * p[0], rs * p[1], act, limit), glu_unit(rs * p[2], rs * p[3], act, limit),
+                                glu_unit(rs * q[0], rs * q[1], act, limit), glu_unit(rs * q[2], rs * q[3], act, limit)};
             st4t(out, r * ff + f, y);
         }
         return;
     }
     for (int f = threadIdx.x; f < ff; f += NT)
-        st(out, r * ff + f, glu_unit(ld(a, (r * ff + f) * 2), ld(a, (r * ff + f) * 2 + 1), act, limit));
+        st(out, r * ff + f, glu_unit(rs * ld(a, (r * ff + f) * 2), rs * ld(a, (r * ff + f) * 2 + 1), act, limit));
 }
 }  // namespace
 
@@ -338,16 +340,17 @@ extern "C" int qsv_rms_pair_mean(void* out, const void* a, const void* wa, const
     return qsv_launch_status("qsv_rms_pair_mean");
 }
 
-extern "C" int qsv_glu(void* out, const void* a, int n_rows, int ff, int act, float limit, int dtype, void* stream) {
+extern "C" int qsv_glu(void* out, const void* a, int n_rows, int ff, int act, float limit, const float* row_scale,
+                       const int64_t* scale_index, int dtype, void* stream) {
     QSV_REQUIRE(out && a && n_rows >= 0 && ff > 0 && (act == 0 || act == 1 || (act == 2 && limit > 0.f)), "qsv_glu: bad arguments");
     if (n_rows == 0) return QSV_OK;
     if (ff % 4 == 0)
         QSV_DISPATCH(dtype, "qsv_glu",
                      hipLaunchKernelGGL((glu_kernel<T, true>), dim3(n_rows), dim3(NT), 0, (hipStream_t)stream, (T*)out, (const T*)a, ff, act,
-                                        limit));
+                                        limit, row_scale, scale_index));
     else
         QSV_DISPATCH(dtype, "qsv_glu",
                      hipLaunchKernelGGL((glu_kernel<T, false>), dim3(n_rows), dim3(NT), 0, (hipStream_t)stream, (T*)out, (const T*)a, ff, act,
-                                        limit));
+                                        limit, row_scale, scale_index));
     return qsv_launch_status("qsv_glu");
 }

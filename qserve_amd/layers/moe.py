@@ -71,33 +71,43 @@ class TopKGatedMoE:
         return self.ops.moe_experts(h, self.up, self.down, idx, wt, act="swiglu")
 
 
-class CorrectedSigmoidMoE:
-    """Mixture of gated experts behind a sigmoid router with a choice correction: scores s = sigmoid(router . h) (float); experts
-    are CHOSEN by s + correction, inside the `keep` groups (of `groups` equal groups of neighbours) whose two largest corrected
-    scores sum highest; the chosen experts are WEIGHTED by their plain s times `scale` (no division by the chosen scores' sum).  Expert: down .
-    (silu(gate . h) * (up . h)).  An optional shared expert of the same form runs for every token.
+class SigmoidMoE:
+    """Mixture of gated experts behind a sigmoid router: scores s = sigmoid(router . h) (float).  The `top_k` experts with the largest s
+    (plus `correction`, where there is one: for the choice only) are chosen, inside the `keep` groups (of `groups` equal groups of
+    neighbours) whose two largest such scores sum highest, and WEIGHTED by their plain s times `scale` (no division by the chosen scores'
+    sum).  weigh "output": the weight multiplies the expert's output; "input": its input.  Expert: down . (silu(gate . h) * (up . h)).  An
+    optional shared expert of the same form runs for every token, unweighted.
     Returns the list of outputs to be summed ([routed] or [routed, shared]): the caller's residual kernel adds them in one pass."""
 
-    def __init__(self, ops, *, router, correction, gate, up, down, top_k, groups=1, keep=1, scale=1.0, shared=None):
-        """router [E, D], correction [E]; gate / up: lists of E [ff, D]; down: list of E [D, ff]; shared: a GatedFeedForward or None."""
+    def __init__(self, ops, *, router, gate, up, down, top_k, correction=None, groups=1, keep=1, scale=1.0, weigh="output", shared=None):
+        """router [E, D], correction [E] or None; gate / up: lists of E [ff, D]; down: list of E [D, ff]; shared: a GatedFeedForward or None."""
         self.ops = ops
-        self.router, self.correction = router.contiguous(), correction.float().contiguous()
+        self.router, self.correction = router.contiguous(), None if correction is None else correction.float().contiguous()
         self.up = _interleave(torch.stack(list(gate)), torch.stack(list(up)))          # [E, 2 ff, D]
         self.down = torch.stack(list(down)).contiguous()
         E, ff2, D = self.up.shape
-        self.top_k, self.groups, self.keep, self.scale, self.shared = int(top_k), int(groups), int(keep), float(scale), shared
-        if self.router.shape != (E, D) or self.correction.shape != (E,) or self.down.shape != (E, D, ff2 // 2):
+        self.top_k, self.groups, self.keep, self.scale, self.shared, self.weigh = int(top_k), int(groups), int(keep), float(scale), shared, weigh
+        if self.router.shape != (E, D) or self.down.shape != (E, D, ff2 // 2) or weigh not in ("input", "output"):
             raise ValueError("mixture of experts: router / expert shapes do not fit each other")
+        if self.correction is not None and self.correction.shape != (E,):
+            raise ValueError(f"mixture of experts: choice correction of shape {tuple(self.correction.shape)} for {E} experts")
         if E % self.groups or not 0 < self.keep <= self.groups or not 0 < self.top_k <= self.keep * (E // self.groups):
             raise ValueError(f"router: {E} experts, {self.groups} groups, keep {self.keep}, top {self.top_k}")
 
     def __call__(self, h):
         idx, wt = self.ops.moe_route(h, self.router, self.top_k, self.groups, self.keep, score="sigmoid", correction=self.correction,
                                      group_top=2, scale=self.scale)
-        y = [self.ops.moe_experts(h, self.up, self.down, idx, wt, act="swiglu")]
+        y = [self.ops.moe_experts(h, self.up, self.down, idx, wt, act="swiglu", weigh=self.weigh)]
         if self.shared is not None:
             y.append(self.shared(h))
         return y
+
+
+class CorrectedSigmoidMoE(SigmoidMoE):
+    """SigmoidMoE with a choice correction, weights on the outputs."""
+
+    def __init__(self, ops, *, correction, **kw):
+        super().__init__(ops, correction=correction, **kw)
 
 
 class ReluSquaredFeedForward:

@@ -217,13 +217,17 @@ class HipOps:
 
     GLU_ACTS = {"silu": 0, "gelu_tanh": 1, "clamped": 2}
 
-    def glu(self, a, act="silu", limit=0.0):
+    def glu(self, a, act="silu", limit=0.0, row_scale=None, scale_index=None):
         """a [n, 2 ff] with (gate, up) as neighbours -> act(gate) * up [n, ff]; act: silu, gelu_tanh (gelu in its tanh form), or
-        clamped: g = min(gate, limit), u = clamp(up, -limit, limit) -> g sigmoid(1.702 g) (u + 1)."""
+        clamped: g = min(gate, limit), u = clamp(up, -limit, limit) -> g sigmoid(1.702 g) (u + 1).  row_scale (float): row r
+        of a is first multiplied by row_scale[scale_index[r]] (scale_index int64, None: r)."""
         n, ff = a.size(0), a.size(1) // 2
         out = torch.empty((n, ff), dtype=self.dtype, device=a.device)
-        self._need(a)
-        self.check(self.L.qsv_glu(out.data_ptr(), a.data_ptr(), n, ff, self.GLU_ACTS[act], float(limit), self.code, self._s()), "glu")
+        self._need(a, row_scale, scale_index)
+        assert row_scale is None or row_scale.dtype == torch.float32
+        self.check(self.L.qsv_glu(out.data_ptr(), a.data_ptr(), n, ff, self.GLU_ACTS[act], float(limit),
+                                  0 if row_scale is None else row_scale.data_ptr(), 0 if scale_index is None else scale_index.data_ptr(),
+                                  self.code, self._s()), "glu")
         return out
 
     # ---- sinusoidal positions, RMS-normed residual, whole-projection query / key norms ----------------------------------------------
@@ -250,12 +254,33 @@ class HipOps:
         return h
 
     def rms_norm_rows(self, x, rows, w, eps):
+        """w: storage type or float."""
         n = x.size(0) if rows is None else rows.numel()
         out = torch.empty((n, x.size(1)), dtype=self.dtype, device=x.device)
         self._need(x, rows, w)
         self.check(self.L.qsv_rms_norm_rows(out.data_ptr(), x.data_ptr(), 0 if rows is None else rows.data_ptr(), w.data_ptr(),
-                                            float(eps), n, x.size(1), self.code, self._s()), "rms_norm_rows")
+                                            dtype_code(w.dtype), float(eps), n, x.size(1), self.code, self._s()), "rms_norm_rows")
         return out
+
+    def scaled_sum_rms_norms(self, x, parts, gains, eps, tokens=None, table=None):
+        """x += sum of scale * y over parts [(y, scale)] (up to three; y storage type, scale per coordinate in the storage type or None) in
+        place, or, with tokens, x <- table[tokens] (+ the parts; x None: made here); -> (x, [rms_norm(x) * g in the storage type for the (up to
+        two) float gains g]), all from one statistic."""
+        assert len(parts) <= 3 and len(gains) <= 2
+        if tokens is not None and x is None:
+            x = torch.empty((tokens.numel(), table.size(1)), dtype=torch.float32, device=table.device)
+        T, D = x.shape
+        hs = [torch.empty((T, D), dtype=self.dtype, device=x.device) for _ in gains]
+        self._need(x, tokens, table, *gains, *[v for p in parts for v in p])
+        assert x.dtype == torch.float32 and all(g.dtype == torch.float32 and g.numel() == D for g in gains)
+        for y, s in parts:
+            assert y.shape == x.shape and y.dtype == self.dtype and (s is None or (s.dtype == self.dtype and s.numel() == D))
+        p = [0 if v is None else v.data_ptr() for part in parts for v in part] + [0] * (6 - 2 * len(parts))
+        hp, gp = ([v.data_ptr() for v in vs] + [0] * (2 - len(vs)) for vs in (hs, gains))
+        self.check(self.L.qsv_scaled_sum_rms_norms(x.data_ptr(), *hp, *p, *gp, 0 if tokens is None else tokens.data_ptr(),
+                                                   0 if table is None else table.data_ptr(), float(eps), T, D, self.code, self._s()),
+                   "scaled_sum_rms_norms")
+        return x, hs
 
     def normed_attention_prep(self, proj, q_off, k_off, v_off, heads, kv_heads, dim, vdim, q_w, k_w, eps, scale, v_first, mix, pool,
                               batch):
@@ -334,18 +359,21 @@ class HipOps:
         return a
 
     def qk_norm_rope_prep(self, q, k, v, heads, kv_heads, dim, vdim, q_w, k_w, per_head, eps, rope, rot_n, scale, pool, batch,
-                          q_b=None, k_b=None, v_b=None, halves=False, head_scale=None, q_pad=None):
+                          q_b=None, k_b=None, v_b=None, halves=False, head_scale=None, q_pad=None, rot_gain=0.0, q_store=False):
         """q [T, heads * dim], k [T, kv_heads * dim], v [T, kv_heads * vdim] (float or storage type, column slices are fine; k and v
         None: the layer caches nothing; v may be k itself: values that are the projected keys).  q_b, k_b, v_b (one per channel) are added
         first.  Queries and keys are RMS-normed per head (weight [dim], shared by the heads) or over the whole projection (weight as wide
         as it), then the first rot_n dimensions of every head turn with the position (pairs of neighbours, or with `halves` (i, i + rot_n
         / 2); rope float [positions, 2, rot_n / 2] or None).  -> float queries [T, heads, q_pad + dim] = [0 | q * scale *
-        head_scale[h]] (q_pad None: vdim); writes the cache rows [v | k] of the step's tokens into pool [kv_heads, rows, vdim + dim]."""
+        head_scale[h]] (q_pad None: vdim); writes the cache rows [v | k] of the step's tokens into pool [kv_heads, rows, vdim + dim].
+        q_w = k_w = None: norms (per head) without weights; rot_gain > 0: those norms follow the rotation, whose cos and sin carry the
+        magnitude sqrt(rot_gain); q_store: the queries come in the storage type."""
         T = q.size(0)
         q_pad = vdim if q_pad is None else int(q_pad)
-        qf = torch.empty((T, heads, q_pad + dim), dtype=torch.float32, device=q.device)
+        qf = torch.empty((T, heads, q_pad + dim), dtype=self.dtype if q_store else torch.float32, device=q.device)
         self._need(q_w, k_w, rope, pool, batch.slot, batch.pos, q_b, k_b, v_b, head_scale)
-        assert q.stride(1) == 1 and q.size(1) == heads * dim and q_w.dtype == self.dtype and q_w.numel() == (dim if per_head else heads * dim)
+        assert q.stride(1) == 1 and q.size(1) == heads * dim and (per_head or q_w is not None) and (q_w is None) == (k_w is None or k is None)
+        assert q_w is None or (q_w.dtype == self.dtype and q_w.numel() == (dim if per_head else heads * dim))
         assert rope is None or (rope.dtype == torch.float32 and rope.size(-1) * 2 == rot_n and rot_n <= dim and rope.size(0) > batch.max_pos)
         for b, n in ((q_b, heads * dim), (k_b, kv_heads * dim), (v_b, kv_heads * vdim)):
             assert b is None or (b.dtype == self.dtype and b.numel() == n)
@@ -353,15 +381,17 @@ class HipOps:
         kp = [0, 0, 0, 0, 0, 0, 0]
         if k is not None:
             assert k.dtype == v.dtype == q.dtype and k.stride(1) == v.stride(1) == 1 and k.size(1) == kv_heads * dim
-            assert v.size(1) == kv_heads * vdim and k_w.dtype == self.dtype and k_w.numel() == (dim if per_head else kv_heads * dim)
+            assert v.size(1) == kv_heads * vdim
+            assert k_w is None or (k_w.dtype == self.dtype and k_w.numel() == (dim if per_head else kv_heads * dim))
             assert pool.shape[0] == kv_heads and pool.shape[2] == vdim + dim and pool.dtype == self.dtype
-            kp = [k.data_ptr(), k.stride(0), v.data_ptr(), v.stride(0), k_w.data_ptr(), pool.data_ptr(), pool.size(1)]
+            kp = [k.data_ptr(), k.stride(0), v.data_ptr(), v.stride(0), 0 if k_w is None else k_w.data_ptr(), pool.data_ptr(), pool.size(1)]
         opt = [0 if b is None else b.data_ptr() for b in (q_b, k_b, v_b)]
         self.check(self.L.qsv_qk_norm_rope_prep(qf.data_ptr(), q.data_ptr(), q.stride(0), *kp[:4], dtype_code(q.dtype), heads, kv_heads,
-                                                dim, vdim, q_w.data_ptr(), kp[4], int(bool(per_head)), float(eps),
+                                                dim, vdim, 0 if q_w is None else q_w.data_ptr(), kp[4], int(bool(per_head)), float(eps),
                                                 0 if rope is None else rope.data_ptr(), int(rot_n if rope is not None else 0),
                                                 float(scale), kp[5], kp[6], batch.slot.data_ptr(), batch.pos.data_ptr(), T, *opt,
-                                                int(bool(halves)), 0 if head_scale is None else head_scale.data_ptr(), q_pad, self.code,
+                                                int(bool(halves)), 0 if head_scale is None else head_scale.data_ptr(), q_pad,
+                                                float(rot_gain), int(bool(q_store)), self.code,
                                                 self._s()), "qk_norm_rope_prep")
         return qf
 
@@ -501,6 +531,41 @@ class HipOps:
                                           self.code, self._s()), "talking_mix")
         return out
 
+    # ---- attention with two key maps over the same values ----------------------------------------------------------------------------
+    def conv_heads_cache(self, proj, conv_w, hist, batch, q_channels, kv_heads, key_width, vdim, pool, scale, temperature=None):
+        """proj [T, >= C] = [q (q_channels) | k (kv_heads * key_width) | v (kv_heads * vdim) | ..]: a causal convolution over time on each of
+        these C channels (conv_w float [taps, C]; hist: two-copy state, the last taps - 1 projected rows, None with one tap).  -> q [T,
+        q_channels] (storage type) times scale and, with temperature = (coef, every), times 1 + coef ln(floor((p + 1) / every) + 1); [v | k] go
+        into the cache rows of pool [kv_heads, rows, vdim + key_width] (kv_heads 0: queries only)."""
+        T, (taps, C) = proj.size(0), conv_w.shape
+        q = torch.empty((T, q_channels), dtype=self.dtype, device=proj.device)
+        self._need(conv_w, hist, pool, batch.slot, batch.pos, batch.run_off, batch.state_rd, batch.state_wr)
+        assert C == q_channels + kv_heads * (key_width + vdim) <= proj.size(1) and proj.stride(1) == 1 and proj.dtype == self.dtype
+        assert conv_w.dtype == torch.float32 and (taps == 1 or (hist.dtype == torch.float32 and hist.shape[1:] == (taps - 1, C)))
+        assert not kv_heads or (pool.dtype == self.dtype and pool.size(0) == kv_heads and pool.size(2) == vdim + key_width)
+        coef, every = temperature if temperature is not None else (0.0, 0.0)
+        self.check(self.L.qsv_conv_heads_cache(q.data_ptr(), pool.data_ptr() if kv_heads else 0, pool.size(1) if kv_heads else 0, proj.data_ptr(),
+                                               proj.stride(0), conv_w.data_ptr(), taps, 0 if hist is None else hist.data_ptr(),
+                                               batch.run_off.data_ptr(), batch.state_rd.data_ptr(), batch.state_wr.data_ptr(),
+                                               batch.slot.data_ptr(), batch.pos.data_ptr(), q_channels, kv_heads, key_width, vdim, float(scale),
+                                               float(coef), float(every), T, self.code, self._s()), "conv_heads_cache")
+        return q
+
+    def diff_attention(self, q, pool, batch, heads, dim, vdim, lam, out_scale, eps, gate, page, variant=0, key_splits=None):
+        """q [T, heads * 2 * dim] (storage type, scaled; per head map 1, map 2), pool [G, rows, vdim + 2 dim] of rows [v | k_1 | k_2]: with a_m the
+        softmax attention of map m over the keys up to the token, o = a_1 - lam a_2; -> o / sqrt(mean(o^2) + eps) * out_scale * sigmoid(gate) [T,
+        heads * vdim] (gate [T, heads * vdim], a column slice is fine, or None)."""
+        T, G = q.size(0), pool.size(0)
+        self._need(q, pool, batch.block_table, batch.seq, batch.pos)
+        assert q.shape == (T, heads * 2 * dim) and q.dtype == self.dtype == pool.dtype and pool.size(2) == vdim + 2 * dim and heads % G == 0
+        assert gate is None or (gate.dtype == self.dtype and gate.stride(1) == 1 and gate.shape == (T, heads * vdim))
+        out = torch.empty((T, heads * vdim), dtype=self.dtype, device=q.device)
+        bt, ep = batch.block_table, (float(lam), float(out_scale), float(eps), 0 if gate is None else gate.data_ptr(), 0 if gate is None else gate.stride(0))
+        self.check(self.L.qsv_diff_attention(out.data_ptr(), q.data_ptr(), pool.data_ptr(), bt.data_ptr(), bt.stride(0), batch.seq.data_ptr(),
+                                             batch.pos.data_ptr(), T, heads, G, dim, vdim, page, pool.stride(0), *ep, self.code, self._s()),
+                   "diff_attention")
+        return out
+
     # ---- recurrences ----------------------------------------------------------------------------------------------------------
     def decay(self, z, bias, a_log, tau, heads, dim):
         """z [T, heads * dim] (storage type; a column slice is fine) -> float decays: a_log given: exp(-exp(a_log[h]) softplus(z +
@@ -590,27 +655,29 @@ class HipOps:
 
     ACTS = {"none": 0, "relu_sq": 1, "swiglu": 2, "clamped_glu": 3}
 
-    def moe_experts(self, h, up, down, idx, wt, act="relu_sq", limit=0.0):
+    def moe_experts(self, h, up, down, idx, wt, act="relu_sq", limit=0.0, weigh="output"):
         """up [E, rows, D], down [E, D, ff]; y[t] = sum_k wt[t, k] * down[idx[t, k]] a(up[idx[t, k]] h[t]).  act "relu_sq":
         a = relu(.)^2, rows = ff; "swiglu": up's rows come in pairs (2f = gate, 2f + 1 = up), a_f = silu(gate_f) up_f, rows = 2 ff;
         "clamped_glu": the same pairs with g = min(gate_f, limit), u = clamp(up_f, -limit, limit), a_f = g sigmoid(1.702 g) (u + 1).
-        Indices at or above E (up.size(0)) name identity experts: their output is h[t] itself."""
+        Indices at or above E (up.size(0)) name identity experts: their output is h[t] itself.  weigh "input": the weight multiplies the
+        expert's input, y[t] = sum_k down[..] a(up[..] (wt[t, k] h[t])) (the products' results are scaled, in float)."""
         T, D = h.shape
         top_k, rows = idx.size(1), up.size(1)
         a = self.ACTS[act]
         ff = rows // 2 if a >= 2 else rows
         if (self.code == BF16 and self.moe_token_slots < T * top_k <= self.moe_expert_major_slots and D % 8 == 0 and ff % 8 == 0
                 and D <= 4096 and ff <= 4096):
-            return self._moe_experts_expert_major(h, up, down, idx, wt, a, limit)
+            return self._moe_experts_expert_major(h, up, down, idx, wt, a, limit, weigh)
         if T * top_k > self.moe_sorted_above:
-            return self._moe_experts_sorted(h, up, down, idx, wt, a, limit)
+            return self._moe_experts_sorted(h, up, down, idx, wt, a, limit, weigh)
         act = torch.empty((T, top_k, ff), dtype=self.dtype, device=h.device)
         y = torch.empty((T, D), dtype=self.dtype, device=h.device)
         self._need(h, up, down, idx, wt)
+        w_in, w_out = self._weights_at(wt, weigh)
         assert up.shape[2] == D and down.shape == (up.size(0), D, ff)
         self.check(self.L.qsv_moe_up(act.data_ptr(), h.data_ptr(), up.data_ptr(), idx.data_ptr(), T, top_k, D, rows, a, float(limit),
-                                     up.size(0), self.code, self._s()), "moe_up")
-        self.check(self.L.qsv_moe_down(y.data_ptr(), act.data_ptr(), down.data_ptr(), idx.data_ptr(), wt.data_ptr(), T, top_k, D,
+                                     up.size(0), w_in, self.code, self._s()), "moe_up")
+        self.check(self.L.qsv_moe_down(y.data_ptr(), act.data_ptr(), down.data_ptr(), idx.data_ptr(), w_out, T, top_k, D,
                                        ff, h.data_ptr(), up.size(0), self.code, self._s()), "moe_down")
         return y
 
@@ -626,16 +693,23 @@ class HipOps:
     moe_token_slots = 8
     moe_expert_major_slots = 1024
 
-    def _combine(self, h, ys, inv, idx, wt, E):
+    @staticmethod
+    def _weights_at(wt, weigh):
+        """-> addresses of the weights for the up products (on the input) and for the sum over the experts."""
+        assert weigh in ("input", "output") and wt.dtype == torch.float32 and wt.is_contiguous()
+        return (wt.data_ptr(), 0) if weigh == "input" else (0, wt.data_ptr())
+
+    def _combine(self, h, ys, inv, idx, w_out, E):
         """y[t] = sum_k wt[t, k] * (ys[inv[t K + k]], or h[t] where idx[t, k] names an identity expert)."""
         T, D = h.shape
         y = torch.empty((T, D), dtype=self.dtype, device=h.device)
-        self.check(self.L.qsv_moe_combine(y.data_ptr(), ys.data_ptr(), inv.data_ptr(), wt.data_ptr(), T, idx.size(1), D, idx.data_ptr(),
+        self.check(self.L.qsv_moe_combine(y.data_ptr(), ys.data_ptr(), inv.data_ptr(), w_out, T, idx.size(1), D, idx.data_ptr(),
                                           h.data_ptr(), E, self.code, self._s()), "moe_combine")
         return y
 
-    def _moe_experts_expert_major(self, h, up, down, idx, wt, a=1, limit=0.0):
+    def _moe_experts_expert_major(self, h, up, down, idx, wt, a=1, limit=0.0, weigh="output"):
         T, D = h.shape
+        w_in, w_out = self._weights_at(wt, weigh)
         E, rows, K = up.size(0), up.size(1), idx.size(1)
         ff = rows // 2 if a >= 2 else rows
         n = T * K
@@ -648,15 +722,16 @@ class HipOps:
         act = torch.empty((n, ff), dtype=self.dtype, device=h.device)
         ys = torch.empty((n, D), dtype=self.dtype, device=h.device)
         self.check(self.L.qsv_expert_rows(act.data_ptr(), h.data_ptr(), order.data_ptr(), K, up.data_ptr(), offsets.data_ptr(),
-                                          E, rows, D, a, float(limit), self._s()), "expert_rows(up)")
+                                          E, rows, D, a, float(limit), w_in, self._s()), "expert_rows(up)")
         self.check(self.L.qsv_expert_rows(ys.data_ptr(), act.data_ptr(), 0, 1, down.data_ptr(), offsets.data_ptr(), E, D, ff, 0, 0.0,
-                                          self._s()), "expert_rows(down)")
-        return self._combine(h, ys, inv, idx, wt, E)
+                                          0, self._s()), "expert_rows(down)")
+        return self._combine(h, ys, inv, idx, w_out, E)
 
-    def _moe_experts_sorted(self, h, up, down, idx, wt, code=1, limit=0.0):
+    def _moe_experts_sorted(self, h, up, down, idx, wt, code=1, limit=0.0, weigh="output"):
         """code >= 2 (gated units): the grouped kernel folds the two halves of a unit in its epilogue; with vendor products the
         first product leaves both halves ([n, 2 ff]) and `glu` folds them."""
         T, D = h.shape
+        w_in, w_out = self._weights_at(wt, weigh)
         E, rows, K = up.size(0), up.size(1), idx.size(1)
         ff = rows // 2 if code >= 2 else rows
         n = T * K
@@ -677,10 +752,10 @@ class HipOps:
             for lo in range(0, len(tiles), 65535):
                 tl = torch.tensor(tiles[lo:lo + 65535], dtype=torch.int32).to(h.device)
                 self.check(self.L.qsv_grouped_gemm(act.data_ptr(), h.data_ptr(), order.data_ptr(), K, up.data_ptr(), tl.data_ptr(),
-                                                   tl.size(0), rows, D, code, float(limit), self._s()), "grouped_gemm(up)")
+                                                   tl.size(0), rows, D, code, float(limit), w_in, self._s()), "grouped_gemm(up)")
                 self.check(self.L.qsv_grouped_gemm(ys.data_ptr(), act.data_ptr(), 0, 1, down.data_ptr(), tl.data_ptr(),
-                                                   tl.size(0), D, ff, 0, 0.0, self._s()), "grouped_gemm(down)")
-            return self._combine(h, ys, inv, idx, wt, E)
+                                                   tl.size(0), D, ff, 0, 0.0, 0, self._s()), "grouped_gemm(down)")
+            return self._combine(h, ys, inv, idx, w_out, E)
         xs = torch.empty((n, D), dtype=self.dtype, device=h.device)
         self.check(self.L.qsv_gather_rows(xs.data_ptr(), h.data_ptr(), order.data_ptr(), K, n, D, self.code, self._s()),
                    "gather_rows")
@@ -692,15 +767,17 @@ class HipOps:
                 torch.matmul(xs[at:at + c], up[e].t(), out=act[at:at + c])
             at += c
         if code >= 2:
-            act = self.glu(act, "silu" if code == 2 else "clamped", limit)
+            act = self.glu(act, "silu" if code == 2 else "clamped", limit, *((wt.view(-1), order) if weigh == "input" else ()))
         else:
+            if weigh == "input":
+                raise ValueError("weights on the input: gated units only in the expert-sorted form with vendor products")
             self.check(self.L.qsv_relu_sq(act.data_ptr(), act.numel(), self.code, self._s()), "relu_sq")
         at = 0
         for e, c in enumerate(counts):
             if c:
                 torch.matmul(act[at:at + c], down[e].t(), out=ys[at:at + c])
             at += c
-        return self._combine(h, ys, inv, idx, wt, E)
+        return self._combine(h, ys, inv, idx, w_out, E)
 
 
 def _rotate(v, rope, pos, rot_n):
@@ -865,17 +942,22 @@ class TorchOps:
         return a
 
     def qk_norm_rope_prep(self, q, k, v, heads, kv_heads, dim, vdim, q_w, k_w, per_head, eps, rope, rot_n, scale, pool, batch,
-                          q_b=None, k_b=None, v_b=None, halves=False, head_scale=None, q_pad=None):
+                          q_b=None, k_b=None, v_b=None, halves=False, head_scale=None, q_pad=None, rot_gain=0.0, q_store=False):
         T = q.size(0)
 
         def biased(u, b):
             return u.float() if b is None else u.float() + b.float()
 
         def prep(u, w, n):
-            u = self._rms(u.reshape(T, n, dim), w, eps) if per_head else self._rms(u, w, eps).view(T, n, dim)
-            if rope is None:
-                return u
-            return self._rotate_halves(u, rope, batch.pos, rot_n) if halves else _rotate(u, rope, batch.pos, rot_n)
+            def turn(u):
+                if rope is None:
+                    return u
+                return self._rotate_halves(u, rope, batch.pos, rot_n) if halves else _rotate(u, rope, batch.pos, rot_n)
+
+            one = torch.ones(dim, device=u.device) if w is None else w
+            if rot_gain > 0:
+                return self._rms(turn(u.reshape(T, n, dim)), one, eps)
+            return turn(self._rms(u.reshape(T, n, dim), one, eps) if per_head else self._rms(u, w, eps).view(T, n, dim))
 
         if k is not None:
             rows = torch.cat([biased(v, v_b).reshape(T, kv_heads, vdim), prep(biased(k, k_b), k_w, kv_heads)], dim=-1)
@@ -883,7 +965,8 @@ class TorchOps:
         out = prep(biased(q, q_b), q_w, heads) * scale
         if head_scale is not None:
             out = out * head_scale[:, None]
-        return torch.cat([torch.zeros(T, heads, vdim if q_pad is None else q_pad, device=q.device), out], dim=-1).contiguous()
+        out = torch.cat([torch.zeros(T, heads, vdim if q_pad is None else q_pad, device=q.device), out], dim=-1).contiguous()
+        return out.to(self.dtype) if q_store else out
 
     def pool_blocks(self, pool, pooled, batch, block, page):
         per_page = (page + block - 1) // block
@@ -1028,8 +1111,10 @@ class TorchOps:
     def rms_pair_mean(self, a, wa, b, wb, eps):
         return (0.5 * (self._rms(a, wa, eps) + self._rms(b, wb, eps))).to(self.dtype)
 
-    def glu(self, a, act="silu", limit=0.0):
+    def glu(self, a, act="silu", limit=0.0, row_scale=None, scale_index=None):
         a = a.float()
+        if row_scale is not None:
+            a = a * (row_scale if scale_index is None else row_scale[scale_index])[:, None]
         g, u = a[..., 0::2], a[..., 1::2]
         if act == "clamped":
             g, u = g.clamp(max=limit), u.clamp(-limit, limit)
@@ -1076,6 +1161,51 @@ class TorchOps:
     def rms_norm_rows(self, x, rows, w, eps):
         return self._rms(x if rows is None else x[rows.long()], w, eps).to(self.dtype)
 
+    def scaled_sum_rms_norms(self, x, parts, gains, eps, tokens=None, table=None):
+        if tokens is not None:
+            start = table[tokens.long()].float()
+            x = start if x is None else x.copy_(start)
+        if parts:
+            x += sum((1.0 if s is None else s.float()) * y.float() for y, s in parts)
+        return x, [self._rms(x, g, eps).to(self.dtype) for g in gains]
+
+    # ---- attention with two key maps over the same values ----------------------------------------------------------------------------
+    def conv_heads_cache(self, proj, conv_w, hist, batch, q_channels, kv_heads, key_width, vdim, pool, scale, temperature=None):
+        taps, C = conv_w.shape
+        u, y = proj[:, :C].float(), torch.empty((proj.size(0), C), device=proj.device)
+        for slot, first, cnt in batch.items:
+            rd, wr = int(batch.state_rd[first]), int(batch.state_wr[first + cnt - 1])
+            past = hist[rd] if rd >= 0 and taps > 1 else torch.zeros((taps - 1, C), device=proj.device)
+            seq = torch.cat([past, u[first:first + cnt]])
+            y[first:first + cnt] = sum(seq[j:j + cnt] * conv_w[j] for j in range(taps))
+            if taps > 1:
+                hist[wr] = seq[cnt:]
+        if kv_heads:
+            T, n = proj.size(0), q_channels + kv_heads * key_width
+            rows = torch.cat([y[:, n:].reshape(T, kv_heads, vdim), y[:, q_channels:n].reshape(T, kv_heads, key_width)], dim=-1)
+            pool[:, batch.slot] = rows.transpose(0, 1).to(self.dtype)
+        q = y[:, :q_channels] * scale
+        if temperature is not None:
+            coef, every = temperature
+            q = q * (1.0 + coef * torch.log(torch.floor((batch.pos.double() + 1.0) / every).float() + 1.0))[:, None]
+        return q.to(self.dtype)
+
+    def diff_attention(self, q, pool, batch, heads, dim, vdim, lam, out_scale, eps, gate, page, variant=0, key_splits=None):
+        T, G = q.size(0), pool.size(0)
+        q, per, bt = q.view(T, heads, 2, dim).float(), heads // G, batch.block_table.long()
+        o = torch.empty((T, heads, vdim), device=q.device)
+        for t in range(T):
+            j = torch.arange(int(batch.pos[t]) + 1, device=q.device)
+            rows = pool[:, bt[int(batch.seq[t]), j // page] * page + j % page].float()                 # [G, n, R]
+            for g in range(G):
+                hs, v = slice(g * per, (g + 1) * per), rows[g, :, :vdim]
+                a1, a2 = (torch.softmax(q[t, hs, m] @ rows[g, :, vdim + m * dim:vdim + (m + 1) * dim].t(), dim=-1) @ v for m in (0, 1))
+                o[t, hs] = a1 - lam * a2
+        o = (o / torch.sqrt((o * o).mean(-1, keepdim=True) + eps) * out_scale).reshape(T, heads * vdim)
+        if gate is not None:
+            o = o * torch.sigmoid(gate.float())
+        return o.to(self.dtype)
+
     def normed_attention_prep(self, proj, q_off, k_off, v_off, heads, kv_heads, dim, vdim, q_w, k_w, eps, scale, v_first, mix, pool,
                               batch):
         T = proj.size(0)
@@ -1100,7 +1230,7 @@ class TorchOps:
             m_state[slot] = prev
         return a, b, m
 
-    def moe_experts(self, h, up, down, idx, wt, act="relu_sq", limit=0.0):
+    def moe_experts(self, h, up, down, idx, wt, act="relu_sq", limit=0.0, weigh="output"):
         T, D = h.shape
         E = up.size(0)
         y = torch.zeros((T, D), dtype=torch.float32, device=h.device)
@@ -1109,13 +1239,15 @@ class TorchOps:
             real = e < E
             e = e.clamp(max=E - 1)
             a = torch.einsum("tfd,td->tf", up[e].float(), h.float())
+            if weigh == "input":
+                a = a * wt[:, k, None]
             if act == "relu_sq":
                 a = torch.relu(a) ** 2
             else:
                 a = self.glu(a.to(self.dtype), "silu" if act == "swiglu" else "clamped", limit).float()
             a = a.to(self.dtype).float()
             o = torch.einsum("tdf,tf->td", down[e].float(), a)
-            y += wt[:, k, None] * torch.where(real[:, None], o, h.float())
+            y += (wt[:, k, None] if weigh == "output" else 1.0) * torch.where(real[:, None], o, h.float())
         return y.to(self.dtype)
 
 

@@ -12,7 +12,8 @@ the softmax-weighted sum of the rows' first vdim elements is the output; one lau
 `NormedChunkAttention` is the position-free sibling on the same cache rows and kernel: queries and keys are RMS-normed over the
 whole projection, positions enter through a learned bias per (distance bucket, head) and through chunks that bound what a query
 sees, and the values may be blended with those an earlier layer computed for the same token.  `SinkWindowAttention` is the windowed
-sibling with a sink, `TalkingHeadsAttention` the one whose weights are mixed across heads.
+sibling with a sink, `TalkingHeadsAttention` the one whose weights are mixed across heads, `DifferentialAttention` the difference of two
+softmax maps over the same values, `TiedRotaryAttention` the one with tied values and norms behind the rotation.
 """
 import math
 
@@ -264,3 +265,81 @@ class TalkingHeadsAttention:
                                    self.rotary.dims if rope is not None else 0, self.scale, pool, batch, q_b=self.q_b, k_b=self.k_b,
                                    v_b=self.k_b, halves=True, head_scale=self.temp, q_pad=0)
         return linear(ops.talking_attention(qf, pool, batch, self.talk, proj[:, o_g:o_g + H], d, self.page, cap=self.cap), self.w_o)
+
+
+class DifferentialAttention:
+    """The difference of two causal softmax attentions over the same values (differential attention), grouped-query.
+
+    q (H heads of two maps of `dim`), k (G heads of two maps), v (G heads of `vdim`) each go through a short causal convolution over time
+    straight after the projection (weights [channels, taps], no bias, no activation; the last taps - 1 projected rows of a sequence are its
+    state).  No rotation; temperature (coef, every): the query at position p is multiplied by 1 + coef ln(floor((p + 1) / every) + 1).  Per
+    head, with a_m the softmax attention of map m and lambda = exp(lq1 . lk1) - exp(lq2 . lk2) + diff: o = a_1 - lambda a_2, divided by its
+    root mean square over vdim, times 1 - diff, times sigmoid(W_g h) element by element.
+    shared_kv: the layer has queries only and reads the pools of another layer of the same key / value sizes.
+    Cache: per key / value head one pool of rows [v | k_1 | k_2], all after their convolutions."""
+
+    def __init__(self, ops, *, heads, kv_heads, dim, vdim, scale, taps, diff, eps, weights, temperature=None, shared_kv=False, page=64):
+        """weights: q [2 H dim, D], q_conv [2 H dim, taps], g [H vdim, D], o [D, H vdim], lq1, lk1, lq2, lk2 [dim]; unless shared_kv: k [2 G dim, D],
+        v [G vdim, D], k_conv, v_conv."""
+        if heads % kv_heads or taps < 1 or (temperature is not None and not float(temperature[1]) > 0.0):
+            raise ValueError(f"differential attention: {heads} heads over {kv_heads}, {taps} taps, temperature {temperature}")
+        self.ops, self.H, self.G, self.dim, self.vdim, self.page = ops, heads, kv_heads, dim, vdim, page
+        self.scale, self.taps, self.eps, self.shared_kv = float(scale), int(taps), float(eps), bool(shared_kv)
+        self.temperature = None if temperature is None else (float(temperature[0]), float(temperature[1]))
+        w = weights
+        D = w["q"].size(1)
+        expect = {"q": (2 * heads * dim, D), "q_conv": (2 * heads * dim, taps), "g": (heads * vdim, D), "o": (D, heads * vdim)}
+        expect.update({n: (dim,) for n in ("lq1", "lk1", "lq2", "lk2")})
+        if not shared_kv:
+            expect.update(k=(2 * kv_heads * dim, D), v=(kv_heads * vdim, D), k_conv=(2 * kv_heads * dim, taps), v_conv=(kv_heads * vdim, taps))
+        for k, shp in expect.items():
+            if tuple(w[k].shape) != shp:
+                raise ValueError(f"differential attention weight {k}: shape {tuple(w[k].shape)}, expected {shp}")
+        from ..serving.cache import StateSpec
+        from .recurrent import pad_rows
+        own = [] if shared_kv else ["k", "v"]
+        self.w_in, self.w_o = pad_rows(torch.cat([w[n] for n in ["q"] + own + ["g"]], dim=0)), w["o"].contiguous()
+        self.conv = torch.cat([w[n + "_conv"] for n in ["q"] + own], dim=0).float().t().contiguous()          # [taps, C]
+        self.C = self.conv.size(1)
+        l1, l2 = (float((w["lq" + i].double() * w["lk" + i].double()).sum()) for i in "12")
+        self.lam, self.out_scale = math.exp(l1) - math.exp(l2) + float(diff), 1.0 - float(diff)
+        self.cache_rows = [] if shared_kv else [(kv_heads, vdim + 2 * dim)]
+        self.state_specs = [StateSpec((taps - 1, self.C), copies=2)] if taps > 1 else []
+
+    def __call__(self, h, batch, pools, states):
+        ops, H, d, dv, pool = self.ops, self.H, self.dim, self.vdim, pools[0]
+        proj = linear(h, self.w_in)
+        q = ops.conv_heads_cache(proj, self.conv, states[0] if self.taps > 1 else None, batch, 2 * H * d, 0 if self.shared_kv else self.G, 2 * d, dv,
+                                 pool, self.scale, self.temperature)
+        o = ops.diff_attention(q, pool, batch, H, d, dv, self.lam, self.out_scale, self.eps, proj[:, self.C:self.C + H * dv], self.page)
+        return linear(o, self.w_o)
+
+
+class TiedRotaryAttention:
+    """Causal grouped-query softmax attention whose values are the projected keys.  The first rotary.dims dimensions of every q and k head turn
+    with the position (halves layout; rotary None: no rotation), THEN q and k are divided by their root mean square over `dim` per head (no
+    weight); score = q . k * scale.  Cache: per key / value head one pool of rows [v | k]."""
+
+    def __init__(self, ops, *, heads, kv_heads, dim, scale, rotary, eps, weights, page=64):
+        """weights: q [H dim, D], k [G dim, D], o [D, H dim]."""
+        if heads % kv_heads or (rotary is not None and rotary.dims > dim):
+            raise ValueError(f"attention: {heads} heads over {kv_heads}, {rotary.dims if rotary else 0} rotated dimensions of {dim}")
+        self.ops, self.H, self.G, self.dim, self.page = ops, heads, kv_heads, dim, page
+        self.scale, self.eps, self.rotary = float(scale), float(eps), rotary
+        w = weights
+        D = w["q"].size(1)
+        for k, shp in {"q": (heads * dim, D), "k": (kv_heads * dim, D), "o": (D, heads * dim)}.items():
+            if tuple(w[k].shape) != shp:
+                raise ValueError(f"attention weight {k}: shape {tuple(w[k].shape)}, expected {shp}")
+        self.w_in, self.w_o = torch.cat([w["q"], w["k"]], dim=0).contiguous(), w["o"].contiguous()
+        self.cache_rows, self.state_specs = [(kv_heads, 2 * dim)], []
+
+    def __call__(self, h, batch, pools, states):
+        ops, T, H, G, d, pool, rot = self.ops, h.size(0), self.H, self.G, self.dim, pools[0], self.rotary
+        proj = linear(h, self.w_in)
+        k = proj[:, H * d:]
+        rope = rot.reserve(batch.max_pos + 1) if rot is not None else None
+        qf = ops.qk_norm_rope_prep(proj[:, :H * d], k, k, H, G, d, d, None, None, True, self.eps, rope, rot.dims if rot is not None else 0,
+                                   self.scale, pool, batch, halves=True, rot_gain=rot.magnitude ** 2 if rot is not None else 0.0)
+        o = ops.latent_attention(qf, pool, batch, None, d, self.page, q_first=d)
+        return linear(o.view(T, H * d), self.w_o)

@@ -7,7 +7,7 @@ import ctypes as C
 import os
 import threading
 
-_vp, _i, _i64, _f = C.c_void_p, C.c_int, C.c_int64, C.c_float
+_vp, _i, _i64, _f, _d = C.c_void_p, C.c_int, C.c_int64, C.c_float, C.c_double
 SIGNATURES = {
     "qsv_version": (_i, []),
     "qsv_arch": (C.c_char_p, []),
@@ -40,11 +40,11 @@ SIGNATURES = {
     "qsv_rotate_qk": (_i, [_vp, _vp, _i64, _i, _i, _i, _vp, _i, _vp, _i, _i, _vp]),
     "qsv_sigmoid_gate": (_i, [_vp, _vp, _i64, _i, _i, _i, _vp]),
     "qsv_moe_route": (_i, [_vp, _vp, _vp, _vp, _vp, _i, _i, _i, _i, _i, _i, _i, _i, _vp, _i, _f, _i, _vp]),
-    "qsv_moe_up": (_i, [_vp, _vp, _vp, _vp, _i, _i, _i, _i, _i, _f, _i, _i, _vp]),
-    "qsv_expert_rows": (_i, [_vp, _vp, _vp, _i, _vp, _vp, _i, _i, _i, _i, _f, _vp]),
+    "qsv_moe_up": (_i, [_vp, _vp, _vp, _vp, _i, _i, _i, _i, _i, _f, _i, _vp, _i, _vp]),
+    "qsv_expert_rows": (_i, [_vp, _vp, _vp, _i, _vp, _vp, _i, _i, _i, _i, _f, _vp, _vp]),
     "qsv_grouped_gemm_tile_slots": (_i, []),
     "qsv_grouped_gemm_k_step": (_i, []),
-    "qsv_grouped_gemm": (_i, [_vp, _vp, _vp, _i, _vp, _vp, _i, _i, _i, _i, _f, _vp]),
+    "qsv_grouped_gemm": (_i, [_vp, _vp, _vp, _i, _vp, _vp, _i, _i, _i, _i, _f, _vp, _vp]),
     "qsv_gather_rows": (_i, [_vp, _vp, _vp, _i, _i, _i, _i, _vp]),
     "qsv_relu_sq": (_i, [_vp, _i64, _i, _vp]),
     "qsv_moe_combine": (_i, [_vp, _vp, _vp, _vp, _i, _i, _i, _vp, _vp, _i, _i, _vp]),
@@ -54,20 +54,23 @@ SIGNATURES = {
     "qsv_hc_write": (_i, [_vp, _vp, _vp, _vp, _i, _i, _i, _vp, _vp, _vp, _vp, _f, _i, _vp]),
     "qsv_dyt_sum_rows": (_i, [_vp, _vp, _vp, _vp, _vp, _f, _i, _i, _i, _i, _vp]),
     "qsv_rms_pair_mean": (_i, [_vp, _vp, _vp, _vp, _vp, _f, _i, _i, _i, _vp]),
-    "qsv_glu": (_i, [_vp, _vp, _i, _i, _i, _f, _i, _vp]),
+    "qsv_glu": (_i, [_vp, _vp, _i, _i, _i, _f, _vp, _vp, _i, _vp]),
     "qsv_decay": (_i, [_vp, _vp, _i64, _vp, _vp, _f, _i, _i, _i, _i, _vp]),
     "qsv_conv_silu_unit": (_i, [_vp, _vp, _i64, _i, _i, _i, _vp, _vp, _vp, _vp, _vp, _i, _i, _i, _i, _i, _vp]),
     "qsv_min_gru_scan": (_i, [_vp, _vp, _i64, _i, _i, _i, _vp, _vp, _vp, _vp, _i, _i, _i, _i, _vp]),
     "qsv_add_normed_rms_norm": (_i, [_vp, _vp, _vp, _vp, _i, _vp, _i, _f, _i, _i, _i, _vp]),
     "qsv_qk_norm_rope_prep": (_i, [_vp, _vp, _i64, _vp, _i64, _vp, _i64, _i, _i, _i, _i, _i, _vp, _vp, _i, _f, _vp, _i, _f, _vp, _i64,
-                                   _vp, _vp, _i, _vp, _vp, _vp, _i, _vp, _i, _i, _vp]),
+                                   _vp, _vp, _i, _vp, _vp, _vp, _i, _vp, _i, _f, _i, _i, _vp]),
+    "qsv_conv_heads_cache": (_i, [_vp, _vp, _i64, _vp, _i64, _vp, _i, _vp, _vp, _vp, _vp, _vp, _vp, _i, _i, _i, _i, _f, _f, _d, _i, _i, _vp]),
+    "qsv_diff_attention": (_i, [_vp, _vp, _vp, _vp, _i, _vp, _vp, _i, _i, _i, _i, _i, _i, _i64, _f, _f, _f, _vp, _i64, _i, _vp]),
     "qsv_recurrent_scan": (_i, [_vp, _vp, _i64, _vp, _i64, _vp, _i64, _i, _vp, _vp, _i64, _i, _vp, _vp, _i, _i, _i, _i, _i, _i, _f, _vp,
                                 _i, _i, _vp]),
     "qsv_head_rms_gate": (_i, [_vp, _vp, _vp, _vp, _i64, _i, _f, _i, _i, _i, _i, _i, _vp, _i, _vp]),
     "qsv_max_gates": (_i, [_vp, _vp, _vp, _vp, _vp, _i64, _vp, _vp, _f, _vp, _vp, _i, _i, _i, _vp]),
     "qsv_embed_sinusoid": (_i, [_vp, _vp, _vp, _vp, _vp, _f, _i, _i, _i, _vp]),
     "qsv_add_rms_norm": (_i, [_vp, _vp, _vp, _vp, _vp, _vp, _f, _i, _i, _i, _vp]),
-    "qsv_rms_norm_rows": (_i, [_vp, _vp, _vp, _vp, _f, _i, _i, _i, _vp]),
+    "qsv_rms_norm_rows": (_i, [_vp, _vp, _vp, _vp, _i, _f, _i, _i, _i, _vp]),
+    "qsv_scaled_sum_rms_norms": (_i, [_vp, _vp, _vp, _vp, _vp, _vp, _vp, _vp, _vp, _vp, _vp, _vp, _vp, _f, _i, _i, _i, _vp]),
     "qsv_normed_attention_prep": (_i, [_vp, _vp, _i64, _vp, _i64, _i, _i, _i, _i, _i, _i, _i, _vp, _vp, _f, _f, _vp, _i64, _f, _vp, _i,
                                        _i, _vp]),
     "qsv_attention_prep": (_i, [_vp, _vp, _i64, _vp, _i64, _i, _i, _i, _i, _i, _i, _i, _i, _vp, _vp, _f, _vp, _vp, _i, _i, _vp]),

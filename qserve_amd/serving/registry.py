@@ -16,7 +16,7 @@ import os
 
 _MODELS = {}
 _BUILTIN = ("qserve_amd.models.vekalorn", "qserve_amd.models.mumelix", "qserve_amd.models.vepolix", "qserve_amd.models.pemolorn",
-            "qserve_amd.models.sagupel", "qserve_amd.models.llama_w4a8")
+            "qserve_amd.models.sagupel", "qserve_amd.models.rivolix", "qserve_amd.models.llama_w4a8")
 
 
 def register_model(architecture, engine="paged"):

@@ -110,14 +110,14 @@ def test_serve_argument_validation_without_gpu():
     assert L.qsv_recurrent_scan(1, 1, 8, 1, 8, 1, 8, 1, 1, None, 0, 0, 1, 1, 1, 5, 2, 2, 8, 8, 1.0, None, 1, 12, None) == 1  # more value columns than the state has
     assert L.qsv_head_rms_gate(1, 1, 1, 1, 16, 1, 1e-5, 2, 2, 8, 8, 1, 1, 0, None) == 1                       # a normaliser without its column
     assert L.qsv_max_gates(1, 1, 1, 1, 1, 4, 1, 1, 0.0, 1, 1, 1, 4, 0, None) == 1                             # gate cap 0
-    assert L.qsv_glu(1, 1, 2, 8, 7, 0.0, 0, None) == 1                                                        # unknown activation
-    assert L.qsv_glu(1, 1, 2, 8, 2, 0.0, 0, None) == 1                                                        # clamped units without a limit
+    assert L.qsv_glu(1, 1, 2, 8, 7, 0.0, None, None, 0, None) == 1                                                        # unknown activation
+    assert L.qsv_glu(1, 1, 2, 8, 2, 0.0, None, None, 0, None) == 1                                                        # clamped units without a limit
     assert L.qsv_add_rms_norm(1, 1, None, None, None, None, 1e-5, 2, 8, 0, None) == 1                         # a norm without its weight
     assert L.qsv_hc_write(1, 1, 1, 1, 2, 17, 8, None, None, None, None, 0.0, 0, None) == 1                    # 17 streams
-    assert L.qsv_moe_up(1, 1, 1, 1, 1, 1, 8, 7, 2, 0.0, 4, 0, None) == 1                                      # gated units, odd rows
-    assert L.qsv_moe_up(1, 1, 1, 1, 1, 1, 8, 8, 3, 0.0, 4, 0, None) == 1                                      # clamped units without a limit
+    assert L.qsv_moe_up(1, 1, 1, 1, 1, 1, 8, 7, 2, 0.0, 4, None, 0, None) == 1                                      # gated units, odd rows
+    assert L.qsv_moe_up(1, 1, 1, 1, 1, 1, 8, 8, 3, 0.0, 4, None, 0, None) == 1                                      # clamped units without a limit
     assert L.qsv_add_normed_rms_norm(1, 1, 1, None, 0, 1, 0, 1e-5, 2, 8, 0, None) == 1                        # an added sublayer output without its gain
-    assert L.qsv_qk_norm_rope_prep(1, 1, 64, None, 0, None, 0, 0, 2, 1, 32, 32, 1, None, 1, 1e-5, 1, 40, 1.0, None, 0, None, 1, 2, None, None, None, 0, None, 32, 0, None) == 1   # 40 rotated dimensions of 32
+    assert L.qsv_qk_norm_rope_prep(1, 1, 64, None, 0, None, 0, 0, 2, 1, 32, 32, 1, None, 1, 1e-5, 1, 40, 1.0, None, 0, None, 1, 2, None, None, None, 0, None, 32, 0.0, 0, 0, None) == 1   # 40 rotated dimensions of 32
     assert L.qsv_min_gru_scan(1, 1, 16, 0, 8, 16, 1, 1, 1, 1, 1, 1, 8, 0, None) == 1                            # the gate's columns lie outside the rows
     assert L.qsv_latent_attention(1, 1, 1, 1, 4, 1, 1, 32, 4, 2, 64, 96, 64, 2, 0, 0, None, 0, 0, None, 1, 0, 16, 4, 1, 0, 1, None) == 1     # distance slopes with pooled blocks
     assert [L.qsv_talking_attention_key_pools(*a) for a in ((8, 4, 64, 0), (8, 4, 64, 1), (32, 8, 128, 1), (32, 1, 64, 1))] == [1, 4, 4, 1]
