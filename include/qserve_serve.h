@@ -281,6 +281,18 @@ int qsv_conv_heads_cache(void* q, void* pool, int64_t pool_rows, const void* pro
                          const int32_t* run_off, const int32_t* state_rd, const int32_t* state_wr, const int64_t* slot, const int32_t* pos,
                          int q_channels, int kv_heads, int key_width, int vdim, float scale, float temp_coef, double temp_every, int n_tokens,
                          int dtype, void* stream);
+/* The matrix-core form (bfloat16; one or two maps; sizes by qsv_maps_attention_ok): q [T, H, maps, dim], rows [v | k_1 ..]; with two maps as
+ * qsv_diff_attention, with one map out = softmax(q . k) v, times sigmoid(gate) where there is a gate.  Tiles int32 [n, 3] = (sequence slot,
+ * first flat token index, tokens): step tiles hold at most N = qsv_maps_attention_tile_tokens(H / G) tokens, prompt tiles at most 4 N.
+ * key_splits > 1: a step tile's keys are cut over that many workgroups; workspace part_o float [key_splits, n_step, G * groups, 32, maps,
+ * vdim] and part_ml float [.., 32, maps, 2] with groups = qsv_maps_attention_head_groups(H / G). */
+int qsv_maps_attention_ok(int dim, int vdim, int maps, int page, int dtype);
+int qsv_maps_attention_tile_tokens(int heads_per_pool);
+int qsv_maps_attention_head_groups(int heads_per_pool);
+int qsv_maps_attention(void* out, const void* q, const void* pool, const int32_t* block_table, int table_stride, const int32_t* pos,
+                       const int32_t* prompt_tiles, int n_prompt, const int32_t* step_tiles, int n_step, int H, int G, int dim, int vdim,
+                       int maps, int page, int64_t pool_stride, float lambda, float out_scale, float eps, const void* gate,
+                       int64_t gate_stride, int key_splits, float* part_o, float* part_ml, void* stream);
 /* q [T, H, 2, dim] (scaled), cache rows [v (vdim) | k_1 (dim) | k_2 (dim)] in G pools (head h reads pool h / (H / G)), keys 0 .. pos[t]:
  * a_m = softmax(q_m . k_m) v, o = a_1 - lambda a_2, out[t, h] = o / sqrt(mean(o^2) + eps) * out_scale * sigmoid(gate[t, h]) (gate NULL: no
  * gate); [T, H, vdim].  Any sizes up to dim 512 and vdim 1024. */

@@ -328,7 +328,7 @@ struct MapsArgs {
     const int32_t *block_table, *pos, *tiles;
     float *part_o, *part_ml;
     int64_t pool_stride, gate_stride;
-    int table_stride, n_tiles, H, per, page, HP, TQ, HG, Z;
+    int table_stride, n_tiles, H, per, page_shift, HP, TQ, HG, Z;
     float lambda, out_scale, eps;
 };
 
@@ -439,6 +439,21 @@ __device__ __forceinline__ void copy_block(const bf16_t* base, unsigned dst, int
     }
 }
 
+// A sequence's page ids, 64 at a time in a register (lane i: page 64 c + i): the key loop looks them up without a memory round trip.
+struct PageIds {
+    const int32_t* bt;
+    int n, ids, c;
+    __device__ __forceinline__ PageIds(const int32_t* table, int entries, int lane) : bt(table), n(entries), c(0) { fetch(lane); }
+    __device__ __forceinline__ void fetch(int lane) { ids = bt[min(64 * c + lane, n - 1)]; }
+    __device__ __forceinline__ int at(int i, int lane) {                 // i: wave-uniform
+        if ((i >> 6) != c) {
+            c = i >> 6;
+            fetch(lane);
+        }
+        return __builtin_amdgcn_readlane(ids, i & 63);
+    }
+};
+
 template <int DT, int CT, int M>
 __global__ __launch_bounds__(NT, (Shape<DT, CT, M>::PROMPT_OCC)) void maps_prompt_kernel(MapsArgs a) {
     using S = Shape<DT, CT, M>;
@@ -462,7 +477,11 @@ __global__ __launch_bounds__(NT, (Shape<DT, CT, M>::PROMPT_OCC)) void maps_promp
     R.start(a.q + ((size_t)t * a.H + (ok ? head : 0)) * (M * S::DIM), ok, hi);
     const unsigned lds = (unsigned)(size_t)(lds_ptr)smem;
     const int ntiles = p_last / (2 * BN) + 1;
-    auto base_of = [&](int k0) { return pool + ((size_t)bt[k0 / a.page] * a.page + (size_t)(k0 % a.page)) * (size_t)(8 * S::PPR); };
+    PageIds pages(bt, (p_last >> a.page_shift) + 1, lane);
+    auto base_of = [&](int k0) {
+        const int page = pages.at(k0 >> a.page_shift, lane);
+        return pool + (((size_t)page << a.page_shift) + (size_t)(k0 & ((1 << a.page_shift) - 1))) * (size_t)(8 * S::PPR);
+    };
     auto copy_tile = [&](int tile, int buf) {
 #pragma unroll
         for (int b = 0; b < 2; ++b) {
@@ -586,13 +605,13 @@ __global__ __launch_bounds__(NT, (Shape<DT, CT, M>::STEP_OCC)) void maps_step_ke
     const unsigned lds = (unsigned)(size_t)(lds_ptr)smem + w * S::BUFS * S::BLOCK;
     const unsigned char* mine = smem + w * S::BUFS * S::BLOCK;
     const int nT = p_last / BN + 1, stride = NW * a.Z, first = z * NW + w;
-    auto copy = [&](int tile, int buf, int page_id) {
-        const int k0 = tile * BN;
-        copy_block<S>(pool + ((size_t)page_id * a.page + (size_t)(k0 % a.page)) * (size_t)(8 * S::PPR), lds + buf * S::BLOCK, p_last - k0, 0, 1, lane);
+    PageIds pages(bt, (p_last >> a.page_shift) + 1, lane);
+    auto copy = [&](int tile, int buf) {
+        const int k0 = tile * BN, page = pages.at(k0 >> a.page_shift, lane);
+        copy_block<S>(pool + (((size_t)page << a.page_shift) + (size_t)(k0 & ((1 << a.page_shift) - 1))) * (size_t)(8 * S::PPR), lds + buf * S::BLOCK,
+                      p_last - k0, 0, 1, lane);
     };
-    auto page_of = [&](int tile) { return bt[min(tile, nT - 1) * BN / a.page]; };
-    int page_next = page_of(first + stride);
-    if (first < nT) copy(first, 0, page_of(first));
+    if (first < nT) copy(first, 0);
 #pragma unroll
     for (int f = 0; f < M; ++f)
 #pragma unroll
@@ -602,17 +621,15 @@ __global__ __launch_bounds__(NT, (Shape<DT, CT, M>::STEP_OCC)) void maps_step_ke
         const bool more = tile + stride < nT;
         if (S::BUFS == 2 && more) {
             asm volatile("s_waitcnt lgkmcnt(0)" ::: "memory");           // (the other buffer has been read)
-            copy(tile + stride, (i + 1) & 1, page_next);
+            copy(tile + stride, (i + 1) & 1);
             asm volatile("s_waitcnt vmcnt(%0)" ::"n"(S::PPR / 2) : "memory");    // this block has landed, the next one may be on its way
         } else {
             asm volatile("s_waitcnt vmcnt(0)" ::: "memory");
         }
-        const int page_now = page_next;
-        page_next = page_of(tile + 2 * stride);
         R.block(mine + (S::BUFS == 2 ? (i & 1) : 0) * S::BLOCK, tile * BN, p_row, tile * BN + BN - 1 > p_first, lane);
         if (S::BUFS == 1 && more) {
             asm volatile("s_waitcnt lgkmcnt(0)" ::: "memory");
-            copy(tile + stride, 0, page_now);
+            copy(tile + stride, 0);
         }
     }
     // ---- merge the four waves ----
@@ -724,9 +741,9 @@ int head_slots(int per) {
 #define QSV_MAPS_SHAPES(F) F(1, 1, 2) F(2, 1, 2) F(2, 2, 2) F(3, 3, 2) F(4, 2, 2) F(4, 4, 2) F(6, 3, 2) F(8, 4, 2) F(2, 1, 1) F(4, 2, 1) F(6, 3, 1) F(8, 4, 1)
 }  // namespace
 
-// 1 if the matrix-core kernels take these sizes (bfloat16 storage), else 0.
+// 1 if the matrix-core kernels take these sizes (bfloat16 storage, pages a power of two from 32 on), else 0.
 extern "C" int qsv_maps_attention_ok(int dim, int vdim, int maps, int page, int dtype) {
-    if (dtype != QSV_BF16 || page <= 0 || page % BN) return 0;
+    if (dtype != QSV_BF16 || page < BN || (page & (page - 1))) return 0;
 #define QSV_MAPS_OK(DT, CT, M) \
     if (dim == 16 * DT && vdim == 32 * CT && maps == M) return 1;
     QSV_MAPS_SHAPES(QSV_MAPS_OK)
@@ -753,7 +770,7 @@ extern "C" int qsv_maps_attention(void* out, const void* q, const void* pool, co
     const int per = H / G, HG = (per + 31) / 32;
     QSV_REQUIRE((int64_t)n_prompt * G * HG < (1ll << 31) && G * HG <= 65535, "qsv_maps_attention: too many tiles");
     MapsArgs a = {(bf16_t*)out, (const bf16_t*)q, (const bf16_t*)pool, (const bf16_t*)gate, block_table, pos, nullptr, part_o, part_ml, pool_stride,
-                  gate_stride, table_stride, 0, H, per, page, head_slots(per), 32 / head_slots(per), HG, key_splits, lambda, out_scale, eps};
+                  gate_stride, table_stride, 0, H, per, __builtin_ctz(page), head_slots(per), 32 / head_slots(per), HG, key_splits, lambda, out_scale, eps};
 #define QSV_MAPS_RUN(DT, CT, M)                      \
     if (dim == 16 * DT && vdim == 32 * CT && maps == M) \
         return launch_maps<DT, CT, M>(a, prompt_tiles, n_prompt, step_tiles, n_step, G, (hipStream_t)stream);

@@ -551,16 +551,51 @@ class HipOps:
                                                float(coef), float(every), T, self.code, self._s()), "conv_heads_cache")
         return q
 
+    step_split_target = 256             # workgroups a launch of the step kernel should at least have (one per CU)
+
+    def maps_attention_ok(self, dim, vdim, maps, page):
+        """Whether the matrix-core kernels of one or two key maps take these sizes."""
+        return bool(self.L.qsv_maps_attention_ok(dim, vdim, maps, page, self.code))
+
+    def single_map_attention(self, q, pool, batch, heads, dim, vdim, page, key_splits=None):
+        """q [T, heads * dim] (storage type, scaled), pool [G, rows, vdim + dim] of rows [v | k]: causal softmax attention -> [T, heads * vdim];
+        only for sizes that `maps_attention_ok` takes."""
+        T = q.size(0)
+        self._need(q, pool, batch.block_table, batch.pos)
+        assert q.numel() == T * heads * dim and q.dtype == self.dtype == pool.dtype and pool.size(2) == vdim + dim and heads % pool.size(0) == 0
+        out = torch.empty((T, heads * vdim), dtype=self.dtype, device=q.device)
+        return self._maps_attention(out, q, pool, batch, heads, dim, vdim, 1, page, (0.0, 1.0, 0.0, 0, 0), key_splits)
+
+    def _maps_attention(self, out, q, pool, batch, heads, dim, vdim, maps, page, epilogue, key_splits):
+        G, bt = pool.size(0), batch.block_table
+        per = heads // G
+        prompt, step = batch.split_tiles(self.L.qsv_maps_attention_tile_tokens(per))
+        groups, n = G * self.L.qsv_maps_attention_head_groups(per), step.size(0)
+        splits, po, pm = 1, None, None
+        if n:                                                # few workgroups and long contexts: the keys are cut over several
+            splits = max(1, min(self.step_split_target // (n * groups), (batch.max_pos + 1) // 256, 32)) if key_splits is None else key_splits
+        if splits > 1:
+            po = torch.empty((splits, n, groups, 32, maps, vdim), dtype=torch.float32, device=q.device)
+            pm = torch.empty((splits, n, groups, 32, maps, 2), dtype=torch.float32, device=q.device)
+        self.check(self.L.qsv_maps_attention(out.data_ptr(), q.data_ptr(), pool.data_ptr(), bt.data_ptr(), bt.stride(0), batch.pos.data_ptr(),
+                                             prompt.data_ptr() if prompt.size(0) else 0, prompt.size(0), step.data_ptr() if n else 0, n, heads, G,
+                                             dim, vdim, maps, page, pool.stride(0), *epilogue, splits, 0 if po is None else po.data_ptr(),
+                                             0 if pm is None else pm.data_ptr(), self._s()), "maps_attention")
+        return out
+
     def diff_attention(self, q, pool, batch, heads, dim, vdim, lam, out_scale, eps, gate, page, variant=0, key_splits=None):
         """q [T, heads * 2 * dim] (storage type, scaled; per head map 1, map 2), pool [G, rows, vdim + 2 dim] of rows [v | k_1 | k_2]: with a_m the
         softmax attention of map m over the keys up to the token, o = a_1 - lam a_2; -> o / sqrt(mean(o^2) + eps) * out_scale * sigmoid(gate) [T,
-        heads * vdim] (gate [T, heads * vdim], a column slice is fine, or None)."""
+        heads * vdim] (gate [T, heads * vdim], a column slice is fine, or None).  variant: 0 = the matrix-core kernels where they take the
+        sizes, 1 = the wave kernel."""
         T, G = q.size(0), pool.size(0)
         self._need(q, pool, batch.block_table, batch.seq, batch.pos)
         assert q.shape == (T, heads * 2 * dim) and q.dtype == self.dtype == pool.dtype and pool.size(2) == vdim + 2 * dim and heads % G == 0
         assert gate is None or (gate.dtype == self.dtype and gate.stride(1) == 1 and gate.shape == (T, heads * vdim))
         out = torch.empty((T, heads * vdim), dtype=self.dtype, device=q.device)
         bt, ep = batch.block_table, (float(lam), float(out_scale), float(eps), 0 if gate is None else gate.data_ptr(), 0 if gate is None else gate.stride(0))
+        if variant == 0 and self.maps_attention_ok(dim, vdim, 2, page) and (gate is None or (gate.stride(0) % 4 == 0 and gate.data_ptr() % 8 == 0)):
+            return self._maps_attention(out, q, pool, batch, heads, dim, vdim, 2, page, ep, key_splits)
         self.check(self.L.qsv_diff_attention(out.data_ptr(), q.data_ptr(), pool.data_ptr(), bt.data_ptr(), bt.stride(0), batch.seq.data_ptr(),
                                              batch.pos.data_ptr(), T, heads, G, dim, vdim, page, pool.stride(0), *ep, self.code, self._s()),
                    "diff_attention")
@@ -1189,6 +1224,9 @@ class TorchOps:
             coef, every = temperature
             q = q * (1.0 + coef * torch.log(torch.floor((batch.pos.double() + 1.0) / every).float() + 1.0))[:, None]
         return q.to(self.dtype)
+
+    def maps_attention_ok(self, dim, vdim, maps, page):
+        return False
 
     def diff_attention(self, q, pool, batch, heads, dim, vdim, lam, out_scale, eps, gate, page, variant=0, key_splits=None):
         T, G = q.size(0), pool.size(0)

@@ -339,7 +339,11 @@ class TiedRotaryAttention:
         proj = linear(h, self.w_in)
         k = proj[:, H * d:]
         rope = rot.reserve(batch.max_pos + 1) if rot is not None else None
-        qf = ops.qk_norm_rope_prep(proj[:, :H * d], k, k, H, G, d, d, None, None, True, self.eps, rope, rot.dims if rot is not None else 0,
-                                   self.scale, pool, batch, halves=True, rot_gain=rot.magnitude ** 2 if rot is not None else 0.0)
-        o = ops.latent_attention(qf, pool, batch, None, d, self.page, q_first=d)
+        plain = ops.maps_attention_ok(d, d, 1, self.page)        # queries in the storage type without the zeros in front
+        q = ops.qk_norm_rope_prep(proj[:, :H * d], k, k, H, G, d, d, None, None, True, self.eps, rope, rot.dims if rot is not None else 0,
+                                  self.scale, pool, batch, halves=True, rot_gain=rot.magnitude ** 2 if rot is not None else 0.0,
+                                  q_pad=0 if plain else d, q_store=plain)
+        if plain:
+            return linear(ops.single_map_attention(q, pool, batch, H, d, d, self.page), self.w_o)
+        o = ops.latent_attention(q, pool, batch, None, d, self.page, q_first=d)
         return linear(o.view(T, H * d), self.w_o)

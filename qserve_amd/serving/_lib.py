@@ -63,6 +63,11 @@ SIGNATURES = {
                                    _vp, _vp, _i, _vp, _vp, _vp, _i, _vp, _i, _f, _i, _i, _vp]),
     "qsv_conv_heads_cache": (_i, [_vp, _vp, _i64, _vp, _i64, _vp, _i, _vp, _vp, _vp, _vp, _vp, _vp, _i, _i, _i, _i, _f, _f, _d, _i, _i, _vp]),
     "qsv_diff_attention": (_i, [_vp, _vp, _vp, _vp, _i, _vp, _vp, _i, _i, _i, _i, _i, _i, _i64, _f, _f, _f, _vp, _i64, _i, _vp]),
+    "qsv_maps_attention_ok": (_i, [_i, _i, _i, _i, _i]),
+    "qsv_maps_attention_tile_tokens": (_i, [_i]),
+    "qsv_maps_attention_head_groups": (_i, [_i]),
+    "qsv_maps_attention": (_i, [_vp, _vp, _vp, _vp, _i, _vp, _vp, _i, _vp, _i, _i, _i, _i, _i, _i, _i, _i64, _f, _f, _f, _vp, _i64, _i, _vp, _vp,
+                                _vp]),
     "qsv_recurrent_scan": (_i, [_vp, _vp, _i64, _vp, _i64, _vp, _i64, _i, _vp, _vp, _i64, _i, _vp, _vp, _i, _i, _i, _i, _i, _i, _f, _vp,
                                 _i, _i, _vp]),
     "qsv_head_rms_gate": (_i, [_vp, _vp, _vp, _vp, _i64, _i, _f, _i, _i, _i, _i, _i, _vp, _i, _vp]),

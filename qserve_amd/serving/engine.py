@@ -56,6 +56,19 @@ class StepBatch:
             self._tiles[tokens_per_tile] = t
         return t
 
+    def split_tiles(self, tokens_per_step_tile):
+        """Work tiles for kernels with a form of their own for short runs: -> (prompt tiles, step tiles), int32 [n, 3] as `tiles`.  Runs of at
+        most `tokens_per_step_tile` tokens become one step tile each, longer ones prompt tiles of up to four times as many tokens."""
+        n = int(tokens_per_step_tile)
+        key = ("split", n)
+        if key not in self._tiles:
+            short = [run for run in self.items if run[2] <= n]
+            long = [(slot, first + o, min(4 * n, cnt - o)) for slot, first, cnt in self.items if cnt > n for o in range(0, cnt, 4 * n)]
+            both = torch.tensor(short + long, dtype=torch.int32).reshape(-1, 3).to(self.pos.device)
+            self._tiles[key] = both
+        both, k = self._tiles[key], sum(1 for run in self.items if run[2] <= n)
+        return both[k:], both[:k]
+
 
 class Engine:
     def __init__(self, model_cls, config, weights, dtype="bfloat16", device="cuda:0", max_tokens=4096, max_seqs=4,

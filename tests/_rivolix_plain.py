@@ -214,7 +214,7 @@ def random_weights(cfg, seed=0):
             W[p + "norm2"], W[p + "ls2"] = rnd(D, s=0.2), rnd(D, s=0.3, mean=0.7)
             q = p + "mlp."
             E, ff = mlp["router"]["experts"], mlp["expert"]["ff"]
-            W[q + "router"] = mat(E, D, 3.0)
+            W[q + "router"] = mat(E, D)
             units = [(f"{q}e{e}.", ff) for e in range(E)] + ([(q + "shared.", mlp["shared"]["ff"])] if mlp.get("shared") else [])
             for name, n in units:
                 W.update({name + "gate": mat(n, D, 1.5), name + "up": mat(n, D, 1.5), name + "down": mat(D, n)})
