@@ -5,6 +5,7 @@
     python bench.py --design vepolix  [--design-sizes w2048,w4096] [--steps K] [--warmup W]     beside Mumelix
     python bench.py --design pemolorn [--design-sizes w2048,w4096] [--steps K] [--warmup W]     beside Mumelix
     python bench.py --design sagupel  [--design-sizes w2048,w4096] [--steps K] [--warmup W]     beside Mumelix
+    python bench.py --design rivolix  [--design-sizes w2048,w4096] [--steps K] [--warmup W]     beside Vepolix
 
 Per size (random weights, 4 layers, vocabulary 32000): prompt phase = 8 prompts x 1024 tokens in one step through
 Engine.execute; decoding = 64 sequences at context 1024, one token each per step.  Beside them the Llama-style W4A8KV4
@@ -80,7 +81,8 @@ class OpTimer:
              "moe_route", "moe_experts", "embed_streams", "hc_read", "hc_write", "dyt_sum_rows", "rms_pair_mean", "glu",
              "attention_prep", "rotate_heads", "decay", "conv_silu_unit", "recurrent_scan", "head_rms_gate", "embed_sinusoid",
              "add_rms_norm", "rms_norm_rows", "normed_attention_prep", "max_gates", "add_normed_rms_norm", "qk_norm_rope_prep", "pool_blocks",
-             "min_gru_scan", "relu_sq", "embed_rms_norm", "residual_conv", "scaled_add_rms_norm", "rotate_qk", "talking_attention")
+             "min_gru_scan", "relu_sq", "embed_rms_norm", "residual_conv", "scaled_add_rms_norm", "rotate_qk", "talking_attention",
+             "scaled_sum_rms_norms", "conv_heads_cache", "diff_attention", "single_map_attention")
 
     def __init__(self, ops):
         self.ops, self.events, self.calls, self.on = ops, [], [], False
@@ -95,7 +97,7 @@ class OpTimer:
         import importlib
         return [importlib.import_module("qserve_amd." + m) for m in
                 ("layers.latent_attention", "layers.moe", "layers.recurrent", "layers.softmax_attention", "models.vekalorn",
-                 "models.mumelix", "models.vepolix", "models.pemolorn", "models.sagupel")]
+                 "models.mumelix", "models.vepolix", "models.pemolorn", "models.sagupel", "models.rivolix")]
 
     def _wrap(self, name, fn):
         def timed(*a, **k):
@@ -520,6 +522,9 @@ def bench_vepolix(name, s, dev, steps, warmup):
     # writes the next input; the first call only norms, the last only adds
     res_bytes = T * (LAYERS * (8.0 * D + 2.0 * D) + (2 * n_att + 3 * n_rec) * 2.0 * D)
     res_pre = res_bytes / (rep_pre["add_rms_norm"] * 1e-3) / 1e9
+    # query / key preparation: the projections in, queries (storage type) and cache rows out
+    prep_bytes = n_att * T * 2.0 * (2 * m["a_heads"] * m["a_dim"] + 2 * m["a_kv"] * R)
+    prep_pre = prep_bytes / (rep_pre["normed_attention_prep"] * 1e-3) / 1e9
     out = dict(model=f"Vepolix-{name}", sizes=m, prefill_tokens_per_s=T / pre * 1e3, prefill_ms=pre, decode_tokens_per_s=NB / dec * 1e3,
                decode_ms=dec, decode_from_hipgraph=graph_ok, decode_ms_eager=dec_eager, decode_ms_gpu_events=dec_events_ms, context=ctx,
                prefill_ops_ms=ops_pre, decode_ops_ms=ops_dec, prefill_kernels_ms=rep_pre, decode_kernels_ms=rep_dec,
@@ -529,6 +534,7 @@ def bench_vepolix(name, s, dev, steps, warmup):
                              decode_experts_gbs=moe_dec, decode_experts_frac_hbm=moe_dec / HBM_PEAK_GBS,
                              prefill_recurrence_tflops=scan_pre, prefill_recurrence_frac_fp32_valu_peak=scan_pre / FP32_VALU_PEAK_TFLOPS,
                              decode_recurrence_gbs=scan_dec, decode_recurrence_frac_hbm=scan_dec / HBM_PEAK_GBS,
+                             prefill_prep_gbs=prep_pre, prefill_prep_frac_hbm=prep_pre / HBM_PEAK_GBS,
                              prefill_residual_kernel_gbs=res_pre, prefill_residual_kernel_frac_hbm=res_pre / HBM_PEAK_GBS))
     for sl in slots:
         eng.close_sequence(sl)
@@ -823,6 +829,130 @@ def bench_sagupel(name, s, dev, steps, warmup):
     return out
 
 
+# ---- Rivolix ----------------------------------------------------------------------------------------------------------------
+def rivolix_config(s, m):
+    """Vepolix's sizes in Rivolix's layers: differential attention with the heads, value size and cache rows of its attention (two maps of half
+    the key size), tied rotary attention with those heads and rows, the same experts and shared expert on every layer.  Layers: differential,
+    tied, differential on the first layer's cache, tied."""
+    mlp = {"kind": "moe", "expert": {"ff": s["ff"]}, "shared": {"ff": s["ff"]}, "router": {"experts": s["experts"], "top": s["top"]}}
+    H, G, d = m["a_heads"], m["a_kv"], m["a_dim"]
+    a = {"heads": H, "kv_heads": G, "dim": d // 2, "vdim": m["a_vdim"], "conv": m["taps"], "diff": 0.35, "q_temp": {"coef": 0.2, "every": 512},
+         "scale": 1.0 / math.sqrt(d // 2)}
+    b = {"heads": H, "kv_heads": G, "dim": d, "vdim": d, "scale": 1.0 / math.sqrt(d),
+         "rot": {"base": 500000.0, "dims": d, "scaling": {"factor": 4.0, "original": 8192, "fast": 32.0, "slow": 1.0}}}
+    one, two = {"type": "attention", "mixer": a, "mlp": mlp}, {"type": "attention_2", "mixer": b, "mlp": mlp}
+    return {"architecture": "Rivolix", "width": s["width"], "vocab": VOCAB, "norm": {"eps": 1e-5},
+            "layers": [one, two, dict(one, mixer=dict(a, kv_from=0)), two][:LAYERS]}
+
+
+def rivolix_weights(cfg, dev, seed=0):
+    g = torch.Generator(device=dev).manual_seed(seed)
+    D, V = cfg["width"], cfg["vocab"]
+
+    def mat(o, i, s=1.0):
+        return (torch.randn((o, i), device=dev, generator=g) * (s / math.sqrt(i))).bfloat16()
+
+    def vec(n, mean=0.0, s=0.1):
+        return (mean + s * torch.randn((n,), device=dev, generator=g)).bfloat16()
+
+    W = {"embed": mat(V, D, math.sqrt(D)), "final.norm": vec(D)}
+    for i, L in enumerate(cfg["layers"]):
+        p, x, q = f"l{i}.", L["mixer"], f"l{i}.mix."
+        W.update({p + "norm1": vec(D), p + "norm2": vec(D), p + "ls1": vec(D, 0.8), p + "ls2": vec(D, 0.8)})
+        H, G, d, dv = x["heads"], x["kv_heads"], x["dim"], x["vdim"]
+        if L["type"] == "attention":
+            W.update({q + "q": mat(2 * H * d, D), q + "q.conv": mat(2 * H * d, x["conv"]), q + "g": mat(H * dv, D), q + "o": mat(D, H * dv)})
+            W.update({q + n: vec(d) for n in ("lq1", "lk1", "lq2", "lk2")})
+            if x.get("kv_from") is None:
+                W.update({q + "k": mat(2 * G * d, D), q + "v": mat(G * dv, D), q + "k.conv": mat(2 * G * d, x["conv"]), q + "v.conv": mat(G * dv, x["conv"])})
+        else:
+            W.update({q + "q": mat(H * d, D), q + "k": mat(G * d, D), q + "o": mat(D, H * d)})
+        mlp, q = L["mlp"], p + "mlp."
+        for e in [f"e{k}." for k in range(mlp["router"]["experts"])] + ["shared."]:
+            ff = mlp["shared" if e == "shared." else "expert"]["ff"]
+            W[q + e + "gate"], W[q + e + "up"], W[q + e + "down"] = mat(ff, D), mat(ff, D), mat(D, ff)
+        W[q + "router"] = mat(mlp["router"]["experts"], D, 3.0)
+    return W
+
+
+def bench_rivolix(name, s, dev, steps, warmup):
+    from ..models.rivolix import Rivolix
+    from .engine import Engine
+    m = MUMELIX[name]
+    cfg = rivolix_config(s, m)
+    NB, L, BP = 64, 1024, 8
+    eng = Engine(Rivolix, cfg, rivolix_weights(cfg, dev), dtype="bfloat16", device=dev, max_tokens=NB * (L + 384), max_seqs=NB)
+    timer = OpTimer(eng.ops)
+    g = torch.Generator().manual_seed(1)
+    prompts = [torch.randint(0, VOCAB, (L,), generator=g).tolist() for _ in range(NB)]
+    slots = [eng.open_sequence() for _ in range(NB)]
+    stateless = ("diff_attention", "single_map_attention", "scaled_sum_rms_norms", "conv_heads_cache", "qk_norm_rope_prep", "glu", "moe_route")
+    pre_ms, ops_pre, rep_pre = [], None, {}
+    for i in range(0, NB, BP):
+        items = [(slots[j], prompts[j]) for j in range(i, i + BP)]
+        want = [k * L + L - 1 for k in range(BP)]
+        if i == BP:                                          # one step with events around every launch
+            ops_pre, _ = timer.step(lambda: eng.execute(items, want))
+            rep_pre = {k: timer.replay(k, 3) for k in stateless}     # (the convolution writes the same history again)
+            continue
+        torch.cuda.synchronize()
+        t0 = time.perf_counter()
+        eng.execute(items, want)
+        torch.cuda.synchronize()
+        if i > 0:
+            pre_ms.append((time.perf_counter() - t0) * 1e3)
+    pre = sorted(pre_ms)[len(pre_ms) // 2]
+    nxt = [[int(torch.randint(0, VOCAB, (1,), generator=g))] for _ in range(NB)]
+    want = list(range(NB))
+
+    def decode():
+        eng.execute([(slots[j], nxt[j]) for j in range(NB)], want)
+
+    dec_eager = timed(decode, steps, warmup)
+    ops_dec, dec_events_ms = timer.step(decode)
+    rep_dec = {k: timer.replay(k, 20) for k in stateless + ("moe_experts",)}
+    eng.decode_graphs = True
+    dec = timed(decode, steps, warmup)
+    graph_ok = any(v is not False for v in eng._graphs.values()) and bool(eng._graphs)
+    ctx = eng.cache.length[slots[0]]
+    T, D = BP * L, s["width"]
+    kinds = [x["type"] for x in cfg["layers"]]
+    n_diff, n_tied = kinds.count("attention"), kinds.count("attention_2")
+    own = sum(1 for x in cfg["layers"] if x["type"] == "attention" and x["mixer"].get("kv_from") is None)
+    H, G, d, dv = m["a_heads"], m["a_kv"], m["a_dim"], m["a_vdim"]
+    R = d + dv                                               # (two maps of d / 2, or one of d)
+    pairs = BP * sum(p + 1 for p in range(L))
+    # useful work per visible pair: the two maps' q.k and p.v; one q.k and p.v
+    diff_pre = n_diff * pairs * H * (d + 2 * dv) * 2.0 / (rep_pre["diff_attention"] * 1e-3) / 1e12
+    tied_pre = n_tied * pairs * H * 2 * d * 2.0 / (rep_pre["single_map_attention"] * 1e-3) / 1e12
+    diff_dec = n_diff * NB * ctx * G * R * 2.0 / (rep_dec["diff_attention"] * 1e-3) / 1e9
+    tied_dec = n_tied * NB * ctx * G * 2 * d * 2.0 / (rep_dec["single_map_attention"] * 1e-3) / 1e9
+    moe_pre = LAYERS * T * s["top"] * 3 * 2.0 * s["ff"] * D / (ops_pre["moe_experts"] * 1e-3) / 1e12
+    moe_dec = LAYERS * min(s["experts"], NB * s["top"]) * 3 * s["ff"] * D * 2.0 / (rep_dec["moe_experts"] * 1e-3) / 1e9
+    # residual kernel: the float stream in and out and two casts per layer; mixer, routed and shared outputs in; the first call gathers
+    res_pre = T * (LAYERS * (8.0 * D + 3 * 2.0 * D + 2 * 2.0 * D) + 6.0 * D) / (rep_pre["scaled_sum_rms_norms"] * 1e-3) / 1e9
+    # preparation: the projections in, queries and cache rows out
+    conv_pre = T * 2.0 * (n_diff * 2 * H * d + own * 2 * G * R) / (rep_pre["conv_heads_cache"] * 1e-3) / 1e9
+    prep_pre = n_tied * T * 2.0 * (2 * H * d + G * d + G * 2 * d) / (rep_pre["qk_norm_rope_prep"] * 1e-3) / 1e9
+    out = dict(model=f"Rivolix-{name}", sizes=m, prefill_tokens_per_s=T / pre * 1e3, prefill_ms=pre, decode_tokens_per_s=NB / dec * 1e3,
+               decode_ms=dec, decode_from_hipgraph=graph_ok, decode_ms_eager=dec_eager, decode_ms_gpu_events=dec_events_ms, context=ctx,
+               prefill_ops_ms=ops_pre, decode_ops_ms=ops_dec, prefill_kernels_ms=rep_pre, decode_kernels_ms=rep_dec,
+               roofline=dict(prefill_diff_attention_tflops=diff_pre, prefill_diff_attention_frac_bf16_peak=diff_pre / BF16_PEAK_TFLOPS,
+                             decode_diff_attention_gbs=diff_dec, decode_diff_attention_frac_hbm=diff_dec / HBM_PEAK_GBS,
+                             prefill_tied_attention_tflops=tied_pre, prefill_tied_attention_frac_bf16_peak=tied_pre / BF16_PEAK_TFLOPS,
+                             decode_tied_attention_gbs=tied_dec, decode_tied_attention_frac_hbm=tied_dec / HBM_PEAK_GBS,
+                             prefill_experts_tflops=moe_pre, prefill_experts_frac_bf16_peak=moe_pre / BF16_PEAK_TFLOPS,
+                             decode_experts_gbs=moe_dec, decode_experts_frac_hbm=moe_dec / HBM_PEAK_GBS,
+                             prefill_residual_kernel_gbs=res_pre, prefill_residual_kernel_frac_hbm=res_pre / HBM_PEAK_GBS,
+                             prefill_conv_prep_gbs=conv_pre, prefill_conv_prep_frac_hbm=conv_pre / HBM_PEAK_GBS,
+                             prefill_tied_prep_gbs=prep_pre, prefill_tied_prep_frac_hbm=prep_pre / HBM_PEAK_GBS))
+    for sl in slots:
+        eng.close_sequence(sl)
+    del eng
+    torch.cuda.empty_cache()
+    return out
+
+
 def main(args, helpers):
     dev = "cuda:0"
     torch.cuda.set_device(0)
@@ -832,12 +962,15 @@ def main(args, helpers):
         build.build(verbose=False)
     steps, warmup = min(args.steps, 32), min(args.warmup, 8)
     for name in args.design_sizes.split(","):
-        if args.design in ("mumelix", "vepolix", "pemolorn", "sagupel") and name not in MUMELIX:      # (sizes that differ in a Vekalorn-only constant)
+        if args.design in ("mumelix", "vepolix", "pemolorn", "sagupel", "rivolix") and name not in MUMELIX:      # (sizes that differ in a Vekalorn-only constant)
             continue
         s = SIZES[name]
         line = {"design": args.design, "size": name, "sizes": s, "layers": LAYERS, "vocab": VOCAB, "dtype": "bf16",
                 "data": "synthetic", "workload": "prefill 8 x 1024 tokens in one step; decode 64 sequences at context 1024"}
-        if args.design == "sagupel":
+        if args.design == "rivolix":
+            line["rivolix"] = bench_rivolix(name, s, dev, steps, warmup)
+            line["vepolix"] = bench_vepolix(name, s, dev, steps, warmup)
+        elif args.design == "sagupel":
             line["sagupel"] = bench_sagupel(name, s, dev, steps, warmup)
             line["mumelix"] = bench_mumelix(name, s, dev, steps, warmup)
         elif args.design == "pemolorn":

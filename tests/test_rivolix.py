@@ -238,10 +238,10 @@ def test_query_temperature_steps(backend):
     b = run_batch(0, len(pos), dev)
     b.pos, b.slot = pos.to(dev), torch.zeros(len(pos), dtype=torch.int64, device=dev)
     proj, w = torch.ones(len(pos), 4, device=dev), torch.ones(1, 4, device=dev)
-    for coef, every in ((0.5, 64), (2.0, 63), (0.1, 1)):
+    for coef, every in ((0.7, 64), (2.0, 63), (0.1, 1)):
         q = ops.conv_heads_cache(proj, w, None, b, 4, 0, 0, 4, None, 1.0, (coef, every))
         assert_close(q[:, 0].double().cpu(), P.temperature(pos.numpy(), coef, every), 1e-6, f"every {every}")
-    q = ops.conv_heads_cache(proj, w, None, b, 4, 0, 0, 4, None, 1.0, (0.5, 64))[:, 0].cpu()
+    q = ops.conv_heads_cache(proj, w, None, b, 4, 0, 0, 4, None, 1.0, (0.7, 64))[:, 0].cpu()
     assert q[1] < q[2] and q[2] == q[3] == q[4] and q[4] < q[5] and q[8] < q[9]
 
 
@@ -328,7 +328,7 @@ def test_tied_rotary_attention_layer_alone(backend):
     _mixer_alone(backend, tied(), 70, [])
     _mixer_alone(backend, tied(), 70, [1, 2, 3, 5, 31, 32, 33, 63, 64, 65, 69])
     _mixer_alone(backend, tied(heads=5, kv_heads=1, dim=6, rot=6, factor=None), 140, [63, 64, 65, 128, 129])
-    _mixer_alone(backend, tied(heads=4, kv_heads=4, dim=64, rot=64, base=1e6, factor=8.0, original=512, fast=32.0, slow=1.0), 40, [7])
+    _mixer_alone(backend, tied(heads=4, kv_heads=4, dim=64, rot=64, base=2e5, factor=5.0, original=512, fast=24.0, slow=1.5), 40, [7])
     _mixer_alone(backend, tied(heads=1, kv_heads=1, dim=2, rot=2), 10, [5])
 
 
@@ -338,7 +338,7 @@ def test_mixers_at_the_matrix_core_sizes(dtype):
     """Sizes the matrix-core kernels take, and some that fall back; prompt tiles, short runs beside long ones, head groups beyond 32."""
     if not torch.cuda.is_available():
         pytest.skip("no GPU")
-    for layers, T, splits in ((diff(heads=4, kv_heads=2, dim=32, vdim=64, conv=4), 300, [87, 88, 89, 126, 170, 298, 299]),
+    for layers, T, splits in ((diff(heads=6, kv_heads=3, dim=32, vdim=64, conv=3), 300, [87, 88, 89, 126, 170, 298, 299]),
                               (diff(heads=6, kv_heads=1, dim=16, vdim=32), 330, [43, 47, 53, 54, 126, 170, 328, 329]),
                               (diff(heads=8, kv_heads=2, dim=64, vdim=128, conv=2), 200, [150, 151, 153, 190]),
                               (diff(heads=3, kv_heads=1, dim=64, vdim=64), 140, [100, 101, 102, 139]),
@@ -347,8 +347,8 @@ def test_mixers_at_the_matrix_core_sizes(dtype):
                               (diff(heads=40, kv_heads=1, dim=16, vdim=32), 90, [33, 34, 80]),
                               (diff(heads=2, kv_heads=2, dim=128, vdim=128), 100, [50, 51, 99]),
                               (diff(heads=4, kv_heads=2, dim=24, vdim=40), 100, [50, 51, 99]),         # (wave kernel)
-                              ([diff(heads=4, kv_heads=2, dim=32, vdim=64), diff(heads=12, kv_heads=2, dim=32, vdim=64, kv_from=0)], 150, [64, 66, 70, 149]),
-                              (tied(heads=8, kv_heads=4, dim=64, rot=64), 300, [87, 88, 89, 126, 170, 298, 299]),
+                              ([diff(heads=6, kv_heads=3, dim=32, vdim=64), diff(heads=12, kv_heads=3, dim=32, vdim=64, kv_from=0)], 150, [64, 66, 70, 149]),
+                              (tied(heads=6, kv_heads=2, dim=64, rot=64), 300, [87, 88, 89, 126, 170, 298, 299]),
                               (tied(heads=3, kv_heads=1, dim=32, rot=8), 150, [100, 101, 102, 140]),
                               (tied(heads=4, kv_heads=2, dim=96, rot=64), 130, [64, 65, 129]),
                               (tied(heads=8, kv_heads=1, dim=128, rot=128), 130, [64, 65, 129]),
@@ -671,7 +671,7 @@ def test_other_sizes(backend, variant):
           diff(heads=4, kv_heads=4, dim=32, vdim=32, conv=4, kv_from=1, mlp=None)], dict(width=96, vocab=200)),
         ([diff(heads=7, kv_heads=1, dim=70, vdim=12, conv=3), diff(heads=7, kv_heads=1, dim=70, vdim=12, kv_from=0), diff(heads=2, kv_heads=1, dim=70, vdim=12, kv_from=0, conv=2)],
          dict(width=41, vocab=33, eps=1e-6)),
-        ([tied(heads=2, kv_heads=2, dim=4, rot=4, factor=32.0, original=4096, fast=32.0, slow=1.0, base=1e6, mlp=moe())] * 3, dict(width=48, vocab=61)),
+        ([tied(heads=2, kv_heads=2, dim=4, rot=4, factor=30.0, original=4096, fast=20.0, slow=2.0, base=9e5, mlp=moe())] * 3, dict(width=48, vocab=61)),
         ([diff(mlp=None, lam=0.0, coef=0.0)], dict(width=20, vocab=9)),
     ][variant]
     cfg = make_config(layers, **kw)
@@ -832,8 +832,8 @@ def test_decode_steps_from_a_graph_match_eager_steps(dtype, sizes, std):
         pytest.skip("no GPU")
     cfg, W, seqs, _, _ = std
     if sizes == "matrix-core":
-        cfg = make_config([diff(heads=4, kv_heads=2, dim=32, vdim=64, conv=4, mlp=moe(4, 2, 64, 64)), tied(heads=4, kv_heads=2, dim=64, rot=32, mlp=moe(4, 1, 64, None)),
-                           diff(heads=4, kv_heads=2, dim=32, vdim=64, kv_from=0, mlp=None)], width=64)
+        cfg = make_config([diff(heads=6, kv_heads=3, dim=32, vdim=64, conv=3, mlp=moe(4, 2, 64, 64)), tied(heads=4, kv_heads=2, dim=64, rot=32, mlp=moe(4, 1, 64, None)),
+                           diff(heads=9, kv_heads=3, dim=32, vdim=64, kv_from=0, mlp=None)], width=64)
         W = P.random_weights(cfg, seed=12)
     outs = []
     for graphs in (False, True):
