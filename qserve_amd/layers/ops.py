@@ -372,7 +372,7 @@ class HipOps:
         q_pad = vdim if q_pad is None else int(q_pad)
         qf = torch.empty((T, heads, q_pad + dim), dtype=self.dtype if q_store else torch.float32, device=q.device)
         self._need(q_w, k_w, rope, pool, batch.slot, batch.pos, q_b, k_b, v_b, head_scale)
-        assert q.stride(1) == 1 and q.size(1) == heads * dim and (per_head or q_w is not None) and (q_w is None) == (k_w is None or k is None)
+        assert q.stride(1) == 1 and q.size(1) == heads * dim and (per_head or q_w is not None) and (k is None or (q_w is None) == (k_w is None))
         assert q_w is None or (q_w.dtype == self.dtype and q_w.numel() == (dim if per_head else heads * dim))
         assert rope is None or (rope.dtype == torch.float32 and rope.size(-1) * 2 == rot_n and rot_n <= dim and rope.size(0) > batch.max_pos)
         for b, n in ((q_b, heads * dim), (k_b, kv_heads * dim), (v_b, kv_heads * vdim)):

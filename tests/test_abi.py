@@ -132,6 +132,18 @@ def test_serve_argument_validation_without_gpu():
     assert L.qsv_residual_conv(1, 1, 1, 3, None, 1, 1, 1, 2, 8, 0, None) == 1                                  # three taps without a history
     assert L.qsv_scaled_add_rms_norm(1, None, 1, 2.0, 1, 1e-5, 1, 3, 1, 1, 1, 2, 8, 0, None) == 1              # a convolution without its output
     assert L.qsv_rotate_qk(1, 1, 64, 2, 8, 8, 1, 10, 1, 2, 0, None) == 1                                       # 10 rotated dimensions of 8
+    assert [L.qsv_maps_attention_ok(*a) for a in ((32, 64, 2, 64, 0), (64, 128, 2, 64, 0), (64, 64, 1, 32, 0), (40, 64, 2, 64, 0), (64, 64, 1, 96, 0), (64, 64, 1, 64, 1),
+                                                  (64, 64, 3, 64, 0))] == [1, 1, 1, 0, 0, 0, 0]
+    assert [L.qsv_maps_attention_tile_tokens(h) for h in (1, 3, 4, 20, 40)] == [32, 8, 8, 1, 1]
+    assert [L.qsv_maps_attention_head_groups(h) for h in (1, 32, 33, 65)] == [1, 1, 2, 3]
+    assert L.qsv_maps_attention(64, 64, 64, 1, 4, 1, 1, 1, None, 0, 3, 2, 32, 64, 2, 64, 0, 0.5, 0.5, 1e-5, None, 0, 1, None, None, None) == 1    # 3 heads over 2
+    assert L.qsv_maps_attention(64, 64, 64, 1, 4, 1, None, 0, 1, 1, 4, 2, 32, 64, 2, 64, 0, 0.5, 0.5, 1e-5, None, 0, 3, None, None, None) == 1  # splits without workspace
+    assert L.qsv_maps_attention(64, 64, 64, 1, 4, 1, 1, 1, None, 0, 4, 2, 32, 64, 2, 64, 0, 0.5, 0.5, 1e-5, 4, 256, 1, None, None, None) == 1   # an unaligned gate
+    assert L.qsv_diff_attention(1, 1, 1, 1, 4, 1, 1, 2, 4, 2, 600, 64, 64, 0, 0.5, 0.5, 1e-5, None, 0, 0, None) == 1                         # heads of 600
+    assert L.qsv_conv_heads_cache(1, None, 0, 1, 64, 1, 4, None, 1, 1, 1, None, 1, 32, 0, 0, 8, 1.0, 0.0, 0.0, 2, 0, None) == 1               # four taps without a history
+    assert L.qsv_conv_heads_cache(1, None, 0, 1, 64, 1, 1, None, 1, 1, 1, None, 1, 32, 2, 8, 8, 1.0, 0.0, 0.0, 2, 0, None) == 1               # keys without a cache
+    assert L.qsv_scaled_sum_rms_norms(1, 1, 1, None, None, None, None, None, None, 1, None, None, None, 1e-5, 2, 8, 0, None) == 1              # a second norm without its gain
+    assert L.qsv_qk_norm_rope_prep(1, 1, 64, None, 0, None, 0, 0, 2, 1, 32, 32, 1, None, 1, 1e-5, 1, 16, 1.0, None, 0, None, 1, 2, None, None, None, 1, None, 32, 1.5, 0, 0, None) == 1   # weights with a norm behind the rotation
     with pytest.raises(RuntimeError):
         check(L.qsv_embed(0, 1, 1, 1, 1, 8, 0, None), "embed")
 
@@ -141,6 +153,6 @@ def test_serving_package_does_not_need_the_w4a8_library():
     the serving kernels."""
     import subprocess
     import sys
-    code = ("import sys; import qserve_amd.serving, qserve_amd.models.vekalorn, qserve_amd.models.mumelix, qserve_amd.models.vepolix, qserve_amd.models.pemolorn, qserve_amd.models.sagupel, qserve_amd.serving.trace; "
+    code = ("import sys; import qserve_amd.serving, qserve_amd.models.vekalorn, qserve_amd.models.mumelix, qserve_amd.models.vepolix, qserve_amd.models.pemolorn, qserve_amd.models.sagupel, qserve_amd.models.rivolix, qserve_amd.serving.trace; "
             "bad = [m for m in sys.modules if m in ('qserve_amd._lib', 'qserve_amd.decode', 'qserve_backend')]; sys.exit(1 if bad else 0)")
     assert subprocess.run([sys.executable, "-c", code], cwd=ROOT).returncode == 0
