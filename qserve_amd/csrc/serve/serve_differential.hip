@@ -7,6 +7,9 @@
 // Scores, maxima, sums, the outputs and their combination are float.
 #include "serve_common.h"
 
+#include <type_traits>
+#include <utility>
+
 namespace {
 constexpr int NT = 256;
 constexpr int NW = NT / 64;
@@ -284,7 +287,7 @@ __global__ __launch_bounds__(NT) void diff_attention_wave_kernel(T* __restrict__
 }
 // ---- matrix-core kernels (bfloat16): M key maps over the same values, dim = 16 DT, vdim = 32 CT ------------------------------------------
 // A wave owns 32 query rows = TQ tokens x HP head slots (one pool's heads, rounded up to a power of two; more than 32: head groups) and ALL
-// M maps of them, so that a value fragment read from LDS serves M products.  Keys come in blocks of 32 cache rows (inside one page), copied
+// M maps of them, so that a value fragment read from LDS serves M products.  Keys come in blocks of 32 cache rows (the prompt kernel: 64, inside one page), copied
 // straight into LDS (global_load_lds) as they lie in memory, 16-byte pieces of a row permuted by the row's number so that neither the
 // key reads (16 bytes per lane, 32 rows) nor the transposing value reads (ds_read_b64_tr_b16, 4 rows) pile up on a bank.  S^T = K Q^T
 // (v_mfma_f32_32x32x16_bf16) leaves a lane 16 of the 32 scores of its own row; the softmax needs one exchange (lanes ^ 32), the weights
@@ -312,6 +315,7 @@ struct Shape {
     static constexpr int PPR = 4 * CT + 2 * M * DT;      // 16-byte pieces of a row
     static constexpr int BLOCK = BN * PPR * 16;          // bytes of a block
     static constexpr int XM = (PPR % 16 == 0 ? 16 : PPR % 8 == 0 ? 8 : PPR % 4 == 0 ? 4 : 2) - 1;
+    __device__ static __forceinline__ int swizzle(int row) { return (((row & 3) << 2) | ((row >> 2) & 3)) & XM; }
     static constexpr int BUFS = 8 * BLOCK <= 144 * 1024 ? 2 : 1;                     // step kernel: buffers per wave
     static constexpr int OROW = VDIM + 4;                // merge: floats per row
     static constexpr int MERGE = NW * M * 32 * OROW * 4, ML = NW * M * 32 * 2 * 4;   // bytes
@@ -331,6 +335,21 @@ struct MapsArgs {
     int table_stride, n_tiles, H, per, page_shift, HP, TQ, HG, Z;
     float lambda, out_scale, eps;
 };
+
+// x ^ N, kept out of the compiler's sight: it would hold every such address of the key loop in a register of its own and spill accumulators
+template <int N>
+__device__ __forceinline__ unsigned flip(unsigned x) {
+    if constexpr (N != 0) asm volatile("v_xor_b32 %0, %1, %0" : "+v"(x) : "n"(N));
+    return x;
+}
+template <int N, class F, int... I>
+__device__ __forceinline__ void each_of(F&& f, std::integer_sequence<int, I...>) {
+    (f(std::integral_constant<int, I>{}), ...);
+}
+template <int N, class F>
+__device__ __forceinline__ void each(F&& f) {            // f(0), .., f(N - 1) with compile-time arguments
+    each_of<N>(f, std::make_integer_sequence<int, N>{});
+}
 
 template <int DT, int CT, int M>
 struct Rows {                                            // the softmax state of a wave's 32 rows
@@ -356,18 +375,18 @@ struct Rows {                                            // the softmax state of
     __device__ __forceinline__ void block(const unsigned char* blk, int k0, int p_row, bool mask, int lane) {
         const int li = lane & 31, hi = lane >> 5;
         const unsigned char* krow = blk + li * (S::PPR * 16);
-        const int ksw = (((li & 3) << 2) | ((li >> 2) & 3)) & S::XM;
+        const unsigned kcol = (unsigned)((hi ^ S::swizzle(li)) * 16);
         unsigned pb[M][2][4];
-#pragma unroll
-        for (int f = 0; f < M; ++f) {
+        each<M>([&](auto fc) {
+            constexpr int f = decltype(fc)::value;
             v16f sc;
 #pragma unroll
             for (int r = 0; r < 16; ++r) sc[r] = 0.f;
-#pragma unroll
-            for (int s = 0; s < DT; ++s) {
-                const v4u a = *(const v4u*)(krow + ((4 * CT + 2 * DT * f + 2 * s + hi) ^ ksw) * 16);
+            each<DT>([&](auto st) {                                      // (piece 4 CT + 2 DT f + 2 s + hi of the row: an even number plus hi)
+                constexpr int s = decltype(st)::value;
+                const v4u a = *(const v4u*)(krow + flip<(4 * CT + 2 * DT * f + 2 * s) * 16>(kcol));
                 sc = __builtin_amdgcn_mfma_f32_32x32x16_bf16(__builtin_bit_cast(bf8, a), __builtin_bit_cast(bf8, qf[f][s]), sc, 0, 0, 0);
-            }
+            });
             // sc[r]: key k0 + (r & 3) + 8 (r >> 2) + 4 hi of this lane's row
             float mx = -INFINITY;
             if (mask) {
@@ -402,15 +421,14 @@ struct Rows {                                            // the softmax state of
 #pragma unroll
                     for (int r = 0; r < 16; ++r) o[f][c][r] *= alpha;
             }
-        }
+        });
         // k-slot (hi, e) of half g <-> key 16 g + 8 (e / 4) + 4 hi + e % 4: exactly the weights this lane holds
         const int ta = lane & 15, g1 = (lane >> 4) & 1;
         const unsigned char* vrow = blk + (4 * hi + (ta >> 2)) * (S::PPR * 16) + (ta & 1) * 8;
-        const int vsw0 = (((ta >> 2) << 2) | hi) & S::XM, vsw1 = (((ta >> 2) << 2) | 2 | hi) & S::XM;
-#pragma unroll
-        for (int c = 0; c < CT; ++c) {
-            const int ch = 4 * c + 2 * g1 + ((ta & 3) >> 1);
-            const int o0 = (ch ^ vsw0) * 16, o1 = (ch ^ vsw1) * 16;
+        const unsigned vcol = (unsigned)(((2 * g1 + ((ta & 3) >> 1)) ^ ((((ta >> 2) << 2) | hi) & S::XM)) * 16);
+        each<CT>([&](auto cc) {
+            constexpr int c = decltype(cc)::value;                       // (rows 8 further on: bit 1 of the swizzle turns)
+            const unsigned o0 = flip<64 * c>(vcol), o1 = flip<(64 * c) ^ ((2 & S::XM) * 16)>(vcol);
 #pragma unroll
             for (int g = 0; g < 2; ++g) {
                 const s4 t0 = __builtin_amdgcn_ds_read_tr16_b64_v4i16((lds_s4)(vrow + (16 * g) * (S::PPR * 16) + o0));
@@ -422,20 +440,32 @@ struct Rows {                                            // the softmax state of
                     o[f][c] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(v, __builtin_bit_cast(bf8, (v4u{pb[f][g][0], pb[f][g][1], pb[f][g][2], pb[f][g][3]})),
                                                                       o[f][c], 0, 0, 0);
             }
-        }
+        });
     }
 };
 
-// Copies of a block's 1 KiB pieces number first, first + step, .. (this wave's); rows past `left` repeat row `left`.  base, dst: wave-uniform.
-template <typename S>
-__device__ __forceinline__ void copy_block(const bf16_t* base, unsigned dst, int left, int first, int step, int lane) {
+// Copy ROWS cache rows that lie behind each other at `base` into LDS at `dst` with WAVES waves (this one is number w), 1 KiB per wave and
+// instruction: piece p = 64 (w + WAVES j) + lane, row p / PPR.  Rows past `left` repeat row `left`.  base, dst, w: wave-uniform.
+template <typename S, int ROWS, int WAVES>
+__device__ __forceinline__ void copy_rows(const bf16_t* base, unsigned dst, int left, int w, int lane) {
+    constexpr int N = ROWS * S::PPR / (64 * WAVES), PER = 64 * WAVES, RPI = PER / S::PPR;        // instructions; pieces, rows of one
+    static_assert(ROWS * S::PPR % (64 * WAVES) == 0, "");
+    auto piece = [&](unsigned off, const bf16_t* from, int j) {
+        asm volatile("s_mov_b32 m0, %2\n\ts_nop 0\n\tglobal_load_lds_dwordx4 %0, %1" ::"v"(off), "s"(from), "s"(dst + (w + WAVES * j) * 1024)
+                     : "memory");
+    };
+    auto offset = [&](int j) {
+        const int p = 64 * (w + WAVES * j) + lane, row = p / S::PPR, c = p - row * S::PPR;
+        return (unsigned)((min(row, left) * S::PPR + (c ^ S::swizzle(row))) * 16);
+    };
+    if (PER % S::PPR == 0 && RPI % 8 == 0 && left >= ROWS - 1) {
+        // every instruction advances by the same rows: one offset, the rows in the base, and (8 rows) a swizzle that alternates
+        const unsigned o0 = offset(0), o1 = o0 ^ (RPI % 16 ? (2 & S::XM) * 16 : 0);
 #pragma unroll
-    for (int i = 0; i < S::PPR / 2; ++i) {
-        if (step > 1 && (i - first) % step != 0) continue;               // (wave-uniform)
-        const int p = i * 64 + lane, row = p / S::PPR, c = p - row * S::PPR;
-        const int src = c ^ ((((row & 3) << 2) | ((row >> 2) & 3)) & S::XM);
-        const unsigned off = (unsigned)((min(row, left) * S::PPR + src) * 16);
-        asm volatile("s_mov_b32 m0, %2\n\ts_nop 0\n\tglobal_load_lds_dwordx4 %0, %1" ::"v"(off), "s"(base), "s"(dst + i * 1024) : "memory");
+        for (int j = 0; j < N; ++j) piece(j & 1 ? o1 : o0, base + (size_t)j * RPI * S::PPR * 8, j);
+    } else {
+#pragma unroll
+        for (int j = 0; j < N; ++j) piece(offset(j), base, j);
     }
 }
 
@@ -483,11 +513,8 @@ __global__ __launch_bounds__(NT, (Shape<DT, CT, M>::PROMPT_OCC)) void maps_promp
         return pool + (((size_t)page << a.page_shift) + (size_t)(k0 & ((1 << a.page_shift) - 1))) * (size_t)(8 * S::PPR);
     };
     auto copy_tile = [&](int tile, int buf) {
-#pragma unroll
-        for (int b = 0; b < 2; ++b) {
-            const int k0 = tile * 2 * BN + b * BN;
-            if (k0 <= p_last) copy_block<S>(base_of(k0), lds + (2 * buf + b) * S::BLOCK, p_last - k0, (w + 2 * b) & 3, 4, lane);
-        }
+        const int k0 = tile * 2 * BN;
+        copy_rows<S, 2 * BN, NW>(base_of(k0), lds + 2 * buf * S::BLOCK, p_last - k0, w, lane);
     };
     copy_tile(0, 0);
 #pragma unroll
@@ -608,8 +635,8 @@ __global__ __launch_bounds__(NT, (Shape<DT, CT, M>::STEP_OCC)) void maps_step_ke
     PageIds pages(bt, (p_last >> a.page_shift) + 1, lane);
     auto copy = [&](int tile, int buf) {
         const int k0 = tile * BN, page = pages.at(k0 >> a.page_shift, lane);
-        copy_block<S>(pool + (((size_t)page << a.page_shift) + (size_t)(k0 & ((1 << a.page_shift) - 1))) * (size_t)(8 * S::PPR), lds + buf * S::BLOCK,
-                      p_last - k0, 0, 1, lane);
+        copy_rows<S, BN, 1>(pool + (((size_t)page << a.page_shift) + (size_t)(k0 & ((1 << a.page_shift) - 1))) * (size_t)(8 * S::PPR), lds + buf * S::BLOCK,
+                            p_last - k0, 0, lane);
     };
     if (first < nT) copy(first, 0);
 #pragma unroll
@@ -741,9 +768,9 @@ int head_slots(int per) {
 #define QSV_MAPS_SHAPES(F) F(1, 1, 2) F(2, 1, 2) F(2, 2, 2) F(3, 3, 2) F(4, 2, 2) F(4, 4, 2) F(6, 3, 2) F(8, 4, 2) F(2, 1, 1) F(4, 2, 1) F(6, 3, 1) F(8, 4, 1)
 }  // namespace
 
-// 1 if the matrix-core kernels take these sizes (bfloat16 storage, pages a power of two from 32 on), else 0.
+// 1 if the matrix-core kernels take these sizes (bfloat16 storage, pages a power of two from 64 on), else 0.
 extern "C" int qsv_maps_attention_ok(int dim, int vdim, int maps, int page, int dtype) {
-    if (dtype != QSV_BF16 || page < BN || (page & (page - 1))) return 0;
+    if (dtype != QSV_BF16 || page < 2 * BN || (page & (page - 1))) return 0;
 #define QSV_MAPS_OK(DT, CT, M) \
     if (dim == 16 * DT && vdim == 32 * CT && maps == M) return 1;
     QSV_MAPS_SHAPES(QSV_MAPS_OK)

@@ -573,7 +573,7 @@ class HipOps:
         groups, n = G * self.L.qsv_maps_attention_head_groups(per), step.size(0)
         splits, po, pm = 1, None, None
         if n:                                                # few workgroups and long contexts: the keys are cut over several
-            splits = max(1, min(self.step_split_target // (n * groups), (batch.max_pos + 1) // 256, 32)) if key_splits is None else key_splits
+            splits = max(1, min(self.step_split_target // (n * groups), (batch.max_pos + 1) // 256, 64)) if key_splits is None else key_splits
         if splits > 1:
             po = torch.empty((splits, n, groups, 32, maps, vdim), dtype=torch.float32, device=q.device)
             pm = torch.empty((splits, n, groups, 32, maps, 2), dtype=torch.float32, device=q.device)

@@ -132,7 +132,7 @@ def test_serve_argument_validation_without_gpu():
     assert L.qsv_residual_conv(1, 1, 1, 3, None, 1, 1, 1, 2, 8, 0, None) == 1                                  # three taps without a history
     assert L.qsv_scaled_add_rms_norm(1, None, 1, 2.0, 1, 1e-5, 1, 3, 1, 1, 1, 2, 8, 0, None) == 1              # a convolution without its output
     assert L.qsv_rotate_qk(1, 1, 64, 2, 8, 8, 1, 10, 1, 2, 0, None) == 1                                       # 10 rotated dimensions of 8
-    assert [L.qsv_maps_attention_ok(*a) for a in ((32, 64, 2, 64, 0), (64, 128, 2, 64, 0), (64, 64, 1, 32, 0), (40, 64, 2, 64, 0), (64, 64, 1, 96, 0), (64, 64, 1, 64, 1),
+    assert [L.qsv_maps_attention_ok(*a) for a in ((32, 64, 2, 64, 0), (64, 128, 2, 64, 0), (64, 64, 1, 128, 0), (40, 64, 2, 64, 0), (64, 64, 1, 96, 0), (64, 64, 1, 64, 1),
                                                   (64, 64, 3, 64, 0))] == [1, 1, 1, 0, 0, 0, 0]
     assert [L.qsv_maps_attention_tile_tokens(h) for h in (1, 3, 4, 20, 40)] == [32, 8, 8, 1, 1]
     assert [L.qsv_maps_attention_head_groups(h) for h in (1, 32, 33, 65)] == [1, 1, 2, 3]
